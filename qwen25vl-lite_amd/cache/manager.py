@@ -63,7 +63,7 @@ class CacheManager:
         self.requests: Dict[object, RequestPages] = {}
         # A shared prefix is only valid where every group still holds all of its pages.
         self.prefix_cache: Optional[RadixPrefixCache] = None
-        if enable_prefix_cache and self.groups and all(g.need.window is None for g in self.groups):
+        if enable_prefix_cache and self.groups and all(g.need.window is None and g.need.chunk is None for g in self.groups):
             self.prefix_cache = RadixPrefixCache(self.pools, self.page_size, max_prefix_nodes)
 
     # ------------------------------------------------------------------ requests and slots
@@ -105,10 +105,7 @@ class CacheManager:
     # ------------------------------------------------------------------ pages
     def _first_needed_page(self, group: int, start: int) -> int:
         """The first page a query at sequence index ``start`` can still see."""
-        window = self.groups[group].need.window
-        if window is None:
-            return 0
-        return max(0, start - window + 1) // self.page_size
+        return self.groups[group].need.first_visible(start) // self.page_size
 
     def pages_missing(self, req_id, upto: int) -> List[int]:
         """Pages each group would have to hand out so that tokens ``[0, upto)`` have a place."""
@@ -138,7 +135,8 @@ class CacheManager:
     def commit(self, req_id, num_tokens: int) -> None:
         """Tokens ``[0, num_tokens)`` are now in the cache.  A windowed group gives back the
         pages no later token can see: the next query sits at index ``num_tokens`` and sees keys
-        from ``num_tokens - window + 1`` on, and the group's first ``keep_first`` keys."""
+        from ``num_tokens - window + 1`` on (in a chunked group: from its chunk's first position on), and
+        the group's first ``keep_first`` keys."""
         rp = self.requests[req_id]
         if num_tokens < rp.num_tokens:
             raise ValueError("a request's cached length cannot shrink")

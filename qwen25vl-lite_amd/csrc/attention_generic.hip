@@ -2,7 +2,11 @@
 // One wave per (token, query head).  It serves prompt portions and decoded tokens alike: a
 // token at sequence index p sees keys lo..p of its request, lo = max(0, p - window + 1) with
 // a window, else 0 (reference attention.py:336-402 for the mask, text.py:78 for the scale); with
-// a window it also sees the request's first `keep_first` keys, wherever the window stands.
+// a window it also sees the request's first `keep_first` keys, wherever the window stands.  With `chunk` it
+// sees the keys from its chunk's first position on (chunks of that many positions from the sequence's start).
+// With `turn` [N, vd/2, 2] (cosines and sines of each token's angles) the values in the cache are turned by their
+// own positions, and a head's output is turned back by its token's: pair m is channels m and m + vd/2, or
+// (`turn_pairs`) 2m and 2m + 1.
 // Values may have another width (vd) than keys (hd).  With `sinks` (one float32 per query head) the
 // softmax's denominator also holds exp(sink): a place that has no key and no value and is not scaled.
 // Keys are walked in blocks of 64 by absolute index, so a token's result does not depend on
@@ -16,12 +20,14 @@ __global__ void attn_generic_kernel(const T* __restrict__ q, const T* __restrict
                                     const int* __restrict__ block_table, int table_width,
                                     const int* __restrict__ token_req, const int* __restrict__ token_seqpos,
                                     T* __restrict__ out, int nh, int nkv, int hd, int vd, int ps, int window,
-                                    int keep_first, float scale, const float* __restrict__ sinks) {
+                                    int keep_first, int chunk, float scale, const float* __restrict__ sinks,
+                                    const float2* __restrict__ turn, int turn_pairs) {
   __shared__ float sq[ATTN_MAX_HD];
   const int n = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int r = token_req[n], p = token_seqpos[n];
   const int kvh = h / (nh / nkv);
-  const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+  int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+  if (chunk > 0) lo = max(lo, p - p % chunk);
   const int kept = keep_first < lo ? keep_first : lo;       // keys [0, kept) are seen besides [lo, p]
   const int skip_from = (kept + 63) / 64, skip_to = lo / 64;  // blocks of 64 keys with nothing to see
   const T* qr = q + ((size_t)n * nh + h) * hd;
@@ -79,6 +85,24 @@ __global__ void attn_generic_kernel(const T* __restrict__ q, const T* __restrict
   }
   T* o = out + ((size_t)n * nh + h) * vd;
   const float inv = 1.0f / l;
+  if (turn) {
+    __syncthreads();          // the query has been read for the last time: its place takes the output
+#pragma unroll
+    for (int i = 0; i < ATTN_MAX_HD / 64; ++i) {
+      const int d = lane + 64 * i;
+      if (d < vd) sq[d] = acc[i] * inv;
+    }
+    __syncthreads();
+    const int half = vd >> 1;
+    const float2* tn = turn + (size_t)n * half;
+    for (int d = lane; d < vd; d += 64) {
+      const bool first = turn_pairs ? !(d & 1) : d < half;
+      const float2 t = tn[turn_pairs ? d >> 1 : (first ? d : d - half)];
+      const float v = sq[d], w = sq[turn_pairs ? d ^ 1 : (first ? d + half : d - half)];
+      stf<T>(o + d, first ? v * t.x + w * t.y : v * t.x - w * t.y);
+    }
+    return;
+  }
 #pragma unroll
   for (int i = 0; i < ATTN_MAX_HD / 64; ++i) {
     const int d = lane + 64 * i;
@@ -88,23 +112,25 @@ __global__ void attn_generic_kernel(const T* __restrict__ q, const T* __restrict
 
 extern "C" int qvl_attn_generic(const void* q, const void* kc, const void* vc, const void* block_table,
                                 int table_width, const void* token_req, const void* token_seqpos, void* out, int N,
-                                int nh, int nkv, int hd, int vd, int ps, int window, int keep_first, float scale,
-                                const void* sinks, int dtype, hipStream_t stream) {
+                                int nh, int nkv, int hd, int vd, int ps, int window, int keep_first, int chunk,
+                                float scale, const void* sinks, const void* turn, int turn_pairs, int dtype,
+                                hipStream_t stream) {
   if (N <= 0) return QVL_OK;
-  if (nh <= 0 || nkv <= 0 || nh % nkv || hd <= 0 || vd <= 0 || ps <= 0 || table_width <= 0 || keep_first < 0)
+  if (nh <= 0 || nkv <= 0 || nh % nkv || hd <= 0 || vd <= 0 || ps <= 0 || table_width <= 0 || keep_first < 0 ||
+      chunk < 0 || (turn && vd % 2))
     return QVL_ERR_SHAPE;
   if (hd > ATTN_MAX_HD || vd > ATTN_MAX_HD || nh > 65535) return QVL_ERR_LIMIT;
   const dim3 grid(N, nh);
   if (dtype == 0)
     hipLaunchKernelGGL(attn_generic_kernel<float>, grid, dim3(64), 0, stream, (const float*)q, (const float*)kc,
                        (const float*)vc, (const int*)block_table, table_width, (const int*)token_req,
-                       (const int*)token_seqpos, (float*)out, nh, nkv, hd, vd, ps, window, keep_first, scale,
-                       (const float*)sinks);
+                       (const int*)token_seqpos, (float*)out, nh, nkv, hd, vd, ps, window, keep_first, chunk,
+                       scale, (const float*)sinks, (const float2*)turn, turn_pairs);
   else if (dtype == 1)
     hipLaunchKernelGGL(attn_generic_kernel<bf16_t>, grid, dim3(64), 0, stream, (const bf16_t*)q, (const bf16_t*)kc,
                        (const bf16_t*)vc, (const int*)block_table, table_width, (const int*)token_req,
-                       (const int*)token_seqpos, (bf16_t*)out, nh, nkv, hd, vd, ps, window, keep_first, scale,
-                       (const float*)sinks);
+                       (const int*)token_seqpos, (bf16_t*)out, nh, nkv, hd, vd, ps, window, keep_first, chunk,
+                       scale, (const float*)sinks, (const float2*)turn, turn_pairs);
   else
     return QVL_ERR_DTYPE;
   return qvl_launch_status();

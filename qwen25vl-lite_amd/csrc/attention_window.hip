@@ -1,6 +1,8 @@
 // Paged attention on the matrix cores for what the other matrix-core kernel does not take: a sliding
 // window that also keeps a request's first keys visible, values of another width than keys, and a softmax
-// whose denominator holds one more term per query head, exp(sink), with no key and no value behind it.
+// whose denominator holds one more term per query head, exp(sink), with no key and no value behind it; chunks
+// of positions in place of a window (a token sees the keys from its chunk's first position on); and values that lie
+// in the cache turned by their positions, so that a head's output is turned back by its token's (`turn`).
 // bfloat16 storage, float32 scores, softmax and sums.  Compiled per key size HD and value size VD.
 //
 // A column is a (token, query head of one key/value head's group) pair; a tile has 16 of them.  A
@@ -34,6 +36,7 @@ typedef float f32x4_t __attribute__((ext_vector_type(4)));
 
 #define KS ((HD + 31) / 32)   // 32-channel steps of the first product
 #define NT ((VD + 15) / 16)   // 16-channel tiles of the second
+#define TURN_BY_LDS (VD % 2 == 0 && VD % 32 != 0)   // turning values back needs other lanes' channels
 
 __device__ __forceinline__ bf16x8_t zero8() { return __builtin_bit_cast(bf16x8_t, uint4{0u, 0u, 0u, 0u}); }
 __device__ __forceinline__ bf16x8_t load8(const bf16_t* p) { return *reinterpret_cast<const bf16x8_t*>(p); }
@@ -53,6 +56,15 @@ struct WindowArgs {
   int nq, nkv, ps, window, keep_first;
   float scale;
   const float* sinks;     // [nq] float32, or null
+  int chunk;              // positions of a chunk, or 0
+  const float2* turn;     // [N, VD/2] cosine and sine of each token's angles, or null
+  int turn_pairs;         // pair m of the turn: channels m and m + VD/2 (0), or 2m and 2m + 1
+  // the first key a token at position p sees, kept first keys aside
+  __device__ __forceinline__ int first_key(int p) const {
+    int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    if (chunk > 0) lo = max(lo, p - p % chunk);
+    return lo;
+  }
 };
 
 // W: waves that share an entry's key blocks (1 or 4).  CT: column tiles of an entry, all carried by the
@@ -62,6 +74,7 @@ template <int W, int CT>
 __global__ __launch_bounds__(256) void attn_window_kernel(WindowArgs a) {
   __shared__ float s_m[3][CT][16], s_l[3][CT][16];
   __shared__ __attribute__((aligned(16))) float s_acc[W > 1 ? 3 : 1][W > 1 ? CT * NT : 1][64][4];
+  __shared__ float s_out[TURN_BY_LDS ? (W > 1 ? 1 : 4) : 1][TURN_BY_LDS ? 16 : 1][TURN_BY_LDS ? VD + 1 : 1];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lg = lane >> 4, r = lane & 15;
   const int entry = W == 1 ? blockIdx.x * 4 + wave : blockIdx.x;
   const int part = W == 1 ? 0 : wave;
@@ -84,7 +97,7 @@ __global__ __launch_bounds__(256) void attn_window_kernel(WindowArgs a) {
     head[c] = kvh * g + (col - i_col * g);
     const int p = ctx - qlen + (valid[c] ? i_col : 0);
     my_p[c] = valid[c] ? p : -1;
-    my_lo[c] = (a.window > 0 && p - a.window + 1 > 0) ? p - a.window + 1 : 0;
+    my_lo[c] = a.first_key(p);
     const bf16_t* qrow = a.q + ((size_t)token[c] * a.nq + head[c]) * HD;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
@@ -96,7 +109,7 @@ __global__ __launch_bounds__(256) void attn_window_kernel(WindowArgs a) {
   int i_last = ((ct0 + CT) * 16 - 1) / g;
   i_last = i_last < qlen - 1 ? i_last : qlen - 1;
   const int p_first = ctx - qlen + i_first, hi_tile = ctx - qlen + i_last;
-  const int lo_tile = (a.window > 0 && p_first - a.window + 1 > 0) ? p_first - a.window + 1 : 0;
+  const int lo_tile = a.first_key(p_first);
   const int kept_tile = a.window > 0 ? (a.keep_first < lo_tile ? a.keep_first : lo_tile) : 0;
   const int n_kept = (kept_tile + 31) / 32;
   const int b_start = lo_tile / 32 > n_kept ? lo_tile / 32 : n_kept;
@@ -236,6 +249,59 @@ __global__ __launch_bounds__(256) void attn_window_kernel(WindowArgs a) {
     }
     const float inv = 1.0f / l[c];
     bf16_t* o = a.out + ((size_t)token[c] * a.nq + head[c]) * VD;
+    if (a.turn) {
+      // channel ch of this lane's column meets its partner: in this lane's own registers where half a value is a
+      // whole number of 16-channel tiles (or pairs are neighbours), else in the wave's place in LDS
+      const float2* tn = a.turn + (size_t)token[c] * (VD / 2);
+      if (VD % 2 == 0 && a.turn_pairs) {
+#pragma unroll
+        for (int dt = 0; dt < NT; ++dt)
+#pragma unroll
+          for (int i = 0; i < 4; i += 2) {
+            const int ch = dt * 16 + 4 * lg + i;
+            const float2 t = tn[ch < VD ? ch >> 1 : 0];
+            const float v = acc[c][dt][i], w = acc[c][dt][i + 1];
+            acc[c][dt][i] = v * t.x + w * t.y;
+            acc[c][dt][i + 1] = w * t.x - v * t.y;
+          }
+      } else if (VD % 32 == 0) {
+#pragma unroll
+        for (int dt = 0; dt < NT / 2; ++dt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const float2 t = tn[dt * 16 + 4 * lg + i];
+            const float v = acc[c][dt][i], w = acc[c][dt + NT / 2][i];
+            acc[c][dt][i] = v * t.x + w * t.y;
+            acc[c][dt + NT / 2][i] = w * t.x - v * t.y;
+          }
+      } else if (TURN_BY_LDS) {
+        // the four lanes of a column write and read the column's own row: they are of one wave
+        float* mine = s_out[W > 1 ? 0 : wave][r];
+#pragma unroll
+        for (int dt = 0; dt < NT; ++dt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int ch = dt * 16 + 4 * lg + i;
+            if (ch < VD) mine[ch] = acc[c][dt][i];
+          }
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+        __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll
+        for (int dt = 0; dt < NT; ++dt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int ch = dt * 16 + 4 * lg + i;
+            if (ch < VD) {
+              const bool first = ch < VD / 2;
+              const float2 t = tn[first ? ch : ch - VD / 2];
+              const float w = mine[first ? ch + VD / 2 : ch - VD / 2];
+              acc[c][dt][i] = first ? acc[c][dt][i] * t.x + w * t.y : acc[c][dt][i] * t.x - w * t.y;
+            }
+          }
+        __builtin_amdgcn_wave_barrier();
+      }
+    }
 #pragma unroll
     for (int dt = 0; dt < NT; ++dt)
 #pragma unroll
@@ -264,10 +330,12 @@ extern "C" int qvl_attn_window_sizes(int* hd, int* vd) {
 // entry of qvl_attn_window_entry_tiles() column tiles (tile_ct counts in such entries).
 extern "C" int qvl_attn_window(const void* q, const void* kc, const void* vc, const void* bt, int table_width,
                                const void* cu_q, const void* ctx_len, const void* tile_req, const void* tile_ct,
-                               int num_tiles, void* out, int nq, int nkv, int ps, int window, int keep_first, float scale,
-                               const void* sinks, int share, hipStream_t stream) {
+                               int num_tiles, void* out, int nq, int nkv, int ps, int window, int keep_first, int chunk,
+                               float scale, const void* sinks, const void* turn, int turn_pairs, int share,
+                               hipStream_t stream) {
   if (num_tiles <= 0) return QVL_OK;
-  if (nq <= 0 || nkv <= 0 || nq % nkv || ps <= 0 || ps % 8 || table_width <= 0 || window < 0 || keep_first < 0)
+  if (nq <= 0 || nkv <= 0 || nq % nkv || ps <= 0 || ps % 8 || table_width <= 0 || window < 0 || keep_first < 0 ||
+      chunk < 0 || (turn && VD % 2))
     return QVL_ERR_SHAPE;
   if ((tile_req == nullptr) != (tile_ct == nullptr) || (!tile_req && (nq / nkv > 16 || !share))) return QVL_ERR_SHAPE;
   if (nkv > 65535) return QVL_ERR_LIMIT;
@@ -277,6 +345,7 @@ extern "C" int qvl_attn_window(const void* q, const void* kc, const void* vc, co
   a.tile_req = (const int*)tile_req; a.tile_ct = (const int*)tile_ct; a.num_tiles = num_tiles; a.out = (bf16_t*)out;
   a.nq = nq; a.nkv = nkv; a.ps = ps; a.window = window; a.keep_first = keep_first; a.scale = scale;
   a.sinks = (const float*)sinks;
+  a.chunk = chunk; a.turn = (const float2*)turn; a.turn_pairs = turn_pairs;
   if (share) hipLaunchKernelGGL((attn_window_kernel<4, 1>), dim3(num_tiles, nkv), dim3(256), 0, stream, a);
   else hipLaunchKernelGGL((attn_window_kernel<1, WIDE_CT>), dim3((num_tiles + 3) / 4, nkv), dim3(256), 0, stream, a);
   return qvl_launch_status();

@@ -43,6 +43,13 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// The activation of a gated feed-forward: silu, or the tanh form of gelu, 0.5 z (1 + tanh(y)) with
+// y = sqrt(2/pi) (z + 0.044715 z^3), written as z sigmoid(2 y).
+__device__ __forceinline__ float gate_act(float z, int gelu) {
+  const float y = gelu ? 1.5957691216057308f * (z + 0.044715f * z * z * z) : z;
+  return z / (1.0f + expf(-y));
+}
+
 // Sum over a block of up to 1024 threads; every thread gets the total.  `red` holds 17 floats.
 __device__ __forceinline__ float block_sum(float v, float* red) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nwaves = (blockDim.x + 63) >> 6;

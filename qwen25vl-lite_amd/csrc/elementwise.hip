@@ -436,13 +436,14 @@ extern "C" int qvl_rope_table(const void* pos, int pos_stride, const void* inv_f
 }
 
 // ---------------------------------------------------------------------------------------
-// SwiGLU: out[n, i] = silu(gate[n, i]) * up[n, i],  silu(z) = z / (1 + exp(-z))  (reference text.py:66)
+// SwiGLU: out[n, i] = silu(gate[n, i]) * up[n, i],  silu(z) = z / (1 + exp(-z))  (reference text.py:66);
+// with `gelu` the activation is the tanh form of gelu.
 // x[n] holds gate and up: plain, gate in columns 0..I-1 and up in I..2I-1; grouped, alternating
 // groups of 8 gate columns and 8 up columns (feature i: gate at 16 (i/8) + i%8, up 8 further),
 // the layout that lets the product before it apply the activation to a 16-row tile by itself.
 // ---------------------------------------------------------------------------------------
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ x, T* __restrict__ out, int I, int grouped) {
+__global__ void swiglu_kernel(const T* __restrict__ x, T* __restrict__ out, int I, int grouped, int gelu) {
   const int n = blockIdx.y;
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= I) return;
@@ -450,12 +451,12 @@ __global__ void swiglu_kernel(const T* __restrict__ x, T* __restrict__ out, int 
   const int gc = grouped ? 16 * (i >> 3) + (i & 7) : i;
   const int uc = grouped ? gc + 8 : I + i;
   const float g = ldf<T>(row + gc), u = ldf<T>(row + uc);
-  stf<T>(out + (size_t)n * I + i, (g / (1.0f + expf(-g))) * u);
+  stf<T>(out + (size_t)n * I + i, gate_act(g, gelu) * u);
 }
 
 // bfloat16 rows whose width is a multiple of 8: eight values per thread, 16-byte loads and stores.
 __global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __restrict__ x, bf16_t* __restrict__ out,
-                                                            int I, long long total8, int grouped) {
+                                                            int I, long long total8, int grouped, int gelu) {
   typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
   const int per_row = I >> 3;
   for (long long idx = (long long)blockIdx.x * blockDim.x + threadIdx.x; idx < total8;
@@ -470,29 +471,29 @@ __global__ __launch_bounds__(256) void swiglu_bf16x8_kernel(const bf16_t* __rest
     for (int k = 0; k < 4; ++k) {
       const float g0 = __uint_as_float(gv[k] << 16), g1 = __uint_as_float(gv[k] & 0xffff0000u);
       const float u0 = __uint_as_float(uv[k] << 16), u1 = __uint_as_float(uv[k] & 0xffff0000u);
-      const float a0 = (g0 / (1.0f + expf(-g0))) * u0, a1 = (g1 / (1.0f + expf(-g1))) * u1;
+      const float a0 = gate_act(g0, gelu) * u0, a1 = gate_act(g1, gelu) * u1;
       o[k] = (uint32_t)f32_to_bf16(a0) | ((uint32_t)f32_to_bf16(a1) << 16);
     }
     *reinterpret_cast<u32x4*>(out + (size_t)n * I + c) = o;
   }
 }
 
-extern "C" int qvl_swiglu(const void* x, void* out, int N, int I, int dtype, int grouped, hipStream_t stream) {
+extern "C" int qvl_swiglu(const void* x, void* out, int N, int I, int dtype, int grouped, int gelu, hipStream_t stream) {
   if (N <= 0) return QVL_OK;
   if (I <= 0 || (grouped && I % 8)) return QVL_ERR_SHAPE;
   if (N > 65535) return QVL_ERR_LIMIT;
   const dim3 grid((I + 255) / 256, N);
   if (dtype == 0)
-    hipLaunchKernelGGL(swiglu_kernel<float>, grid, dim3(256), 0, stream, (const float*)x, (float*)out, I, grouped);
+    hipLaunchKernelGGL(swiglu_kernel<float>, grid, dim3(256), 0, stream, (const float*)x, (float*)out, I, grouped, gelu);
   else if (dtype == 1 && I % 8 == 0 && (((uintptr_t)x | (uintptr_t)out) & 15) == 0) {
     const long long total8 = (long long)N * (I >> 3);
     long long blocks = (total8 + 255) / 256;
     blocks = blocks > 8192 ? 8192 : blocks;
     hipLaunchKernelGGL(swiglu_bf16x8_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, (const bf16_t*)x,
-                       (bf16_t*)out, I, total8, grouped);
+                       (bf16_t*)out, I, total8, grouped, gelu);
   } else if (dtype == 1)
     hipLaunchKernelGGL(swiglu_kernel<bf16_t>, grid, dim3(256), 0, stream, (const bf16_t*)x, (bf16_t*)out, I,
-                       grouped);
+                       grouped, gelu);
   else
     return QVL_ERR_DTYPE;
   return qvl_launch_status();

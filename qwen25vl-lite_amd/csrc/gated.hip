@@ -132,20 +132,43 @@ extern "C" int qvl_gated_act(const void* x, void* out, int N, int I, int dtype, 
 }
 
 // ---------------------------------------------------------------------------------------
-// logits = cap * tanh(logits / cap), in place, float32
+// logits = scale * logits, then, with a cap above zero, cap * tanh(logits / cap); in place, float32
 // ---------------------------------------------------------------------------------------
-__global__ void softcap_kernel(float* __restrict__ x, long long total, float cap) {
+__global__ void softcap_kernel(float* __restrict__ x, long long total, float scale, float cap) {
   const long long step = (long long)gridDim.x * blockDim.x;
-  const float inv = 1.0f / cap;
-  for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += step)
-    x[i] = cap * tanhf(x[i] * inv);
+  const float inv = cap > 0.f ? 1.0f / cap : 0.f;
+  for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += step) {
+    const float v = scale * x[i];
+    x[i] = cap > 0.f ? cap * tanhf(v * inv) : v;
+  }
 }
 
-extern "C" int qvl_softcap(void* x, long long total, float cap, hipStream_t stream) {
+extern "C" int qvl_softcap(void* x, long long total, float scale, float cap, hipStream_t stream) {
   if (total <= 0) return QVL_OK;
-  if (!(cap > 0.f)) return QVL_ERR_SHAPE;
+  if (cap < 0.f) return QVL_ERR_SHAPE;
   const int blocks = (int)((total + 255) / 256 > 4096 ? 4096 : (total + 255) / 256);
-  hipLaunchKernelGGL(softcap_kernel, dim3(blocks), dim3(256), 0, stream, (float*)x, total, cap);
+  hipLaunchKernelGGL(softcap_kernel, dim3(blocks), dim3(256), 0, stream, (float*)x, total, scale, cap);
+  return qvl_launch_status();
+}
+
+// ---------------------------------------------------------------------------------------
+// out = tanh(x), float32 in, float32 or bfloat16 out
+// ---------------------------------------------------------------------------------------
+template <typename TO>
+__global__ __launch_bounds__(256) void tanh_kernel(const float* __restrict__ x, TO* __restrict__ out, long long total) {
+  const long long step = (long long)gridDim.x * blockDim.x;
+  for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += step) stf<TO>(out + i, tanhf(x[i]));
+}
+
+extern "C" int qvl_tanh(const void* x, void* out, long long total, int out_dtype, hipStream_t stream) {
+  if (total <= 0) return QVL_OK;
+  const int blocks = (int)((total + 255) / 256 > 4096 ? 4096 : (total + 255) / 256);
+  if (out_dtype == 0)
+    hipLaunchKernelGGL(tanh_kernel<float>, dim3(blocks), dim3(256), 0, stream, (const float*)x, (float*)out, total);
+  else if (out_dtype == 1)
+    hipLaunchKernelGGL(tanh_kernel<bf16_t>, dim3(blocks), dim3(256), 0, stream, (const float*)x, (bf16_t*)out, total);
+  else
+    return QVL_ERR_DTYPE;
   return qvl_launch_status();
 }
 
@@ -329,6 +352,8 @@ extern "C" int qvl_head_gate(void* o, const void* gate, long long gate_stride, i
 //   come in `row_rs` [N, 2] (row_inv_rms below forms them) and the weights span all heads' columns.
 //   Queries go to q_out [N, nq hd]; keys into k_cache [pages, nkv, ps, hd] at slots[n]; values
 //   (the key head before norm and rotation, or the value head) into v_cache [pages, nkv, vd, ps].
+//   `vcs` [N, vd/2, 2] (or null): value heads are turned by these angles over all their channels, channel c with
+//   c + vd/2 (`interleaved`: 2f with 2f + 1), before they are written.
 // One wave per (token, head); a block holds 4 of them.  hd, vd <= 512.
 // ---------------------------------------------------------------------------------------
 #define QKN_MAX_HD 512
@@ -338,7 +363,8 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
     const float* __restrict__ x, long long x_stride, const float* __restrict__ bias, const float* __restrict__ qw,
     const float* __restrict__ kw, const float2* __restrict__ cs, const int* __restrict__ slots, T* __restrict__ q_out,
     T* __restrict__ k_cache, T* __restrict__ v_cache, int N, int nq, int nkv, int hd, int vd, int rot_half, int ps,
-    float eps, int interleaved, int v_from_k, int write_kv, int norm_mode, const float* __restrict__ row_rs) {
+    float eps, int interleaved, int v_from_k, int write_kv, int norm_mode, const float* __restrict__ row_rs,
+    const float2* __restrict__ vcs) {
   __shared__ float buf[4][QKN_MAX_HD];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int heads = nq + (write_kv ? (v_from_k ? nkv : 2 * nkv) : 0);
@@ -357,7 +383,19 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
   if (kind == 2) {
     const int kvh = head - nq - nkv;
     T* vrow = v_cache + ((page * nkv + kvh) * vd) * (size_t)ps + in_page;
-    for (int c = lane; c < vd; c += 64) stf<T>(vrow + (size_t)c * ps, a[c] + (b ? b[c] : 0.f));
+    for (int c = lane; c < vd; c += 64) {
+      float v = a[c] + (b ? b[c] : 0.f);
+      if (vcs) {
+        const int half = vd >> 1;
+        const int f = interleaved ? c >> 1 : (c < half ? c : c - half);
+        const bool first = interleaved ? !(c & 1) : c < half;
+        const int partner = interleaved ? c ^ 1 : (first ? c + half : c - half);
+        const float2 t = vcs[(size_t)n * half + f];
+        const float p = a[partner] + (b ? b[partner] : 0.f);
+        v = first ? v * t.x - p * t.y : v * t.x + p * t.y;
+      }
+      stf<T>(vrow + (size_t)c * ps, v);
+    }
     return;
   }
   float ss = 0.f;
@@ -421,11 +459,12 @@ extern "C" int qvl_qk_norm_rope_write(const void* x, long long x_stride, const v
                                       const void* kw, const void* cs, const void* slots, void* q_out, void* k_cache,
                                       void* v_cache, int N, int nq, int nkv, int hd, int vd, int rot_half, int ps,
                                       float eps, int interleaved, int v_from_k, int write_kv, int norm_mode,
-                                      const void* row_rs, int dtype, hipStream_t stream) {
+                                      const void* row_rs, const void* vcs, int dtype, hipStream_t stream) {
   if (N <= 0) return QVL_OK;
   if (nq <= 0 || nkv < 0 || hd <= 0 || vd <= 0 || rot_half < 0 || 2 * rot_half > hd || ps <= 0) return QVL_ERR_SHAPE;
   if (write_kv && (!slots || !k_cache || !v_cache || nkv <= 0)) return QVL_ERR_SHAPE;
   if (norm_mode < 0 || norm_mode > 3 || (norm_mode == 3 && !row_rs) || (v_from_k && vd != hd)) return QVL_ERR_SHAPE;
+  if (vcs && (v_from_k || vd % 2)) return QVL_ERR_SHAPE;
   if (hd > QKN_MAX_HD || vd > QKN_MAX_HD) return QVL_ERR_LIMIT;
   const int heads = nq + (write_kv ? (v_from_k ? nkv : 2 * nkv) : 0);
   const long long items = (long long)N * heads;
@@ -434,7 +473,7 @@ extern "C" int qvl_qk_norm_rope_write(const void* x, long long x_stride, const v
   hipLaunchKernelGGL(qk_norm_rope_write_kernel<T>, dim3(blocks), dim3(256), 0, stream, (const float*)x, x_stride,   \
                      (const float*)bias, (const float*)qw, (const float*)kw, (const float2*)cs, (const int*)slots, \
                      (T*)q_out, (T*)k_cache, (T*)v_cache, N, nq, nkv, hd, vd, rot_half, ps, eps, interleaved,      \
-                     v_from_k, write_kv, norm_mode, (const float*)row_rs)
+                     v_from_k, write_kv, norm_mode, (const float*)row_rs, (const float2*)vcs)
   if (dtype == 0) LAUNCH(float);
   else if (dtype == 1) LAUNCH(bf16_t);
   else return QVL_ERR_DTYPE;

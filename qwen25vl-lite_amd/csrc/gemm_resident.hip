@@ -36,7 +36,7 @@
 //                           each wave sums its own 256 columns, the block adds the waves in order)
 //   epilogue  EPI_RESIDUAL  out += product, out being the float32 residual
 //             EPI_SWIGLU    W's rows come in groups of 8 gate rows, 8 up rows; out[M, N/2] =
-//                           silu(gate) * up, in bfloat16
+//                           act(gate) * up, in bfloat16 (act: silu, or the tanh form of gelu)
 //             EPI_ROPE      W is the stacked query | key | value projection.  A tile of a query or
 //                           key head takes 8 channels and the 8 channels they are rotated with
 //                           (half a head further), so the rotation happens here; queries are
@@ -122,6 +122,7 @@ struct ResidentArgs {
   // is cut into `parts` tiles of `pairs` gate rows and their up rows, so that the last round of
   // tiles is as even as the rounds before it
   int whole_tiles, parts, pairs;
+  int gelu;              // EPI_SWIGLU: the activation is the tanh form of gelu
 #ifdef QVL_TIMELINE
   unsigned long long* timeline;
 #endif
@@ -332,7 +333,7 @@ __global__ __launch_bounds__(64 * RW) void gemm_resident_kernel(ResidentArgs p) 
         const float up = __shfl_down(sum, 8, QVL_WAVE);  // rows 8..15 of the tile are the up rows
         if (nl < 8 && m < p.M && n >= 0 && n < p.N) {
           bf16_t* o = reinterpret_cast<bf16_t*>(p.out);
-          o[(size_t)m * p.ldo + (n >> 4) * 8 + (n & 7)] = f32_to_bf16((sum / (1.0f + expf(-sum))) * up);
+          o[(size_t)m * p.ldo + (n >> 4) * 8 + (n & 7)] = f32_to_bf16(gate_act(sum, p.gelu) * up);
         }
       } else if (EPI == EPI_ROPE) {
         sum += epi.bias;
@@ -560,12 +561,14 @@ extern "C" int qvl_gemm_resident_two_tile_k() { return 32 * XHI_STEPS; }
 
 // x: bfloat16 [M, K] (h null), or h: float32 [M, K] with norm_w [K] and eps (x null): X = rmsnorm(h) * norm_w.
 // epilogue 0: out[M, N] in out_dtype (0 float32, 1 bfloat16); 1: out (float32 [M, N]) += product;
-// 2: out[M, N/2] bfloat16 = silu(gate) * up for W rows in groups of 8 gate, 8 up.
+// 2: out[M, N/2] bfloat16 = silu(gate) * up for W rows in groups of 8 gate, 8 up; 4: the same with gelu's tanh form.
 // max_blocks: blocks to launch at most (the number of compute units).
 extern "C" int qvl_gemm_resident(const void* x, int ldx, const void* h, int ldh, const void* norm_w, float eps,
                                  const void* W, int ldw, const void* bias, void* out, int ldo, int M, int N, int K,
                                  int out_dtype, int epilogue, int max_blocks, hipStream_t stream) {
   if (M <= 0 || N <= 0) return QVL_OK;
+  const int gelu = epilogue == 4;
+  if (gelu) epilogue = EPI_SWIGLU;
   if (M > 64) return QVL_ERR_LIMIT;
   if (M > 32 && K > PASS_K) return QVL_ERR_LIMIT;   // teams of more than two keep their rows for a single pass
   if (K <= 0 || K % 8 || ldw % 8 || ldw < K || max_blocks <= 0 || !W || !out) return QVL_ERR_SHAPE;
@@ -587,7 +590,7 @@ extern "C" int qvl_gemm_resident(const void* x, int ldx, const void* h, int ldh,
   ResidentArgs p;
   p.X = (const bf16_t*)x; p.ldx = ldx; p.H = (const float*)h; p.ldh = ldh; p.norm_w = (const float*)norm_w;
   p.eps = eps; p.W = (const bf16_t*)W; p.ldw = ldw; p.bias = (const float*)bias; p.out = out; p.ldo = ldo;
-  p.M = M; p.N = N; p.K = K;
+  p.M = M; p.N = N; p.K = K; p.gelu = gelu;
 #ifdef QVL_TIMELINE
   p.timeline = timeline_buffer;
 #endif
@@ -652,7 +655,7 @@ extern "C" int qvl_gemm_resident_rope(const void* x, int ldx, const void* h, int
   ResidentArgs p;
   p.X = (const bf16_t*)x; p.ldx = ldx; p.H = (const float*)h; p.ldh = ldh; p.norm_w = (const float*)norm_w;
   p.eps = eps; p.W = (const bf16_t*)W; p.ldw = ldw; p.bias = (const float*)bias; p.out = nullptr; p.ldo = 0;
-  p.M = M; p.N = (nq + 2 * nkv) * hd; p.K = K;
+  p.M = M; p.N = (nq + 2 * nkv) * hd; p.K = K; p.gelu = 0;
 #ifdef QVL_TIMELINE
   p.timeline = timeline_buffer;
 #endif

@@ -4,6 +4,7 @@ norm and the output head (reference src/qwen25vl_lite/text.py:209-279, model.py:
 
 from __future__ import annotations
 
+from dataclasses import replace
 from typing import Dict, List, Optional, Tuple
 
 import torch
@@ -29,14 +30,13 @@ def _prefix_of(name: str) -> str:
 
 
 def _mixers_of(block: Part, prefix: str = "") -> List[Tuple[str, Part]]:
-    """Every mixer inside a block, however deep, and every other part that keeps a cache or a per-request
-    state (a short convolution), with its dotted sub-part name."""
+    """Every mixer inside a block, however deep (a mixer's own sub-parts too), and every other part that
+    keeps a cache or a per-request state (a short convolution), with its dotted sub-part name."""
     found: List[Tuple[str, Part]] = []
     for name, sub in block.sub_parts().items():
         if isinstance(sub, Mixer) or sub.state_need() is not None or sub.cache_need() is not None:
             found.append((prefix + name, sub))
-        else:
-            found.extend(_mixers_of(sub, f"{prefix}{name}."))
+        found.extend(_mixers_of(sub, f"{prefix}{name}."))
     return found
 
 
@@ -185,6 +185,14 @@ class DecoderModel:
                 self.entry_writes.append(True)
                 self.group_layers[g] += 1
             self.entry_places.append(places)
+        # the embedding's place, behind all others, if it keeps a state per request
+        self.embed_place: Optional[int] = None
+        if self.embedding.state_need() is not None:
+            self.embed_place = len(self.entry_state)
+            self.entry_state.append(self.embedding.state_need())
+            self.entry_group.append(None)
+            self.entry_cache_layer.append(None)
+            self.entry_writes.append(False)
 
         self.params: Dict[str, Tuple[Optional[Part], str, ParamSpec]] = {}
         _collect(self.embedding, _prefix_of(spec.embed_name), self.params)
@@ -243,9 +251,10 @@ class DecoderModel:
         return getattr(self.head_part, "weight", None)
 
     def make_slots(self, storage, state_tensors: List[Optional[torch.Tensor]]) -> List[LayerSlot]:
-        """One slot per run entry.  ``state_tensors`` has one element per place (see
-        ``entry_state``).  The slot of an entry is its first mixer's; a block with several
-        mixers finds each one's under the mixer's sub-part name in ``slot.by_part``."""
+        """One slot per run entry, and one more at the end for an embedding that keeps a state.
+        ``state_tensors`` has one element per place (see ``entry_state``).  The slot of an entry stands for
+        its first mixer's; a block with several mixers finds each one's under the mixer's dotted sub-part
+        name in ``slot.by_part``, and a mixer made of mixers finds its own sub-parts' in its slot."""
         def place_slot(p: int) -> LayerSlot:
             g, layer = self.entry_group[p], self.entry_cache_layer[p]
             return LayerSlot(
@@ -259,9 +268,11 @@ class DecoderModel:
         slots = []
         for places in self.entry_places:
             by_part = {name: place_slot(p) for name, p in places.items()}
-            first = next(iter(by_part.values()), LayerSlot(writes=False))
-            first.by_part = by_part
-            slots.append(first)
+            for name, slot in by_part.items():
+                slot.by_part = {sub[len(name) + 1:]: s for sub, s in by_part.items() if sub.startswith(name + ".")}
+            slots.append(replace(next(iter(by_part.values()), LayerSlot(writes=False)), by_part=by_part))
+        if self.embed_place is not None:
+            slots.append(place_slot(self.embed_place))
         return slots
 
     # ------------------------------------------------------------------ the step
@@ -270,7 +281,10 @@ class DecoderModel:
         ``step.logit_rows``."""
         if not self._has_weights:
             raise RuntimeError("the model has no weights yet")
-        stream = ResidualStream(self.embedding.forward(step.token_ids, step))
+        if self.embed_place is not None:
+            stream = ResidualStream(self.embedding.forward(step.token_ids, step, slots[len(self.spec.run)]))
+        else:
+            stream = ResidualStream(self.embedding.forward(step.token_ids, step))
         first_share = None
         if self.pass_mix is not None and any(e.mix_input for e in self.spec.run):
             first_share = self.pass_mix.from_first(stream.h)     # before any layer changes the sum in place

@@ -14,7 +14,7 @@ import torch
 from .kernels import _check, _dev, _fn, _need, _ptr, _stream, dtype_code
 
 __all__ = ["residual_add", "gated_act", "softcap_", "group_norm_gate", "head_gate_", "qk_norm_rope_write", "sandwich_norm",
-           "row_inv_rms"]
+           "row_inv_rms", "tanh_to"]
 
 _c_int, _c_float, _c_ptr, _c_ll = ctypes.c_int, ctypes.c_float, ctypes.c_void_p, ctypes.c_longlong
 GATE_ACTS = {None: 0, "sigmoid": 1, "silu": 2}
@@ -51,13 +51,24 @@ def gated_act(x: torch.Tensor, alpha: float = 1.0, limit: Optional[float] = None
     return out
 
 
-def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
-    """``x = cap * tanh(x / cap)`` in place on float32."""
+def softcap_(x: torch.Tensor, cap: Optional[float], scale: float = 1.0) -> torch.Tensor:
+    """``x = scale * x``, then, unless ``cap`` is None, ``x = cap * tanh(x / cap)``, in place on float32."""
+    _need(cap is None or cap > 0, "a soft cap must be positive")
     _dev(x)
     _need(x.dtype == torch.float32 and x.is_contiguous(), "x must be contiguous float32")
-    fn = _fn("gated", "qvl_softcap", [_c_ptr, _c_ll, _c_float, _c_ptr])
-    _check(fn(_ptr(x), x.numel(), float(cap), _stream()), "softcap")
+    fn = _fn("gated", "qvl_softcap", [_c_ptr, _c_ll, _c_float, _c_float, _c_ptr])
+    _check(fn(_ptr(x), x.numel(), float(scale), float(cap or 0.0), _stream()), "softcap")
     return x
+
+
+def tanh_to(x: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """``tanh(x)`` of float32 ``x`` in ``out_dtype``."""
+    _dev(x)
+    _need(x.dtype == torch.float32 and x.is_contiguous(), "x must be contiguous float32")
+    out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+    fn = _fn("gated", "qvl_tanh", [_c_ptr, _c_ptr, _c_ll, _c_int, _c_ptr])
+    _check(fn(_ptr(x), _ptr(out), x.numel(), dtype_code(out_dtype), _stream()), "tanh")
+    return out
 
 
 def group_norm_gate(x: torch.Tensor, weight: torch.Tensor, span: int, eps: float, out_dtype: torch.dtype,
@@ -122,7 +133,7 @@ def qk_norm_rope_write(x: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: 
                        v_cache: Optional[torch.Tensor], num_q_heads: int, num_kv_heads: int, head_dim: int,
                        page_size: int, out_dtype: torch.dtype, *, interleaved: bool, values_are_keys: bool,
                        norm: Optional[str] = "before", bias: Optional[torch.Tensor] = None,
-                       value_dim: Optional[int] = None) -> torch.Tensor:
+                       value_dim: Optional[int] = None, value_cs: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per head: ``bias`` (float32 over all columns, or None) is added; RMS norm over the head
     (``norm`` ``"before"`` or ``"after"`` the rotation, None: no norm; weights ``q_norm`` / ``k_norm``
     of ``[head_dim]``, None: a gain of one; ``norm`` ``"whole"``: before the rotation and over all query heads of a
@@ -131,8 +142,9 @@ def qk_norm_rope_write(x: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: 
     queries are returned; rotated keys and the values go into the page slots (``slots`` None:
     queries only).  ``x`` is float32 ``[N, >= nq hd + nkv hd (+ nkv vd)]``: query heads, key heads, and value
     heads of ``value_dim`` channels unless ``values_are_keys``, in which case a key head as projected
-    (before norm and rotation) is its own value."""
-    _dev(x, q_norm, k_norm, cs, slots, k_cache, v_cache, bias)
+    (before norm and rotation) is its own value.  ``value_cs`` (``[N, vd/2, 2]``): value heads are turned by these
+    angles over all their channels, in the same layout of pairs, before they are written."""
+    _dev(x, q_norm, k_norm, cs, slots, k_cache, v_cache, bias, value_cs)
     nq, nkv, hd = int(num_q_heads), int(num_kv_heads), int(head_dim)
     vd = hd if value_dim is None else int(value_dim)
     write = slots is not None
@@ -154,6 +166,9 @@ def qk_norm_rope_write(x: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: 
                            and bias.is_contiguous()), "the bias must be float32 over the heads' columns")
     _need(cs.dtype == torch.float32 and cs.dim() == 3 and cs.is_contiguous() and cs.shape[0] >= n
           and cs.shape[2] == 2 and 2 * cs.shape[1] <= hd, "cs must be float32 [N, rot/2, 2] with rot <= head_dim")
+    _need(value_cs is None or (value_cs.dtype == torch.float32 and value_cs.dim() == 3 and value_cs.is_contiguous()
+                               and value_cs.shape[0] >= n and tuple(value_cs.shape[1:]) == (vd // 2, 2) and vd % 2 == 0
+                               and not values_are_keys), "value_cs must be float32 [N, vd/2, 2], for values of their own")
     if write:
         _need(slots.dtype == torch.int32 and slots.shape == (n,) and slots.is_contiguous(), "slots must be int32 [N]")
         _need(k_cache is not None and v_cache is not None and k_cache.dtype == v_cache.dtype == out_dtype,
@@ -165,11 +180,12 @@ def qk_norm_rope_write(x: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: 
     q_out = torch.empty((n, nq * hd), dtype=out_dtype, device=x.device)
     fn = _fn("gated", "qvl_qk_norm_rope_write",
              [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
-              _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_ptr])
+              _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr])
     _check(fn(_ptr(x), x.stride(0), _ptr(bias), _ptr(q_norm), _ptr(k_norm), _ptr(cs), _ptr(slots), _ptr(q_out),
               _ptr(k_cache) if write else None, _ptr(v_cache) if write else None, n, nq, nkv, hd, vd, cs.shape[1],
               int(page_size), float(eps), int(interleaved), int(values_are_keys), int(write),
-              {None: 0, "before": 1, "after": 2, "whole": 3}[norm], _ptr(row_rs), dtype_code(out_dtype), _stream()),
+              {None: 0, "before": 1, "after": 2, "whole": 3}[norm], _ptr(row_rs), _ptr(value_cs), dtype_code(out_dtype),
+              _stream()),
            "qk_norm_rope_write")
     return q_out
 

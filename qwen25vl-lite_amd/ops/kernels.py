@@ -21,6 +21,7 @@ __all__ = ["rope_table", "copy_pages",
 
 _c_int, _c_float, _c_ptr = ctypes.c_int, ctypes.c_float, ctypes.c_void_p
 
+GATED_ACTS = {"silu": 0, "gelu_tanh": 1}   # activations of a gated feed-forward, by the kernels' flag
 _ERRORS = {1: "shape", 2: "dtype", 3: "launch", 4: "size limit"}
 
 
@@ -244,7 +245,8 @@ def paged_attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
                             block_table: torch.Tensor, token_req: torch.Tensor, token_seqpos: torch.Tensor,
                             num_q_heads: int, window: Optional[int], scale: float,
                             out: Optional[torch.Tensor] = None, keep_first: int = 0,
-                            sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+                            sinks: Optional[torch.Tensor] = None, chunk: Optional[int] = None,
+                            turn: Optional[torch.Tensor] = None, turn_pairs: bool = False) -> torch.Tensor:
     """Attention of every token over its request's pages; any head size, float32 arithmetic.
 
     ``q`` is ``[N, nq hd]``; token ``n`` belongs to row ``token_req[n]`` of ``block_table`` and
@@ -252,8 +254,11 @@ def paged_attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
     with a window, the first ``keep_first`` keys of its request.  The result is ``[N, nq vd]``,
     ``vd`` being the value width of ``v_cache [pages, nkv, vd, page_size]``.  ``sinks`` (float32 ``[nq]``): the
     softmax's denominator of head ``h`` also holds ``exp(sinks[h])``, a term with no key and no value.
+    ``chunk``: a token sees the keys from its chunk's first position on (chunks of that many positions from the
+    sequence's start).  ``turn`` (float32 ``[N, vd/2, 2]``): the cached values are turned by their positions; each
+    head's output is turned back by these angles (``turn_pairs``: channel 2m with 2m + 1, else m with m + vd/2).
     """
-    _dev(q, k_cache, v_cache, block_table, token_req, token_seqpos, out, sinks)
+    _dev(q, k_cache, v_cache, block_table, token_req, token_seqpos, out, sinks, turn)
     n = q.shape[0]
     nq = int(num_q_heads)
     _need(k_cache.dim() == 4 and k_cache.is_contiguous() and v_cache.is_contiguous(), "cache must be contiguous")
@@ -273,18 +278,22 @@ def paged_attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
     _need(keep_first >= 0, "keep_first cannot be negative")
     _need(sinks is None or (sinks.dtype == torch.float32 and sinks.shape == (nq,) and sinks.is_contiguous()),
           "sinks must be float32 [nq]")
+    _need(turn is None or (turn.dtype == torch.float32 and turn.dim() == 3 and turn.is_contiguous() and vd % 2 == 0
+                           and turn.shape[0] >= n and tuple(turn.shape[1:]) == (vd // 2, 2)), "turn must be float32 [N, vd/2, 2]")
+    _need(chunk is None or chunk > 0, "a chunk holds at least one position")
     fn = _fn("attention_generic", "qvl_attn_generic",
              [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int,
-              _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_int, _c_ptr])
+              _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr])
     _check(fn(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(token_req),
               _ptr(token_seqpos), _ptr(out), n, nq, nkv, hd, vd, ps, int(window or 0),
-              int(keep_first) if window else 0, float(scale), _ptr(sinks), dtype_code(q.dtype), _stream()),
+              int(keep_first) if window else 0, int(chunk or 0), float(scale), _ptr(sinks), _ptr(turn), int(turn_pairs),
+              dtype_code(q.dtype), _stream()),
            "paged_attention_generic")
     return out
 
 
-def swiglu(x: torch.Tensor, out: Optional[torch.Tensor] = None, grouped: bool = False) -> torch.Tensor:
-    """``silu(gate) * up`` for ``x`` of ``[N, 2 I]``: gate in the first ``I`` columns and up in the
+def swiglu(x: torch.Tensor, out: Optional[torch.Tensor] = None, grouped: bool = False, act: str = "silu") -> torch.Tensor:
+    """``act(gate) * up`` (``act`` ``"silu"``, or ``"gelu_tanh"``, the tanh form of gelu) for ``x`` of ``[N, 2 I]``: gate in the first ``I`` columns and up in the
     rest, or, ``grouped``, in alternating groups of 8 gate and 8 up columns."""
     _dev(x, out)
     _need(x.dim() == 2 and x.shape[1] % 2 == 0 and x.is_contiguous(), "x must be contiguous [N, 2 I]")
@@ -293,8 +302,8 @@ def swiglu(x: torch.Tensor, out: Optional[torch.Tensor] = None, grouped: bool = 
         out = torch.empty((n, inter), dtype=x.dtype, device=x.device)
     _need(out.shape == (n, inter) and out.dtype == x.dtype and out.is_contiguous(), "out must be [N, I]")
     _need(not grouped or inter % 8 == 0, "grouped columns need a width in steps of 8")
-    fn = _fn("elementwise", "qvl_swiglu", [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr])
-    _check(fn(_ptr(x), _ptr(out), n, inter, dtype_code(x.dtype), int(grouped), _stream()), "swiglu")
+    fn = _fn("elementwise", "qvl_swiglu", [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr])
+    _check(fn(_ptr(x), _ptr(out), n, inter, dtype_code(x.dtype), int(grouped), GATED_ACTS[act], _stream()), "swiglu")
     return out
 
 

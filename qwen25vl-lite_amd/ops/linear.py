@@ -15,7 +15,7 @@ import torch
 
 from . import kernels, skinny
 
-__all__ = ["NormedRows", "linear", "linear_into", "gate_up_swiglu", "tune_library_products"]
+__all__ = ["NormedRows", "linear", "linear_into", "linear_stack", "gate_up_swiglu", "tune_library_products"]
 
 
 class NormedRows:
@@ -30,7 +30,9 @@ class NormedRows:
         return kernels.add_rmsnorm(self.h, None, self.weight, self.eps, self.dtype)
 
 
-def _library(x: torch.Tensor, weight: torch.Tensor, bias, out_dtype) -> torch.Tensor:
+def _library(x: torch.Tensor, weight: torch.Tensor, bias, out_dtype, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    if out is not None:
+        return torch.mm(x, weight.t(), out=out)
     if out_dtype == torch.float32:
         y = torch.mm(x, weight.t(), out_dtype=torch.float32)  # float32 accumulator written out unrounded
     else:
@@ -67,6 +69,23 @@ def linear(x: Union[torch.Tensor, NormedRows], weight: torch.Tensor, bias: Optio
     if x.dtype == torch.float32 and weight.dtype == torch.float32:
         return kernels.gemm_f32(x, weight, bias)
     raise kernels.KernelError(f"linear: operands {x.dtype}/{weight.dtype} are not built")
+
+
+def linear_stack(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """``x[i] @ weight[i].T`` for ``x [S, M, K]`` and ``weight [S, N, K]``: ``[S, M, N]`` in the run dtype."""
+    s, m, k = x.shape
+    kernels._need(weight.dim() == 3 and weight.shape[0] == s and weight.shape[2] == k and weight.is_contiguous()
+                  and x.stride(2) == 1 and x.dtype == weight.dtype, "x [S, M, K] and weight [S, N, K] of one dtype")
+    kernels._dev(x, weight)
+    out = torch.empty((s, m, weight.shape[1]), dtype=x.dtype, device=x.device)
+    for i in range(s):
+        if weight.dtype == torch.float32:
+            kernels.gemm_f32(x[i], weight[i], out=out[i])
+        elif m <= skinny.ONE_BLOCK_ROWS and skinny.takes_resident(m, k, weight[i]) and _aligned(x[i]):
+            skinny.resident_product(weight[i], x=x[i], out=out[i], out_dtype=torch.bfloat16)
+        else:
+            _library(x[i], weight[i], None, torch.bfloat16, out=out[i])
+    return out
 
 
 def _aligned(x: torch.Tensor) -> bool:
@@ -108,8 +127,8 @@ def tune_library_products(enable: bool = True, max_ms: int = 3000) -> None:
     tunable.tuning_enable(enable)
 
 
-def gate_up_swiglu(x: Union[torch.Tensor, NormedRows], weight: torch.Tensor, grouped: bool) -> torch.Tensor:
-    """``silu(x Wg^T) * (x Wu^T)`` for ``weight`` holding gate and up rows: plain (gate rows, then up
+def gate_up_swiglu(x: Union[torch.Tensor, NormedRows], weight: torch.Tensor, grouped: bool, act: str = "silu") -> torch.Tensor:
+    """``act(x Wg^T) * (x Wu^T)`` (``act`` ``"silu"`` or ``"gelu_tanh"``) for ``weight`` holding gate and up rows: plain (gate rows, then up
     rows) or ``grouped`` (alternating groups of 8 gate rows and 8 up rows).  With few bfloat16 rows
     and grouped rows the activation is applied inside the product's kernel."""
     m, k = x.shape
@@ -117,7 +136,7 @@ def gate_up_swiglu(x: Union[torch.Tensor, NormedRows], weight: torch.Tensor, gro
             and m <= skinny.ONE_BLOCK_ROWS):
         lazy = isinstance(x, NormedRows)
         if lazy and skinny.takes_resident(m, k, weight, norm=True):
-            return skinny.resident_product(weight, h=x.h, norm_weight=x.weight, eps=x.eps, epilogue=skinny.SWIGLU)
+            return skinny.resident_product(weight, h=x.h, norm_weight=x.weight, eps=x.eps, epilogue=skinny.GATED[act])
         if not lazy and x.dtype == torch.bfloat16 and skinny.takes_resident(m, k, weight) and _aligned(x):
-            return skinny.resident_product(weight, x=x, epilogue=skinny.SWIGLU)
-    return kernels.swiglu(linear(x, weight), grouped=grouped)
+            return skinny.resident_product(weight, x=x, epilogue=skinny.GATED[act])
+    return kernels.swiglu(linear(x, weight), grouped=grouped, act=act)

@@ -31,10 +31,12 @@ def decayed_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, num_hea
                  state: torch.Tensor, cu_q: torch.Tensor, req_slots: torch.Tensor, *,
                  head_decay: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None, tau: float = 1.0,
                  silu=False, q_scale: float = 1.0, groups: int = 1, out: Optional[torch.Tensor] = None,
-                 lower: Optional[torch.Tensor] = None, z_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 lower: Optional[torch.Tensor] = None, z_bias: Optional[torch.Tensor] = None,
+                 exp_decay: bool = False, bonus: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Run every request's tokens of the step through the recurrence, from and into ``state``.
 
-    ``proj [N, cols]`` (float32 or bfloat16) holds, per token, ``heads * dim`` query columns from
+    ``proj [N, cols]`` or ``[parts, N, cols]`` (float32 or bfloat16; an offset then counts through the parts,
+    ``part * cols + column``) holds, per token, ``heads * dim`` query columns from
     ``q_off``, as many key columns from ``k_off`` and ``heads * vdim`` value columns from ``v_off``;
     ``silu`` applies the activation as they are read (True: to all three; or a string naming which, e.g.
     ``"q"``), ``q_scale`` scales the queries.
@@ -42,19 +44,21 @@ def decayed_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, num_hea
     channel, ``sigmoid(z)^(1/tau)`` for float32 ``z [N, heads * dim]``, or, with ``lower`` (float32
     ``[heads * dim]``, and ``z_bias`` of the same shape or None), the floored forget gate
     ``lower + (1 - lower) sigmoid(z + z_bias)``, whose complement ``1 - decay`` is then the key (no key
-    columns are read).  ``cu_q [R + 1]`` bounds each
+    columns are read), or, with ``exp_decay``, ``exp(-exp(z + z_bias))`` (``z_bias`` of that shape or None); then
+    with ``bonus`` (float32 ``[heads * dim]``) the outputs are ``o_t = (S_(t-1) + diag(bonus) k_t v_t^T)^T q_t``,
+    formed before the state moves on.  ``cu_q [R + 1]`` bounds each
     request's run of tokens, ``req_slots [R]`` names its row of ``state``.  Returns float32
     ``[groups, N, heads * vdim]``: with ``groups`` above 1 (2, 4 or 8; the key size must be a multiple
     of four times it) the key channels are cut into that many groups with blocks of their own, and the
     output is the sum of the slabs (see :func:`scan_groups`)."""
-    _dev(proj, state, cu_q, req_slots, head_decay, z, lower, z_bias)
+    _dev(proj, state, cu_q, req_slots, head_decay, z, lower, z_bias, bonus)
     h, d, v = int(num_heads), int(dim), int(vdim)
-    n = proj.shape[0]
+    n = proj.shape[-2]
     _need(1 <= d <= MAX_KEY_SIZE, f"key sizes up to {MAX_KEY_SIZE} are built")
-    _need(proj.dim() == 2 and proj.stride(1) == 1, "proj must be [N, cols] with contiguous rows")
-    _check_forget(lower, z_bias, z, h * d)
-    for off, width in ((q_off, h * d), (q_off if lower is not None else k_off, h * d), (v_off, h * v)):
-        _need(0 <= off and off + width <= proj.shape[1], "q, k or v columns lie outside proj")
+    _need(proj.dim() in (2, 3) and proj.stride(-1) == 1, "proj must be [N, cols] or [parts, N, cols] with contiguous rows")
+    _check_forget(lower, z_bias, z, h * d, exp_decay, bonus)
+    offs = [_place(proj, off, width) for off, width in
+            ((q_off, h * d), (q_off if lower is not None else k_off, h * d), (v_off, h * v))]
     _need(state.dtype == torch.float32 and state.dim() == 4 and tuple(state.shape[1:]) == (h, d, v)
           and state.is_contiguous(), "state must be contiguous float32 [slots, heads, dim, vdim]")
     for t in (cu_q, req_slots):
@@ -77,12 +81,12 @@ def decayed_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, num_hea
     _need(out.dtype == torch.float32 and out.shape == (groups, n, h * v) and out.is_contiguous() and out.is_cuda,
           "out must be contiguous float32 [groups, N, heads vdim]")
     fn = _fn("linear_attention", "qvl_la_scan",
-             [_c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ll, _c_float, _c_ptr, _c_ptr, _c_ptr,
-              _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr],
+             [_c_ptr, _c_ll, _c_ll, _c_ll, _c_ll, _c_int, _c_ptr, _c_ptr, _c_ll, _c_float, _c_ptr, _c_ptr, _c_int, _c_ptr,
+              _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr],
              {"LA_DIM": d})
-    _check(fn(_ptr(proj), proj.stride(0), int(q_off), int(k_off), int(v_off), dtype_code(proj.dtype),
-              _ptr(head_decay), _ptr(z), zstride, 1.0 / float(tau), _ptr(lower), _ptr(z_bias), _ptr(state), _ptr(cu_q),
-              _ptr(req_slots), _ptr(out), out.stride(0), int(groups), r, h, d, v, silu_mask(silu), float(q_scale),
+    _check(fn(_ptr(proj), proj.stride(-2), *offs, dtype_code(proj.dtype),
+              _ptr(head_decay), _ptr(z), zstride, 1.0 / float(tau), _ptr(lower), _ptr(z_bias), int(bool(exp_decay)),
+              _ptr(bonus), _ptr(state), _ptr(cu_q), _ptr(req_slots), _ptr(out), out.stride(0), int(groups), r, h, d, v, silu_mask(silu), float(q_scale),
               _stream()), "decayed_scan")
     return out
 
@@ -98,14 +102,26 @@ def silu_mask(silu) -> int:
     return sum(bit for name, bit in (("q", 1), ("k", 2), ("v", 4)) if name in silu)
 
 
-def _check_forget(lower, z_bias, z, width: int) -> None:
-    if lower is None:
-        _need(z_bias is None, "a bias on z belongs to the floored forget gate")
+def _check_forget(lower, z_bias, z, width: int, exp_decay: bool, bonus) -> None:
+    _need(not (exp_decay and lower is not None), "a decay is a floored forget gate or a double exponential")
+    _need(bonus is None or exp_decay, "the bonus is built for the double exponential's decay")
+    if lower is None and not exp_decay:
+        _need(z_bias is None, "a bias on z belongs to the floored forget gate or the double exponential")
         return
-    _need(z is not None, "the floored forget gate needs z")
-    for t in (lower, z_bias):
+    _need(z is not None, "the floored forget gate and the double exponential need z")
+    for t in (lower, z_bias, bonus):
         _need(t is None or (t.dtype == torch.float32 and t.shape == (width,) and t.is_contiguous()),
-              "lower and z_bias must be float32 [heads dim]")
+              "lower, z_bias and bonus must be float32 [heads dim]")
+
+
+def _place(proj: torch.Tensor, off: int, width: int) -> int:
+    """Where columns ``off ..`` of the first row start, in values from the tensor's start; ``off`` counts columns, through
+    the parts of a tensor of several."""
+    cols = proj.shape[-1]
+    part, col = divmod(int(off), cols)
+    _need(0 <= off and col + width <= cols and part < (proj.shape[0] if proj.dim() == 3 else 1),
+          "q, k or v columns lie outside proj")
+    return part * (proj.stride(0) if proj.dim() == 3 else 0) + col
 
 
 def scan_groups(num_reqs: int, max_run: int, num_heads: int, dim: int, vdim: int, device=None) -> int:
@@ -155,29 +171,33 @@ def chunked_scan(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, num_hea
                  state: torch.Tensor, plan: ChunkPlan, req_slots: torch.Tensor, *,
                  head_decay: Optional[torch.Tensor] = None, z: Optional[torch.Tensor] = None, tau: float = 1.0,
                  silu=False, q_scale: float = 1.0, lower: Optional[torch.Tensor] = None,
-                 z_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 z_bias: Optional[torch.Tensor] = None, exp_decay: bool = False,
+                 bonus: Optional[torch.Tensor] = None) -> torch.Tensor:
     """:func:`decayed_scan` for steps with long runs: the chunks of ``plan`` are scanned side by side
     from zero states, the states are carried from chunk to chunk, and what the state before a chunk
     adds to the chunk's outputs is one float32 matrix product per (chunk, head), ``(q_t P_t) S``
-    with ``P_t`` the product of the decays from the chunk's first token to ``t``.  Returns float32
+    with ``P_t`` the product of the decays from the chunk's first token to ``t`` (with a bonus: to the token before).  Returns float32
     ``[slabs, N, heads * vdim]`` whose sum over the slabs is the output (the last slab holds the
     second term)."""
     h, d, v = int(num_heads), int(dim), int(vdim)
-    n = proj.shape[0]
+    n = proj.shape[-2]
     nch, clen = plan.chunks, plan.chunk_len
     scratch = torch.zeros((nch, h, d, v), dtype=torch.float32, device=proj.device)
     groups = scan_groups(nch, clen, h, d, v, proj.device)
     out = torch.empty((groups + 1, n, h * v), dtype=torch.float32, device=proj.device)
     decayed_scan(proj, q_off, k_off, v_off, h, d, v, scratch, plan.chunk_cu, plan.chunk_rows, head_decay=head_decay,
-                 z=z, tau=tau, silu=silu, q_scale=q_scale, groups=groups, out=out[:groups], lower=lower, z_bias=z_bias)
+                 z=z, tau=tau, silu=silu, q_scale=q_scale, groups=groups, out=out[:groups], lower=lower, z_bias=z_bias,
+                 exp_decay=exp_decay, bonus=bonus)
     qp = torch.zeros((nch, h, clen, d), dtype=torch.float32, device=proj.device)
     last = torch.empty((nch, h, d), dtype=torch.float32, device=proj.device)
     defines = {"LA_DIM": d}
     fn = _fn("linear_attention", "qvl_la_prefix",
-             [_c_ptr, _c_ll, _c_int, _c_int, _c_ptr, _c_ptr, _c_ll, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+             [_c_ptr, _c_ll, _c_ll, _c_int, _c_ptr, _c_ptr, _c_ll, _c_float, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr,
+              _c_ptr, _c_ptr,
               _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr], defines)
-    _check(fn(_ptr(proj), proj.stride(0), int(q_off), dtype_code(proj.dtype), _ptr(head_decay), _ptr(z),
-              z.stride(0) if z is not None else 0, 1.0 / float(tau), _ptr(lower), _ptr(z_bias), _ptr(plan.chunk_cu),
+    _check(fn(_ptr(proj), proj.stride(-2), _place(proj, q_off, h * d), dtype_code(proj.dtype), _ptr(head_decay), _ptr(z),
+              z.stride(0) if z is not None else 0, 1.0 / float(tau), _ptr(lower), _ptr(z_bias), int(bool(exp_decay)),
+              int(bonus is not None), _ptr(plan.chunk_cu),
               _ptr(qp), _ptr(last), nch, h, d, clen, silu_mask(silu), float(q_scale), _stream()), "chunk prefix")
     r = req_slots.shape[0]
     _need(plan.req_first.shape[0] == r + 1, "the chunk plan belongs to another step")

@@ -16,7 +16,7 @@ import torch
 from .kernels import _check, _fn, _ptr, _stream, dtype_code
 
 __all__ = ["resident_product", "takes_resident", "qkv_rope_product", "takes_qkv_rope", "RESIDENT_ROWS", "resident_norm_k", "resident_two_tile_k", "folds_norm", "ONE_BLOCK_ROWS", "split_product", "takes_split", "prefers_split", "SPLIT_ROWS",
-           "STORE", "RESIDUAL", "SWIGLU"]
+           "STORE", "RESIDUAL", "SWIGLU", "GEGLU", "GATED"]
 
 RESIDENT_ROWS = 64       # up to here the resident kernel runs
 ONE_TILE_ROWS = 16       # the rows of one column tile of the matrix instruction
@@ -25,7 +25,8 @@ ONE_BLOCK_ROWS = 32      # up to here one block carries all rows: beyond, teams 
 _MAX_WEIGHT_BYTES = 0xffffff00   # qvl_gemm_resident_max_weight_bytes() + 1
 _pass_k = None
 _two_tile_k = None
-STORE, RESIDUAL, SWIGLU = 0, 1, 2
+STORE, RESIDUAL, SWIGLU, GEGLU = 0, 1, 2, 4
+GATED = {"silu": SWIGLU, "gelu_tanh": GEGLU}
 _c_int, _c_float, _c_ptr = ctypes.c_int, ctypes.c_float, ctypes.c_void_p
 _cu_count = {}
 
@@ -106,9 +107,9 @@ def resident_product(weight: torch.Tensor, *, x: Optional[torch.Tensor] = None, 
                      out: Optional[torch.Tensor] = None, out_dtype: torch.dtype = torch.float32) -> torch.Tensor:
     """``X @ weight.T`` for at most 64 rows (``h`` for at most 32).  ``X`` is ``x`` (bfloat16), or ``rmsnorm(h) * norm_weight``
     formed inside the kernel from the float32 rows ``h``.  ``epilogue``: ``STORE`` writes the product
-    (plus ``bias``) to a new tensor of ``out_dtype``; ``RESIDUAL`` adds it to ``out`` (float32) in
+    (plus ``bias``) to ``out``, or to a new tensor, of ``out_dtype``; ``RESIDUAL`` adds it to ``out`` (float32) in
     place; ``SWIGLU`` takes ``weight``'s rows as groups of 8 gate, 8 up rows and returns
-    ``silu(gate) * up`` as bfloat16 ``[M, N/2]``."""
+    ``silu(gate) * up`` as bfloat16 ``[M, N/2]`` (``GEGLU``: with the tanh form of gelu)."""
     src = x if x is not None else h
     m, k = src.shape
     n = weight.shape[0]
@@ -125,12 +126,16 @@ def resident_product(weight: torch.Tensor, *, x: Optional[torch.Tensor] = None, 
         if out is None or out.dtype != torch.float32 or out.shape != (m, n) or out.stride(1) != 1:
             raise ValueError("the residual must be float32 [M, N]")
         odt = torch.float32
-    elif epilogue == SWIGLU:
+    elif epilogue in (SWIGLU, GEGLU):
         if n % 16:
             raise ValueError("gate | up rows must come in groups of 8 + 8")
         out, odt = torch.empty((m, n // 2), dtype=torch.bfloat16, device=src.device), torch.bfloat16
     else:
-        out, odt = torch.empty((m, n), dtype=out_dtype, device=src.device), out_dtype
+        odt = out_dtype
+        if out is None:
+            out = torch.empty((m, n), dtype=odt, device=src.device)
+        elif out.dtype != odt or out.shape != (m, n) or out.stride(1) != 1:
+            raise ValueError("out must be [M, N] of out_dtype")
     fn = _fn("gemm_resident", "qvl_gemm_resident",
              [_c_ptr, _c_int, _c_ptr, _c_int, _c_ptr, _c_float, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int,
               _c_int, _c_int, _c_int, _c_int, _c_ptr], _build_for(k))

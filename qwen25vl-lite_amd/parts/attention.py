@@ -51,7 +51,11 @@ class PagedAttention(Mixer):
     convolution over time, ``y_t = sum_j w[:, j] u_(t - taps + 1 + j)`` per channel with weights ``q_conv`` /
     ``k_conv`` of ``[channels, taps]``, before norm and rotation; keys that are their own values are taken behind
     it; a request's last ``taps - 1`` projected rows are its state), ``sinks`` (True: a tensor ``sink [heads]``
-    whose ``exp`` joins each head's softmax denominator).  Any of these except the output bias and the sinks
+    whose ``exp`` joins each head's softmax denominator), ``chunk`` (a number: positions are cut into chunks of
+    that many from the sequence's start and a token sees the keys of its own chunk up to itself), ``value_rotation`` (a
+    base: the value of position j is turned by j over all its channels before it is cached, in the position encoding's
+    layout of pairs, pair m by ``j base^(-2m/value_dim)``, and each head's output at position i is turned back by i).
+    Any of these except the output bias, the sinks and the chunks
     takes the projection through float32 and one kernel that norms, rotates and writes the cache."""
 
     graph_safe = True
@@ -79,6 +83,9 @@ class PagedAttention(Mixer):
         self.qk_norm_scope = str(params.get("qk_norm_scope", "head"))
         self.conv_taps = int(params.get("conv_taps") or 0)
         self.has_sinks = bool(params.get("sinks", False))
+        self.chunk: Optional[int] = None if params.get("chunk") is None else int(params["chunk"])
+        if self.chunk is not None and self.chunk < 1:
+            raise ValueError("a chunk holds at least one position")
         self.vd = int(params.get("value_dim") or self.hd)
         self.keep_first = int(params.get("keep_first") or 0) if self.window else 0
         if self.qk_norm_where not in ("before", "after"):
@@ -87,6 +94,12 @@ class PagedAttention(Mixer):
             raise ValueError("an attention mixer has one kind of output gate at most")
         if self.values_are_keys and self.vd != self.hd:
             raise ValueError("keys that are their own values have the keys' width")
+        self.value_position = None
+        if params.get("value_rotation") is not None:
+            if self.values_are_keys or self.kv_shared or self.vd % 2:
+                raise ValueError("values that are turned by their positions are projections of their own, of even width")
+            self.value_position = build_part("position", PartSpec("rope", {"theta": float(params["value_rotation"])}), dtype,
+                                             device)
         if self.keep_first < 0:
             raise ValueError("keep_first cannot be negative")
         if self.qk_norm_scope not in ("head", "whole"):
@@ -109,7 +122,8 @@ class PagedAttention(Mixer):
         self.position = build_part("position", pos, dtype, device)
         self.interleaved = bool(getattr(self.position, "interleaved", False))
         self.normed_path = (self.qk_norm_eps is not None or self.values_are_keys or self.head_gate
-                            or self.element_gate or self.interleaved or self.vd != self.hd or bool(self.conv_taps))
+                            or self.element_gate or self.interleaved or self.vd != self.hd or bool(self.conv_taps)
+                            or self.value_position is not None)
         self.gate_rows = self.nq if self.head_gate else (self.nq * self.vd if self.element_gate else 0)
         self.w_in: Optional[torch.Tensor] = None
         self.b_in: Optional[torch.Tensor] = None
@@ -119,7 +133,7 @@ class PagedAttention(Mixer):
         self.sink: Optional[torch.Tensor] = None
 
     def cache_need(self) -> CacheNeed:
-        return CacheNeed(self.nkv, self.hd, self.window, self.keep_first, None if self.vd == self.hd else self.vd)
+        return CacheNeed(self.nkv, self.hd, self.window, self.keep_first, None if self.vd == self.hd else self.vd, self.chunk)
 
     @property
     def conv_channels(self) -> int:
@@ -234,7 +248,7 @@ class PagedAttention(Mixer):
         if q is None:
             q = self._project(x, step, group, slot, write, inv_freq, freq_row)
         o = paged_attention(q, slot.k_cache, slot.v_cache, group.block_table, step, self.nq, self.window, self.scale,
-                            keep_first=self.keep_first, sinks=self.sink)
+                            keep_first=self.keep_first, sinks=self.sink, chunk=self.chunk)
         return self._output(o, step)
 
     def _output(self, o: torch.Tensor, step: StepContext):
@@ -252,6 +266,10 @@ class PagedAttention(Mixer):
 
         proj = linear(x, self.w_in, out_dtype=torch.float32)     # the bias is added by the kernel that norms
         cs = self._rotation_table(step, inv_freq, freq_row, proj.shape[0])
+        value_cs = None
+        if self.value_position is not None:
+            value_cs = self._rotation_table(step, *self.value_position.rotary_tables(self.vd), proj.shape[0],
+                                            self.value_position, self.vd)
         heads_in = proj
         if self.conv_taps:
             from ..ops.short_conv import short_conv
@@ -264,9 +282,11 @@ class PagedAttention(Mixer):
             heads_in, self.q_norm, self.k_norm, self.qk_norm_eps if self.qk_norm_eps is not None else 0.0, cs,
             group.slot_mapping if write else None, slot.k_cache if write else None, slot.v_cache if write else None,
             self.nq, self.nkv, self.hd, group.page_size, self.dtype, interleaved=self.interleaved,
-            values_are_keys=self.values_are_keys, norm=norm, bias=self.b_in, value_dim=self.vd)
+            values_are_keys=self.values_are_keys, norm=norm, bias=self.b_in, value_dim=self.vd,
+            value_cs=value_cs)
         o = paged_attention(q, slot.k_cache, slot.v_cache, group.block_table, step, self.nq, self.window, self.scale,
-                            keep_first=self.keep_first, sinks=self.sink)
+                            keep_first=self.keep_first, sinks=self.sink, chunk=self.chunk, turn=value_cs,
+                            turn_pairs=self.interleaved)
         if self.gate_rows:
             # one gate per head, or one per element (a "head" of one channel)
             at = self.w_in.shape[0] - self.gate_rows
@@ -290,14 +310,15 @@ class PagedAttention(Mixer):
             group.slot_mapping if write else None, slot.k_cache if write else None, slot.v_cache if write else None,
             self.nq, self.nkv if write else 0, self.hd, group.page_size, out_dtype=self.dtype, cs=cs)
 
-    def _rotation_table(self, step, inv_freq, freq_row, n: int) -> torch.Tensor:
+    def _rotation_table(self, step, inv_freq, freq_row, n: int, position=None, width: Optional[int] = None) -> torch.Tensor:
         """Cosines and sines of the step's angles: computed once per pass and position encoding,
         by the first layer that needs them, and read by every head of every layer."""
-        key = ("rope_cs", self.position.table_key(self.hd))
+        position = self.position if position is None else position
+        key = ("rope_cs", position.table_key(self.hd if width is None else width))
         cs = step.per_pass.get(key)
         if cs is None:
             cs = step.per_pass[key] = kernels.rope_table(step.positions, inv_freq, freq_row, n,
-                                                         amplitude=float(getattr(self.position, "amplitude", 1.0)))
+                                                         amplitude=float(getattr(position, "amplitude", 1.0)))
         return cs
 
     def _project_few_rows(self, x, step, group, slot, write, inv_freq, freq_row) -> Optional[torch.Tensor]:

@@ -19,8 +19,10 @@ Kinds of parts and what each must provide:
 * ``PositionEncoding``: ``rotary_tables(head_dim, device)`` gives the per-frequency inverse
   frequencies and the row of the position tensor each frequency reads.
 * ``Block``: ``forward(stream, step, slot)`` arranges two norms, a mixer and a feed-forward.
-* ``Filter``: ``forward(h, step, slot) -> x``: what a sublayer reads, made from the float32 residual (a
-  short convolution over time); it may keep a per-request state like a mixer.
+* ``Filter``: ``forward(h, step, slot) -> x``: what a sublayer reads, made from float32 rows (a short
+  convolution over time, a step towards the token before); it may keep a per-request state like a mixer.
+* ``Embedding``: ``forward(token_ids, step) -> h``; one with a ``state_need()`` of its own is called with its
+  slot as a third argument.
 
 New kinds are added with :func:`register_part` and named in a model's layer specs.
 """
@@ -34,6 +36,7 @@ import torch
 
 __all__ = [
     "ParamSpec", "PartSpec", "CacheNeed", "StateNeed", "LayerSlot", "GroupStep", "StepContext", "ResidualStream",
+    "NormedMean",
     "Part", "Norm", "Mixer", "FeedForward", "Filter", "PositionEncoding", "Block", "register_part", "build_part",
     "known_parts", "Embedding", "Head",
 ]
@@ -46,11 +49,20 @@ class ParamSpec:
     float32 (norm weights, biases: they enter float32 arithmetic), ``"int"`` as int32.
     ``init`` says how the random-weights mode draws it: ``"normal"`` N(0, std),
     ``"around_one"`` 1 + N(0, std) (a gain), ``"zeros"``, ``"ones"``, ``"unit_interval"`` uniform on [0, 1)
-    (a floor of a gate)."""
+    (a floor of a gate), ``"identity"`` a square matrix of N(0, std) plus the identity.  ``free``: the axes
+    whose size the checkpoint decides (the part takes whatever comes and checks that its tensors fit each
+    other); ``shape`` then holds the size the random-weights mode draws."""
 
     shape: Tuple[int, ...]
     role: str = "matrix"
     init: str = "normal"
+    free: Tuple[int, ...] = ()
+
+    def takes(self, shape) -> bool:
+        """Whether a stored tensor of this shape fits."""
+        shape = tuple(shape)
+        return len(shape) == len(self.shape) and all(
+            got > 0 if axis in self.free else got == want for axis, (got, want) in enumerate(zip(shape, self.shape)))
 
 
 @dataclass(frozen=True)
@@ -66,17 +78,28 @@ class CacheNeed:
     """Keys and values a mixer keeps per token.  ``window`` None: all keys stay; a number:
     only the last ``window`` keys are read, older pages may be given back, except the pages of
     the first ``keep_first`` tokens, which every later token still reads.  ``value_dim`` None:
-    values are as wide as keys (``head_dim``)."""
+    values are as wide as keys (``head_dim``).  ``chunk`` a number: positions are cut into chunks of
+    that many from the sequence's start on and only keys of a token's own chunk are read."""
 
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     keep_first: int = 0
     value_dim: Optional[int] = None
+    chunk: Optional[int] = None
 
     @property
     def v_dim(self) -> int:
         return self.head_dim if self.value_dim is None else self.value_dim
+
+    def first_visible(self, position: int) -> int:
+        """The first key that a token at ``position``, and with it any later one, sees (kept first keys aside)."""
+        first = 0
+        if self.window is not None:
+            first = max(first, position - self.window + 1)
+        if self.chunk is not None:
+            first = max(first, position - position % self.chunk)
+        return first
 
 
 @dataclass(frozen=True)
@@ -97,9 +120,13 @@ class LayerSlot:
     v_cache: Optional[torch.Tensor] = None  # [pages, nkv, vd, page_size]
     writes: bool = True
     state: Optional[torch.Tensor] = None    # [max_num_seqs, *StateNeed.shape]
-    # a block with several mixers: each one's slot under the mixer's sub-part name (this slot is
-    # the first of them)
+    # the slot of a run entry: every part's that owns anything under its dotted name in the block (this
+    # slot stands for the first of them); the slot of a part: its own sub-parts' under their names in it
     by_part: Dict[str, "LayerSlot"] = field(default_factory=dict)
+
+    def of(self, name: str) -> "LayerSlot":
+        """The named part's slot, or this one where none is kept under that name."""
+        return self.by_part.get(name, self)
 
 
 @dataclass
@@ -152,6 +179,25 @@ class ResidualStream:
     pending_norm: Optional[Tuple[torch.Tensor, float, float]] = None
     # a vector float32 [hidden] that the next norm adds to every row of the sum
     row_addend: Optional[torch.Tensor] = None
+    # several copies of the sum, mixed anew by every sublayer (hyper-connections): float32 [N, copies, hidden].
+    # None while every copy still equals ``h`` (the embedding's output)
+    copies: Optional[torch.Tensor] = None
+    # (mix [copies, copies], out [copies]) float32: how the pending addend joins the copies
+    pending_join: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
+
+
+@dataclass
+class NormedMean:
+    """A sublayer's result that is ``factor * (rmsnorm(first) gain_first + rmsnorm(second) gain_second)`` and
+    has not been computed yet: the kernel that adds it to the sum forms it on the way.  The addends are ``[N, hidden]``
+    (float32 or run dtype) or float32 slabs ``[slabs, N, hidden]`` that are added in order."""
+
+    first: torch.Tensor
+    second: torch.Tensor
+    gain_first: torch.Tensor
+    gain_second: torch.Tensor
+    eps: float
+    factor: float
 
 
 class Part:
@@ -197,6 +243,10 @@ class Norm(Part):
 
 
 class Mixer(Part):
+    # a mixer that reads several mixes of a token's input with the one's before it names the sub-part that
+    # holds their weights (a TokenMixes part): a block may then hand it the mixes instead of the input
+    token_mixes: Optional[Part] = None
+
     def forward(self, x: torch.Tensor, step: StepContext, slot: LayerSlot) -> torch.Tensor:
         raise NotImplementedError
 
@@ -207,8 +257,8 @@ class FeedForward(Part):
 
 
 class Filter(Part):
-    """A transform of the float32 residual's rows on their way into a sublayer (a short convolution over
-    time); it may keep a state per request."""
+    """A transform of float32 rows (the residual's, or a norm's) on their way into a sublayer (a short
+    convolution over time, a step towards the token before); it may keep a state per request."""
 
     def forward(self, h: torch.Tensor, step: StepContext, slot: LayerSlot) -> torch.Tensor:
         """float32 ``[N, hidden]`` -> ``[N, hidden]`` in the run dtype."""
@@ -234,11 +284,12 @@ class Block(Part):
 
 
 class Embedding(Part):
-    """Token ids to the start of the residual sum.  ``table`` is the tensor a tied head shares."""
+    """Token ids to the start of the residual sum.  ``table`` is the tensor a tied head shares.  An
+    embedding may keep a state per request (``state_need``); ``forward`` then gets its slot too."""
 
     table: Optional[torch.Tensor] = None
 
-    def forward(self, token_ids: torch.Tensor, step: StepContext) -> torch.Tensor:
+    def forward(self, token_ids: torch.Tensor, step: StepContext, slot: Optional[LayerSlot] = None) -> torch.Tensor:
         """int32 ``[N]`` -> float32 ``[N, hidden]``."""
         raise NotImplementedError
 

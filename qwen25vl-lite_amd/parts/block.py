@@ -37,7 +37,7 @@ class PreNormBlock(Block):
     def forward(self, stream: ResidualStream, step: StepContext, slot: LayerSlot) -> ResidualStream:
         x = self.norm1.forward(stream, lazy=self.mixer.takes_lazy_norm)
         step.residual = stream.h            # the mixer may add its result in place and return None
-        stream.pending = self.mixer.forward(x, step, slot)
+        stream.pending = self.mixer.forward(x, step, slot.of(self.names["mixer"]))
         y = self.norm2.forward(stream, lazy=self.ffn.takes_lazy_norm)
         step.residual = stream.h
         stream.pending = self.ffn.forward(y, step)
@@ -89,7 +89,7 @@ class ParallelBlock(Block):
             x = self.norm.forward(stream)    # never lazily: h changes before the second reader would look
             x2 = x if self.norm2 is None else self.norm2.forward(stream)   # the sum is folded: this one only norms
         step.residual = stream.h
-        y = self.mixer.forward(x, step, slot)
+        y = self.mixer.forward(x, step, slot.of(self.names["mixer"]))
         if self.ffn is None:
             stream.pending = y
         else:
@@ -140,7 +140,7 @@ class SandwichBlock(Block):
     def forward(self, stream: ResidualStream, step: StepContext, slot: LayerSlot) -> ResidualStream:
         x = self.norm1.forward(stream)
         step.residual = None                 # a sublayer's result is normed before it joins the sum
-        stream.pending = self.mixer.forward(x, step, slot)
+        stream.pending = self.mixer.forward(x, step, slot.of(self.names["mixer"]))
         stream.pending_norm = (self.norm1b.weight, self.norm1b.eps, self.mult)
         if self.ffn is not None:
             y = self.norm2.forward(stream)
@@ -201,7 +201,7 @@ class PostNormBlock(Block):
             stream.pending = None
         h = stream.h
         step.residual = None                 # a sublayer's result is normed before it joins the sum
-        mixer_slot = slot.by_part.get(self.names["mixer"], slot)
+        mixer_slot = slot.of(self.names["mixer"])
         if self.filter is not None:
             x = self.filter.forward(h, step, slot.by_part.get(self.names["filter"]))
         else:

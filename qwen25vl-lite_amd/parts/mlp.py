@@ -13,9 +13,10 @@ __all__ = ["SwiGLU", "ClampedGatedFF", "PlainFF"]
 
 
 class SwiGLU(FeedForward):
-    """``down(silu(gate(x)) * up(x))`` without biases.
+    """``down(act(gate(x)) * up(x))`` without biases.
 
-    params: ``hidden_size``, ``intermediate_size``, ``names`` (local names of the gate, up and down matrices;
+    params: ``hidden_size``, ``intermediate_size``, ``activation`` (``"silu"``, the default, or ``"gelu_tanh"``, the
+    tanh form of gelu), ``names`` (local names of the gate, up and down matrices;
     default ``gate_proj``, ``up_proj``, ``down_proj``).
     """
 
@@ -29,6 +30,9 @@ class SwiGLU(FeedForward):
         # gate and up rows alternate in groups of 8 where the size allows: a 16-row tile of the
         # product then holds 8 features' gate and up and can apply the activation itself
         self.grouped = self.inter % 8 == 0
+        self.activation = str(params.get("activation", "silu"))
+        if self.activation not in ("silu", "gelu_tanh"):
+            raise ValueError(f"activation {self.activation!r}; known: silu, gelu_tanh")
         names = dict(params.get("names") or {})
         self.names = {k: names.get(k, f"{k}_proj") for k in ("gate", "up", "down")}
         self.w_gate_up: Optional[torch.Tensor] = None
@@ -61,7 +65,7 @@ class SwiGLU(FeedForward):
                 f"{self.names['down']}.weight": self.w_down}
 
     def forward(self, x, step: StepContext):
-        act = gate_up_swiglu(x, self.w_gate_up, self.grouped)
+        act = gate_up_swiglu(x, self.w_gate_up, self.grouped, self.activation)
         return linear_into(step.residual if step is not None else None, act, self.w_down)
 
 

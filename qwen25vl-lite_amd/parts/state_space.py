@@ -1,0 +1,134 @@
+"""A selective state-space mixer: a short convolution, step sizes and projections that depend on the token, and a
+diagonal recurrence per channel.
+
+``[x; z] = Win h``; ``x`` passes a causal convolution per channel with a bias and silu; ``[dt; B; C] = Wx x``; step
+sizes ``softplus(Wdt dt + b)``, one per channel; per channel c and state n ``S <- exp(step_c A[c, n]) S + step_c x_c B_n``,
+``y_c = sum_n S[c, n] C_n + D_c x_c``; then ``Wo (y silu(z))``.
+"""
+
+from __future__ import annotations
+
+from typing import Dict, Optional
+
+import torch
+
+from ..ops.linear import linear, linear_into
+from .base import LayerSlot, Mixer, ParamSpec, Part, StateNeed, StepContext, register_part
+
+__all__ = ["SelectiveStateSpace", "ConvolvedInput"]
+
+
+class ConvolvedInput(Part):
+    """``silu(b + sum_j w[:, j] x_(t - taps + 1 + j))`` per channel, zeros before a sequence's first token.  The last
+    ``taps - 1`` rows a request has brought are its state (float32, oldest first).  The weight is ``[channels, taps]``
+    in a checkpoint and kept tap-major in float32."""
+
+    graph_safe = True
+
+    def __init__(self, channels: int, taps: int, dtype, device):
+        super().__init__(dtype, device)
+        self.channels, self.taps = int(channels), int(taps)
+        if self.taps < 1:
+            raise ValueError("a convolution has at least one tap")
+        self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
+
+    def state_need(self) -> Optional[StateNeed]:
+        return StateNeed((self.taps - 1, self.channels), torch.float32) if self.taps > 1 else None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        return {"weight": ParamSpec((self.channels, self.taps), "vector"), "bias": ParamSpec((self.channels,), "vector")}
+
+    def load(self, tensors):
+        self.weight = tensors["weight"].t().contiguous()
+        self.bias = tensors["bias"]
+
+    def named_weights(self) -> Dict[str, torch.Tensor]:
+        return {"weight": self.weight.t(), "bias": self.bias}
+
+    def forward(self, x: torch.Tensor, step: StepContext, slot: LayerSlot) -> torch.Tensor:
+        from ..ops.short_conv import short_conv
+        if self.taps > 1 and slot.state is None:
+            raise RuntimeError("a convolution with more than one tap needs a state slot")
+        return short_conv(x, self.weight, slot.state if self.taps > 1 else None, step.cu_q, step.req_slots,
+                          step.token_req, self.dtype, bias=self.bias, silu=True)
+
+
+class SelectiveStateSpace(Mixer):
+    """params: ``hidden_size``, ``inner_size``, ``state_size``, ``dt_rank``, ``conv_taps``, ``names`` (local names of the
+    tensors' owners: ``in``, ``conv``, ``x``, ``dt``, ``a_log``, ``d``, ``o``; default these).
+
+    The input projection and what the convolution gives are in the run dtype; step sizes, decays, B, C and the state
+    (float32 ``[state_size, inner_size]`` per request) are float32.
+    """
+
+    graph_safe = True
+
+    def __init__(self, params, dtype, device):
+        super().__init__(dtype, device)
+        self.hidden, self.inner = int(params["hidden_size"]), int(params["inner_size"])
+        self.states, self.rank = int(params["state_size"]), int(params["dt_rank"])
+        names = dict(params.get("names") or {})
+        self.names = {k: names.get(k, k) for k in ("in", "conv", "x", "dt", "a_log", "d", "o")}
+        self.conv = ConvolvedInput(self.inner, int(params["conv_taps"]), dtype, device)
+        self.w_in: Optional[torch.Tensor] = None
+        self.w_x: Optional[torch.Tensor] = None
+        self.w_dt: Optional[torch.Tensor] = None
+        self.b_dt: Optional[torch.Tensor] = None
+        self.a_log: Optional[torch.Tensor] = None
+        self.a2: Optional[torch.Tensor] = None          # float32 [states, inner]: -exp(a_log) log2(e)
+        self.skip: Optional[torch.Tensor] = None
+        self.w_out: Optional[torch.Tensor] = None
+
+    def sub_parts(self) -> Dict[str, Part]:
+        return {self.names["conv"]: self.conv}
+
+    def state_need(self) -> StateNeed:
+        return StateNeed((self.states, self.inner), torch.float32)
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        n, c = self.names, self.inner
+        return {f"{n['in']}.weight": ParamSpec((2 * c, self.hidden)),
+                f"{n['x']}.weight": ParamSpec((self.rank + 2 * self.states, c)),
+                f"{n['dt']}.weight": ParamSpec((c, self.rank)),
+                f"{n['dt']}.bias": ParamSpec((c,), "vector"),
+                f"{n['a_log']}.weight": ParamSpec((c, self.states), "vector"),
+                f"{n['d']}.weight": ParamSpec((c,), "vector", init="around_one"),
+                f"{n['o']}.weight": ParamSpec((self.hidden, c))}
+
+    def load(self, tensors):
+        from ..ops.selective_scan import LOG2_E
+        n = self.names
+        self.w_in, self.w_x = tensors[f"{n['in']}.weight"], tensors[f"{n['x']}.weight"]
+        self.w_dt, self.b_dt = tensors[f"{n['dt']}.weight"], tensors[f"{n['dt']}.bias"]
+        self.a_log, self.skip = tensors[f"{n['a_log']}.weight"], tensors[f"{n['d']}.weight"]
+        self.a2 = (-torch.exp(self.a_log.t().double()) * LOG2_E).float().contiguous()
+        self.w_out = tensors[f"{n['o']}.weight"]
+
+    def named_weights(self) -> Dict[str, torch.Tensor]:
+        n = self.names
+        return {f"{n['in']}.weight": self.w_in, f"{n['x']}.weight": self.w_x, f"{n['dt']}.weight": self.w_dt,
+                f"{n['dt']}.bias": self.b_dt, f"{n['a_log']}.weight": self.a_log, f"{n['d']}.weight": self.skip,
+                f"{n['o']}.weight": self.w_out}
+
+    def forward(self, x: torch.Tensor, step: StepContext, slot: LayerSlot):
+        from ..ops.linear_attention import plan_chunks
+        from ..ops.selective_scan import CHUNKED_FROM, selective_scan
+
+        if slot.state is None:
+            raise RuntimeError("a state-space mixer needs a state slot")
+        both = linear(x, self.w_in)                                     # [N, x | z] in the run dtype
+        u = self.conv.forward(both[:, :self.inner], step, slot.of(self.names["conv"]))
+        low = linear(u, self.w_x, out_dtype=torch.float32)              # [N, dt | B | C]
+        dt = linear(low[:, :self.rank].to(self.dtype).contiguous(), self.w_dt, out_dtype=torch.float32)
+        plan = None
+        if step.max_q_len >= CHUNKED_FROM and len(step.cu_q_host) == step.num_reqs + 1:
+            plan = step.derived.get("la_chunks")
+            if plan is None:
+                plan = step.derived["la_chunks"] = plan_chunks(step.cu_q_host, self.device)
+        y = selective_scan(u, dt, self.b_dt, self.a2, low, self.rank, self.rank + self.states, self.skip,
+                           both[:, self.inner:], slot.state, step.cu_q, step.req_slots, plan)
+        return linear_into(step.residual, y, self.w_out)
+
+
+register_part("mixer", "selective_state_space", SelectiveStateSpace)

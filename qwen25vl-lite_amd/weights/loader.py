@@ -89,7 +89,7 @@ def load_weights(model_dir: str, model, *, strict: bool = True, progress=None) -
             tied = True
         wrong_shape, wrong_dtype = [], []
         for name, (f, raw) in where.items():
-            if f.shape(raw) != tuple(expected[name].shape):
+            if not expected[name].takes(f.shape(raw)):
                 wrong_shape.append((raw, f.shape(raw), tuple(expected[name].shape)))
             is_float = f.dtype(raw).is_floating_point
             if is_float != (expected[name].role != "int"):

@@ -34,7 +34,7 @@ def _draw(name: str, shape, seed: int, std: float, device, dtype: torch.dtype, i
         gen = torch.Generator(device=device)
         gen.manual_seed(_seed_for(seed, name))
         return torch.empty(tuple(shape), dtype=torch.float32, device=device).uniform_(0.0, 1.0, generator=gen).to(dtype)
-    if init not in ("normal", "around_one"):
+    if init not in ("normal", "around_one", "identity"):
         raise ValueError(f"{name}: no rule to draw a tensor with init {init!r}")
     gen = torch.Generator(device=device)
     gen.manual_seed(_seed_for(seed, name))
@@ -42,6 +42,8 @@ def _draw(name: str, shape, seed: int, std: float, device, dtype: torch.dtype, i
     t.normal_(0.0, std, generator=gen)
     if init == "around_one":
         t += 1.0
+    elif init == "identity":
+        t += torch.eye(*shape, dtype=t.dtype, device=device)
     return t.to(dtype)
 
 
