@@ -169,6 +169,31 @@ def rofapel_config(layers, size="7b", order=ROFAPEL_ORDER, experts=32, top=6, wi
     return cfg
 
 
+ZAPOSUN_ORDER = ("parallel", "wkv")
+
+
+def zaposun_config(layers, size="7b", order=ZAPOSUN_ORDER, chunk=1024, streams=4, groups=8):
+    """A Zaposun decoder with the width, head counts, feed-forward size and vocabulary of one of SIZES.  Layers in
+    the given order (repeated): ``parallel`` (attention with heads of 128 channels in chunks of ``chunk`` positions
+    beside a selective state space of twice the width, 16 states a channel and 4 taps), ``wkv`` (heads of 64 channels
+    that make up the width); ``streams`` copies of the residual sum, norms in ``groups`` parts, every layer with its
+    feed-forward."""
+    s = SIZES[size]
+    nh, nkv, hd, width = s["num_attention_heads"], s["num_key_value_heads"], 128, s["hidden_size"]
+    mixers = {
+        "parallel": {"left": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": chunk},
+                              "rot": {"base": 100000.0, "dims": hd // 2}},
+                     "right": {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4}},
+        "wkv": {"heads": width // 64, "dim": 64},
+    }
+    mlp = {"kind": "dense", "ff": s["intermediate_size"]}
+    return {"architecture": "Zaposun", "width": width, "vocab": s["vocab_size"], "norm": {"eps": 1e-6, "groups": groups},
+            "streams": streams, "logit_scale": 0.25,
+            "embedding": {"bigram": {"buckets": 65521, "mul_prev": 1009, "mul_cur": 31}},
+            "layers": [{"type": order[i % len(order)], "mixer": mixers[order[i % len(order)]], "mlp": mlp}
+                       for i in range(int(layers))]}
+
+
 def step_bytes(t, batch, ctx, bytes_per_value=2):
     """Bytes a decode step has to read: every weight it uses once (all layers and the head; of the
     embedding only the rows looked up) and the keys and values of the live requests."""
@@ -323,15 +348,15 @@ def main(argv=None) -> int:
     ap.add_argument("--attention", type=int, nargs="+", metavar="TOKENS",
                     help="instead: the prefill attention alone (one request of that many tokens in one step, the "
                          "chosen size's heads, bfloat16, pages in shuffled order), microseconds and TFLOP/s for each length")
-    ap.add_argument("--design", choices=["gogudra", "dazapel", "rapisun", "rofapel"],
+    ap.add_argument("--design", choices=["gogudra", "dazapel", "rapisun", "rofapel", "zaposun"],
                     help="instead: prefill (2,048 tokens) and decode throughput of this design at the chosen size's "
                          "width, heads and feed-forward (random weights), beside the Qwen2.5-VL decoder with as many layers")
-    ap.add_argument("--beside", choices=["qwen25vl", "gogudra", "dazapel", "rapisun"], default="qwen25vl",
+    ap.add_argument("--beside", choices=["qwen25vl", "gogudra", "dazapel", "rapisun", "rofapel"], default="qwen25vl",
                     help="with --design: the model the design is measured beside, at the same sizes")
     ap.add_argument("--order", default=None,
-                    help="with --design gogudra, rapisun or rofapel: the mixers of successive layers, repeated (gogudra: "
-                         "gla,gla,lightning,attention; rapisun: " + ",".join(RAPISUN_ORDER) + "; rofapel: "
-                         + ",".join(ROFAPEL_ORDER) + ")")
+                    help="with --design gogudra, rapisun, rofapel or zaposun: the mixers of successive layers, repeated "
+                         "(gogudra: gla,gla,lightning,attention; rapisun: " + ",".join(RAPISUN_ORDER) + "; rofapel: "
+                         + ",".join(ROFAPEL_ORDER) + "; zaposun: " + ",".join(ZAPOSUN_ORDER) + ")")
     ap.add_argument("--loop", default=None, metavar="START,STOP,TIMES",
                     help="with --design rofapel: layers START .. STOP-1 run TIMES times in a row (default: no loop)")
     ap.add_argument("--no-graph", action="store_true", help="do not replay decode steps from a HIP graph")
@@ -360,7 +385,7 @@ def main(argv=None) -> int:
     if args.design and not args.layers:
         args.layers = 8
     if args.order is None:
-        args.order = ",".join({"rapisun": RAPISUN_ORDER, "rofapel": ROFAPEL_ORDER}.get(
+        args.order = ",".join({"rapisun": RAPISUN_ORDER, "rofapel": ROFAPEL_ORDER, "zaposun": ZAPOSUN_ORDER}.get(
             args.design, ("gla", "gla", "lightning", "attention")))
     cfg = Qwen25VLConfig.from_dict(decoder_config(args.layers, args.size))
     t = cfg.text_config
@@ -436,7 +461,7 @@ def main(argv=None) -> int:
         beside = "the Qwen2.5-VL decoder" if args.beside == "qwen25vl" else args.beside
         out = {"metric": f"prefill and decode tok/s, {args.design} beside {beside} "
                          f"({args.size} sizes, {args.layers} layers, {args.dtype})", "unit": "tokens/s",
-               "order": args.order.split(",") if args.design in ("gogudra", "rapisun", "rofapel") else None,
+               "order": args.order.split(",") if args.design in ("gogudra", "rapisun", "rofapel", "zaposun") else None,
                "batch": args.batch, "prompt_tokens": args.prompt_tokens, "data": "synthetic"}
         if args.design == "rofapel" and args.loop:
             out["loop"] = [int(v) for v in args.loop.split(",")]
@@ -448,8 +473,10 @@ def main(argv=None) -> int:
                 return rapisun_config(args.layers, args.size, tuple(args.order.split(",")) if name == args.design
                                       else RAPISUN_ORDER)
             if name == "rofapel":
-                return rofapel_config(args.layers, args.size, tuple(args.order.split(",")),
-                                      loop=[int(v) for v in args.loop.split(",")] if args.loop else None)
+                return rofapel_config(args.layers, args.size, tuple(args.order.split(",")) if name == args.design
+                                      else ROFAPEL_ORDER, loop=[int(v) for v in args.loop.split(",")] if args.loop else None)
+            if name == "zaposun":
+                return zaposun_config(args.layers, args.size, tuple(args.order.split(",")))
             return gogudra_config(args.layers, args.size, tuple(args.order.split(",")) if name == args.design
                                   else ("gla", "gla", "lightning", "attention"))
 

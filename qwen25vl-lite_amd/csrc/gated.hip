@@ -210,7 +210,7 @@ __global__ void group_norm_gate_kernel(const float* __restrict__ x, const float*
   }
 }
 
-// The same with a team of TEAM threads (a wave, or the block) per group, four values at a time, the
+// The same with a team of TEAM threads (16, a wave, or the block) per group, four values at a time, the
 // group's values held in registers between the two passes: span a multiple of 4 and at most
 // TEAM * 4 * GN_VEC.  Blocks of 256 threads; blockIdx.x counts teams over all (token, group) pairs.
 #define GN_VEC 4
@@ -244,7 +244,14 @@ __global__ __launch_bounds__(256) void group_norm_gate_vec_kernel(
       ss += v[j].x * v[j].x + v[j].y * v[j].y + v[j].z * v[j].z + v[j].w * v[j].w;
     }
   }
-  const float total = TEAM == 64 ? wave_sum(ss) : block_sum(ss, red);
+  float total;
+  if (TEAM < 64) {
+    total = ss;
+#pragma unroll
+    for (int o = TEAM / 2; o > 0; o >>= 1) total += __shfl_xor(total, o, QVL_WAVE);
+  } else {
+    total = TEAM == 64 ? wave_sum(ss) : block_sum(ss, red);
+  }
   if (!live) return;
   const float rs = 1.0f / sqrtf(total / (float)span + eps);
   TO* o = out + n * (size_t)C + c0;
@@ -279,14 +286,14 @@ extern "C" int qvl_group_norm_gate(const void* x, const void* w, int wlen, const
                    (!gate || (gate_stride % 4 == 0 && (uintptr_t)gate % (4 * gbytes) == 0));
   if (vec) {
     const long long items = (long long)N * (C / span);
-    const bool wave = span <= 64 * 4 * GN_VEC;
-    const long long blocks = wave ? (items + 3) / 4 : items;
+    const bool wave = span <= 64 * 4 * GN_VEC, narrow = span <= 128;
+    const long long blocks = narrow ? (items + 15) / 16 : (wave ? (items + 3) / 4 : items);
     if (blocks > 0x7fffffffLL) return QVL_ERR_LIMIT;
 #define LAUNCHV(TG, TO, TEAM)                                                                                      \
     hipLaunchKernelGGL((group_norm_gate_vec_kernel<TG, TO, TEAM>), dim3((unsigned)blocks), dim3(256), 0, stream,   \
                        (const float*)x, (const float*)w, wlen, (const TG*)gate, gate_stride, (TO*)out, C, span,    \
                        eps, act, nslabs, slab_stride, items)
-#define BY_TEAM(TG, TO) if (wave) LAUNCHV(TG, TO, 64); else LAUNCHV(TG, TO, 256)
+#define BY_TEAM(TG, TO) if (narrow) LAUNCHV(TG, TO, 16); else if (wave) LAUNCHV(TG, TO, 64); else LAUNCHV(TG, TO, 256)
     if (gate_dtype == 0 && out_dtype == 0) { BY_TEAM(float, float); }
     else if (gate_dtype == 1 && out_dtype == 1) { BY_TEAM(bf16_t, bf16_t); }
     else if (gate_dtype == 0 && out_dtype == 1) { BY_TEAM(float, bf16_t); }

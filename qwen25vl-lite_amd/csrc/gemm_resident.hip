@@ -123,6 +123,10 @@ struct ResidentArgs {
   // tiles is as even as the rounds before it
   int whole_tiles, parts, pairs;
   int gelu;              // EPI_SWIGLU: the activation is the tanh form of gelu
+  // Several products of the same sizes side by side (EPI_STORE, one block a team): product i has the blocks
+  // i * stack_blocks .. and its operands and result lie i strides further on (in elements)
+  int stack_blocks;      // 0: one product
+  long long stack_x, stack_w, stack_o;
 #ifdef QVL_TIMELINE
   unsigned long long* timeline;
 #endif
@@ -153,6 +157,15 @@ __global__ __launch_bounds__(64 * RW) void gemm_resident_kernel(ResidentArgs p) 
   float (*gains)[RK * 32] = MT == 1 ? gains_own : reinterpret_cast<float (*)[RK * 32]>(&red[0][0][0]);  // norm weights of each wave's columns
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, lg = lane >> 4, r = lane & 15;
   const int k_lane = wave * RK * 32 + 8 * lg;  // first K index of this lane within a pass
+  int block = blockIdx.x, blocks = gridDim.x;
+  if (EPI == EPI_STORE && p.stack_blocks > 0) {
+    const int item = block / p.stack_blocks;
+    block -= item * p.stack_blocks;
+    blocks = p.stack_blocks;
+    p.X += item * p.stack_x;
+    p.W += item * p.stack_w;
+    p.out = reinterpret_cast<TO*>(p.out) + item * p.stack_o;
+  }
   STAMP(0);
   // how many of this lane's 32-wide steps of the pass that starts at k0 begin inside K (K is a
   // multiple of 8, as is every lane's first index: a step lies inside K or outside)
@@ -168,7 +181,7 @@ __global__ __launch_bounds__(64 * RW) void gemm_resident_kernel(ResidentArgs p) 
   const rsrc_t slot_buf = buffer_of(p.slot, (unsigned long long)p.M * 4);
   // Workgroups go to the XCDs in turn, so blocks b, b + 8, b + 16, ... share an XCD: consecutive
   // ones of them form a team.
-  int team = blockIdx.x, teams = gridDim.x, m0 = 0;   // m0: this block's first row of X
+  int team = block, teams = blocks, m0 = 0;   // m0: this block's first row of X
   if (p.groups > 1) {   // the grid is a multiple of 8 groups
     const int xcd_turn = blockIdx.x >> 3;
     team = (xcd_turn / p.groups) * 8 + (blockIdx.x & 7);
@@ -590,7 +603,7 @@ extern "C" int qvl_gemm_resident(const void* x, int ldx, const void* h, int ldh,
   ResidentArgs p;
   p.X = (const bf16_t*)x; p.ldx = ldx; p.H = (const float*)h; p.ldh = ldh; p.norm_w = (const float*)norm_w;
   p.eps = eps; p.W = (const bf16_t*)W; p.ldw = ldw; p.bias = (const float*)bias; p.out = out; p.ldo = ldo;
-  p.M = M; p.N = N; p.K = K; p.gelu = gelu;
+  p.M = M; p.N = N; p.K = K; p.gelu = gelu; p.stack_blocks = 0; p.stack_x = p.stack_w = p.stack_o = 0;
 #ifdef QVL_TIMELINE
   p.timeline = timeline_buffer;
 #endif
@@ -624,6 +637,45 @@ extern "C" int qvl_gemm_resident(const void* x, int ldx, const void* h, int ldh,
   return QVL_ERR_DTYPE;
 }
 
+// out[i] = x[i] W[i]^T for `count` products of the same sizes, bfloat16 in, out_dtype out: x [M, K] (rows ldx apart) every
+// x_stride elements, W [N, K] every w_stride, out [M, N] every o_stride.  M at most 32, K for one pass over the
+// weights; every product gets its share of max_blocks (at least one).
+extern "C" int qvl_gemm_resident_stack(const void* x, int ldx, long long x_stride, const void* W, int ldw, long long w_stride,
+                                       void* out, int ldo, long long o_stride, int count, int M, int N, int K, int out_dtype,
+                                       int max_blocks, hipStream_t stream) {
+  if (M <= 0 || N <= 0 || count <= 0) return QVL_OK;
+  if (K <= 0 || K % 8 || ldw % 8 || ldw < K || ldx % 8 || ldx < K || ldo < N || x_stride % 8 || w_stride % 8 || !x || !W || !out ||
+      max_blocks < count)
+    return QVL_ERR_SHAPE;
+  if (M > 32 || !fits_descriptors(M, N, K, ldw, ldx, 0, ldo)) return QVL_ERR_LIMIT;
+  const int share = max_blocks / count;
+  const Plan pl = plan_for(M, K, false, share);
+  if (pl.groups != 1 || !pl.one_pass || pl.mt < 1) return QVL_ERR_LIMIT;
+  ResidentArgs p;
+  p.X = (const bf16_t*)x; p.ldx = ldx; p.H = nullptr; p.ldh = 0; p.norm_w = nullptr; p.eps = 0.f; p.W = (const bf16_t*)W;
+  p.ldw = ldw; p.bias = nullptr; p.out = out; p.ldo = ldo; p.M = M; p.N = N; p.K = K; p.gelu = 0; p.groups = 1;
+#ifdef QVL_TIMELINE
+  p.timeline = nullptr;
+#endif
+  p.cs = nullptr; p.slot = nullptr;
+  p.q_out = nullptr; p.kc = nullptr; p.vc = nullptr; p.nq = p.nkv = p.hd = p.ps = 0; p.pair_tiles = 0;
+  const long long rounds = (N + 16LL * share - 1) / (16LL * share);
+  p.rows = (int)((N + rounds * share - 1) / (rounds * share));
+  p.ntiles = (N + p.rows - 1) / p.rows;
+  p.whole_tiles = p.ntiles; p.parts = 1; p.pairs = 8;
+  p.stack_blocks = share < p.ntiles ? share : p.ntiles;
+  p.stack_x = x_stride; p.stack_w = w_stride; p.stack_o = o_stride;
+  const dim3 grid(p.stack_blocks * count), block(64 * RW);
+#define QVL_STACK(TO)                                                                                                      \
+  if (pl.mt == 1) hipLaunchKernelGGL((gemm_resident_kernel<TO, PRO_PLAIN, EPI_STORE, true, 1>), grid, block, 0, stream, p); \
+  else hipLaunchKernelGGL((gemm_resident_kernel<TO, PRO_PLAIN, EPI_STORE, true, 2>), grid, block, 0, stream, p)
+  if (out_dtype == 0) { QVL_STACK(float); }
+  else if (out_dtype == 1) { QVL_STACK(bf16_t); }
+  else return QVL_ERR_DTYPE;
+#undef QVL_STACK
+  return qvl_launch_status();
+}
+
 // The stacked query | key | value projection of at most 32 tokens with rotation and cache write
 // folded in (EPI_ROPE).  x / h / norm_w / eps as in qvl_gemm_resident.  W: [(nq + 2 nkv) hd, K];
 // bias: float32 [(nq + 2 nkv) hd] or null.  cs: float32 [M, hd / 2, 2], cosine and sine of every
@@ -655,7 +707,7 @@ extern "C" int qvl_gemm_resident_rope(const void* x, int ldx, const void* h, int
   ResidentArgs p;
   p.X = (const bf16_t*)x; p.ldx = ldx; p.H = (const float*)h; p.ldh = ldh; p.norm_w = (const float*)norm_w;
   p.eps = eps; p.W = (const bf16_t*)W; p.ldw = ldw; p.bias = (const float*)bias; p.out = nullptr; p.ldo = 0;
-  p.M = M; p.N = (nq + 2 * nkv) * hd; p.K = K; p.gelu = 0;
+  p.M = M; p.N = (nq + 2 * nkv) * hd; p.K = K; p.gelu = 0; p.stack_blocks = 0; p.stack_x = p.stack_w = p.stack_o = 0;
 #ifdef QVL_TIMELINE
   p.timeline = timeline_buffer;
 #endif

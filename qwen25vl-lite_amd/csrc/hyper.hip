@@ -93,10 +93,15 @@ __device__ __forceinline__ Cols<VEC> ld_addend(const void* y, int dtype, int sla
   if (dtype) return ldc16<VEC>(reinterpret_cast<const bf16_t*>(y) + at);
   const float* p = reinterpret_cast<const float*>(y) + at;
   Cols<VEC> a = ldc<VEC>(p);
-  for (int s = 1; s < slabs; ++s) {
-    const Cols<VEC> b = ldc<VEC>(p + (size_t)s * slab_stride);
+  // eight slabs' loads are on their way together (past the last: slab 0 again, not counted); the sum keeps the order
+  for (int s0 = 1; s0 < slabs; s0 += 8) {
+    Cols<VEC> b[8];
 #pragma unroll
-    for (int k = 0; k < VEC; ++k) a.v[k] += b.v[k];
+    for (int s = 0; s < 8; ++s) b[s] = ldc<VEC>(p + (size_t)(s0 + s < slabs ? s0 + s : 0) * slab_stride);
+#pragma unroll
+    for (int s = 0; s < 8; ++s)
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) a.v[k] += s0 + s < slabs ? b[s].v[k] : 0.f;
   }
   return a;
 }

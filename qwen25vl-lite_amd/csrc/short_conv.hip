@@ -6,8 +6,8 @@
 // of the request's next run and replaced at the end of this one.  x is float32 (the residual, a projection)
 // or bfloat16 (a projection); the result is written in the run's storage type or in float32.
 //
-// Grid (N + R, channel blocks); a thread owns one channel, or four neighbouring ones where 4 divides C.
-// Rows below N are tokens: a token that stands at least taps - 1 tokens into its run reads only x.  The last R rows are requests: the thread of a channel forms the outputs of the
+// Grid (token rows + R, channel blocks); a thread owns one channel, or four neighbouring ones where 4 divides C.
+// The first rows are TOK tokens each: a token that stands at least taps - 1 tokens into its run reads only x.  The last R rows are requests: the thread of a channel forms the outputs of the
 // run's first taps - 1 tokens from the old state and then writes the new one, so nobody else reads or
 // writes that channel of the slot in this launch.
 #include "common.h"
@@ -60,8 +60,9 @@ template <typename TO, int VEC> __device__ __forceinline__ void st_out(TO* p, Ch
   for (int u = 0; u < VEC; ++u) stf<TO>(p + u, a.v[u]);
 }
 
-// MAXT: up to this many taps a token's loads are issued together
-template <typename TX, typename TO, int VEC, int MAXT>
+#define SC_TOKENS 4
+// MAXT: up to this many taps the loads of a row's tokens are issued together, every input once
+template <typename TX, typename TO, int VEC, int MAXT, int TOK>
 __global__ __launch_bounds__(256) void short_conv_kernel(const TX* __restrict__ x, const float* __restrict__ w,
                                                          const float* __restrict__ bias, float* __restrict__ state, const int* __restrict__ cu_q,
                                                          const int* __restrict__ req_slots,
@@ -72,49 +73,69 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const TX* __restrict__ 
   const float* wc = w + c;                      // tap j of channels c ..: wc[j * C]
   const float* bc = bias ? bias + c : nullptr;
   const int keep = taps - 1;
-  if ((int)blockIdx.x < N) {
-    const int t = blockIdx.x;
-    const int i = t - cu_q[token_req[t]];
-    if (i < keep) return;                       // the request's row forms it from the state
+  const int token_rows = (N + TOK - 1) / TOK;
+  if ((int)blockIdx.x < token_rows) {
+    const int t0 = blockIdx.x * TOK;
+    bool mine[TOK];                             // tokens this row forms; the request's row forms the others from the state
+    bool any = false;
+#pragma unroll
+    for (int k = 0; k < TOK; ++k) {
+      const int t = t0 + k < N ? t0 + k : N - 1;
+      mine[k] = t0 + k < N && t - cu_q[token_req[t]] >= keep;
+      any |= mine[k];
+    }
+    if (!any) return;
     if (taps <= MAXT) {
-      // every load is on its way before the first is used: tap j >= taps reads tap taps - 1 again and counts zero
-      Chan<VEC> xv[MAXT];
-      float wv[VEC][MAXT];
+      // every load is on its way before the first is used.  By distance back: weight d is tap keep - d, zero beyond the
+      // taps; an input before the step's first token is never one of a token that is formed here
+      Chan<VEC> xv[TOK + MAXT - 1], wd[MAXT];
 #pragma unroll
-      for (int j = 0; j < MAXT; ++j) {
-        const int jj = j < taps ? j : keep;
-        xv[j] = ld_chan<VEC>(x + (size_t)(t - keep + jj) * xs + c);
-        const Chan<VEC> wj = ld_chan<VEC>(wc + (size_t)jj * C);
-#pragma unroll
-        for (int u = 0; u < VEC; ++u) wv[u][j] = wj.v[u];
+      for (int j = 0; j < TOK + MAXT - 1; ++j) {
+        int t = t0 - (MAXT - 1) + j;
+        t = t < 0 ? 0 : (t < N ? t : N - 1);
+        xv[j] = ld_chan<VEC>(x + (size_t)t * xs + c);
       }
-      Chan<VEC> acc = xv[MAXT - 1];              // x[t]
+#pragma unroll
+      for (int d = 0; d < MAXT; ++d) {
+        wd[d] = ld_chan<VEC>(wc + (size_t)(d <= keep ? keep - d : 0) * C);
+#pragma unroll
+        for (int u = 0; u < VEC; ++u) wd[d].v[u] = d <= keep ? wd[d].v[u] : 0.f;
+      }
+#pragma unroll
+      for (int k = 0; k < TOK; ++k) {
+        if (!mine[k]) continue;
+        Chan<VEC> acc = xv[k + MAXT - 1];        // x[t]
+        if (!plus) {
+#pragma unroll
+          for (int u = 0; u < VEC; ++u) acc.v[u] = 0.f;
+        }
+#pragma unroll
+        for (int d = MAXT - 1; d >= 0; --d)
+#pragma unroll
+          for (int u = 0; u < VEC; ++u) acc.v[u] += wd[d].v[u] * xv[k + MAXT - 1 - d].v[u];
+        st_out<TO, VEC>(out + (size_t)(t0 + k) * C + c, acc, bc, silu);
+      }
+      return;
+    }
+    for (int k = 0; k < TOK; ++k) {
+      if (!mine[k]) continue;
+      const int t = t0 + k;
+      Chan<VEC> acc = ld_chan<VEC>(x + (size_t)t * xs + c);
       if (!plus) {
 #pragma unroll
         for (int u = 0; u < VEC; ++u) acc.v[u] = 0.f;
       }
+      for (int j = 0; j < taps; ++j) {
+        const Chan<VEC> v = ld_chan<VEC>(x + (size_t)(t - keep + j) * xs + c);
+        const Chan<VEC> wj = ld_chan<VEC>(wc + (size_t)j * C);
 #pragma unroll
-      for (int j = 0; j < MAXT; ++j)
-#pragma unroll
-        for (int u = 0; u < VEC; ++u) acc.v[u] += (j < taps ? wv[u][j] : 0.f) * xv[j].v[u];
+        for (int u = 0; u < VEC; ++u) acc.v[u] += wj.v[u] * v.v[u];
+      }
       st_out<TO, VEC>(out + (size_t)t * C + c, acc, bc, silu);
-      return;
     }
-    Chan<VEC> acc = ld_chan<VEC>(x + (size_t)t * xs + c);
-    if (!plus) {
-#pragma unroll
-      for (int u = 0; u < VEC; ++u) acc.v[u] = 0.f;
-    }
-    for (int j = 0; j < taps; ++j) {
-      const Chan<VEC> v = ld_chan<VEC>(x + (size_t)(t - keep + j) * xs + c);
-      const Chan<VEC> wj = ld_chan<VEC>(wc + (size_t)j * C);
-#pragma unroll
-      for (int u = 0; u < VEC; ++u) acc.v[u] += wj.v[u] * v.v[u];
-    }
-    st_out<TO, VEC>(out + (size_t)t * C + c, acc, bc, silu);
     return;
   }
-  const int r = blockIdx.x - N;
+  const int r = blockIdx.x - token_rows;
   const int begin = cu_q[r], n = cu_q[r + 1] - begin;
   if (n <= 0) return;
   float* st = state + (size_t)req_slots[r] * keep * C + c;      // st[k * C]: input number k of the kept ones
@@ -152,13 +173,13 @@ extern "C" int qvl_short_conv(const void* x, int x_dtype, const void* w, const v
   if (R <= 0 || C <= 0 || taps < 1 || !x || !w || !out || !cu_q || !token_req) return QVL_ERR_SHAPE;
   if (taps > 1 && (!state || !req_slots)) return QVL_ERR_SHAPE;
   if (x_stride < C) return QVL_ERR_SHAPE;
-  const long long rows = (long long)N + (taps > 1 ? R : 0);
+  const long long rows = ((long long)N + SC_TOKENS - 1) / SC_TOKENS + (taps > 1 ? R : 0);
   if (rows > 0x7fffffffll || (C + 255) / 256 > 65535) return QVL_ERR_LIMIT;
   const bool vec = C % 4 == 0 && x_stride % 4 == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)w & 15) == 0 && ((uintptr_t)state & 15) == 0 && ((uintptr_t)out & 15) == 0 && ((uintptr_t)bias & 15) == 0;
   const int per_block = vec ? 1024 : 256;
   const dim3 grid((unsigned)rows, (C + per_block - 1) / per_block);
 #define SC_LAUNCH(TX, TO, VEC)                                                                                      \
-  hipLaunchKernelGGL((short_conv_kernel<TX, TO, VEC, 4>), grid, dim3(256), 0, stream, (const TX*)x, (const float*)w,    \
+  hipLaunchKernelGGL((short_conv_kernel<TX, TO, VEC, 4, SC_TOKENS>), grid, dim3(256), 0, stream, (const TX*)x, (const float*)w,    \
                      (const float*)bias, (float*)state, (const int*)cu_q, (const int*)req_slots, (const int*)token_req,  \
                      (TO*)out, N, C, taps, x_stride, plus_input, silu)
 #define SC_BY_VEC(TX, TO) { if (vec) SC_LAUNCH(TX, TO, 4); else SC_LAUNCH(TX, TO, 1); }

@@ -28,7 +28,7 @@ LIBRARIES = [
     # the kernel that joins copies of the residual sum is compiled per number of copies, the selective scan per state
     # size; these are what the tests and the benchmark use
     *[("hyper", {"HC_S": s}) for s in (1, 2, 3, 4, 5)],
-    *[("selective_scan", {"SSM_STATE": n}) for n in (1, 3, 8, 16, 40)],
+    *[("selective_scan", {"SSM_STATE": n}) for n in (1, 3, 8, 16, 35, 40)],
     # the linear-attention kernels are compiled per key size (the sizes the tests and the benchmark
     # use; any other size up to 512 is compiled at its first use)
     *[("linear_attention", {"LA_DIM": d}) for d in (5, 6, 8, 12, 16, 20, 32, 64, 128, 320)],

@@ -78,6 +78,8 @@ def linear_stack(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
                   and x.stride(2) == 1 and x.dtype == weight.dtype, "x [S, M, K] and weight [S, N, K] of one dtype")
     kernels._dev(x, weight)
     out = torch.empty((s, m, weight.shape[1]), dtype=x.dtype, device=x.device)
+    if weight.dtype == torch.bfloat16 and _aligned(x[0]) and x.stride(0) % 8 == 0 and skinny.takes_stack(m, k, weight):
+        return skinny.stack_product(weight, x, out)      # a decode step's few rows: one launch
     for i in range(s):
         if weight.dtype == torch.float32:
             kernels.gemm_f32(x[i], weight[i], out=out[i])

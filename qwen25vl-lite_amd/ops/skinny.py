@@ -16,7 +16,7 @@ import torch
 from .kernels import _check, _fn, _ptr, _stream, dtype_code
 
 __all__ = ["resident_product", "takes_resident", "qkv_rope_product", "takes_qkv_rope", "RESIDENT_ROWS", "resident_norm_k", "resident_two_tile_k", "folds_norm", "ONE_BLOCK_ROWS", "split_product", "takes_split", "prefers_split", "SPLIT_ROWS",
-           "STORE", "RESIDUAL", "SWIGLU", "GEGLU", "GATED"]
+           "takes_stack", "stack_product", "STORE", "RESIDUAL", "SWIGLU", "GEGLU", "GATED"]
 
 RESIDENT_ROWS = 64       # up to here the resident kernel runs
 ONE_TILE_ROWS = 16       # the rows of one column tile of the matrix instruction
@@ -143,6 +143,29 @@ def resident_product(weight: torch.Tensor, *, x: Optional[torch.Tensor] = None, 
               _ptr(norm_weight), float(eps), _ptr(weight), weight.stride(0), _ptr(bias), _ptr(out), out.stride(0),
               m, n, k, dtype_code(odt), epilogue, _compute_units(src.device), _stream()),
            "linear (resident)")
+    return out
+
+
+def takes_stack(m: int, k: int, weight: torch.Tensor) -> bool:
+    """Whether the resident kernel runs a stack of products (``weight [S, N, K]``) of ``m`` rows each in one launch:
+    few rows, an inner size for one pass over the weights, and a compute unit for each product at least."""
+    return (m <= ONE_BLOCK_ROWS and weight.shape[0] <= _compute_units(weight.device) and takes_resident(m, k, weight[0])
+            and k <= (resident_norm_k() if m <= ONE_TILE_ROWS else resident_two_tile_k()))
+
+
+def stack_product(weight: torch.Tensor, x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """``out[i] = x[i] @ weight[i].T`` (``x [S, M, K]``, ``weight [S, N, K]``, both bfloat16; ``out [S, M, N]``) in one launch,
+    the compute units divided among the products."""
+    s, m, k = x.shape
+    n = weight.shape[1]
+    if (not takes_stack(m, k, weight) or weight.shape != (s, n, k) or not weight.is_contiguous() or x.dtype != torch.bfloat16
+            or not _rows_aligned(x[0], 8) or x.stride(0) % 8 or out.shape != (s, m, n) or not out.is_contiguous()):
+        raise ValueError("the resident kernel does not take this stack of products")
+    fn = _fn("gemm_resident", "qvl_gemm_resident_stack",
+             [_c_ptr, _c_int, ctypes.c_longlong, _c_ptr, _c_int, ctypes.c_longlong, _c_ptr, _c_int, ctypes.c_longlong, _c_int,
+              _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr], _build_for(k))
+    _check(fn(_ptr(x), x.stride(1), x.stride(0), _ptr(weight), k, n * k, _ptr(out), n, m * n, s, m, n, k,
+              dtype_code(out.dtype), _compute_units(x.device), _stream()), "linear (resident, a stack of products)")
     return out
 
 
