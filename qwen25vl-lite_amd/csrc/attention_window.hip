@@ -70,11 +70,14 @@ struct WindowArgs {
 // W: waves that share an entry's key blocks (1 or 4).  CT: column tiles of an entry, all carried by the
 // same wave: a key or value fragment that has been fetched is multiplied with each of them, and what a
 // kernel of this kind waits for is its fetches (its keys and values come from L2 for every entry anew).
-template <int W, int CT>
-__global__ __launch_bounds__(256) void attn_window_kernel(WindowArgs a) {
+// TURN: values lie turned in the cache.  Two waves a SIMD is what the registers of a walk allow; told so, the compiler
+// keeps all of a block's key fetches in flight instead of saving registers for waves that cannot come (a walk with the
+// turn behind it: 161 us a 2,048-token prompt without, 106 with).
+template <int W, int CT, bool TURN>
+__attribute__((amdgpu_waves_per_eu(2, 2))) __global__ __launch_bounds__(256) void attn_window_kernel(WindowArgs a) {
   __shared__ float s_m[3][CT][16], s_l[3][CT][16];
   __shared__ __attribute__((aligned(16))) float s_acc[W > 1 ? 3 : 1][W > 1 ? CT * NT : 1][64][4];
-  __shared__ float s_out[TURN_BY_LDS ? (W > 1 ? 1 : 4) : 1][TURN_BY_LDS ? 16 : 1][TURN_BY_LDS ? VD + 1 : 1];
+  __shared__ float s_out[TURN && TURN_BY_LDS ? (W > 1 ? 1 : 4) : 1][TURN && TURN_BY_LDS ? 16 : 1][TURN && TURN_BY_LDS ? VD + 1 : 1];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lg = lane >> 4, r = lane & 15;
   const int entry = W == 1 ? blockIdx.x * 4 + wave : blockIdx.x;
   const int part = W == 1 ? 0 : wave;
@@ -249,7 +252,7 @@ __global__ __launch_bounds__(256) void attn_window_kernel(WindowArgs a) {
     }
     const float inv = 1.0f / l[c];
     bf16_t* o = a.out + ((size_t)token[c] * a.nq + head[c]) * VD;
-    if (a.turn) {
+    if constexpr (TURN) {
       // channel ch of this lane's column meets its partner: in this lane's own registers where half a value is a
       // whole number of 16-channel tiles (or pairs are neighbours), else in the wave's place in LDS
       const float2* tn = a.turn + (size_t)token[c] * (VD / 2);
@@ -346,7 +349,11 @@ extern "C" int qvl_attn_window(const void* q, const void* kc, const void* vc, co
   a.nq = nq; a.nkv = nkv; a.ps = ps; a.window = window; a.keep_first = keep_first; a.scale = scale;
   a.sinks = (const float*)sinks;
   a.chunk = chunk; a.turn = (const float2*)turn; a.turn_pairs = turn_pairs;
-  if (share) hipLaunchKernelGGL((attn_window_kernel<4, 1>), dim3(num_tiles, nkv), dim3(256), 0, stream, a);
-  else hipLaunchKernelGGL((attn_window_kernel<1, WIDE_CT>), dim3((num_tiles + 3) / 4, nkv), dim3(256), 0, stream, a);
+#define LAUNCH(TURN)                                                                                                   \
+  if (share) hipLaunchKernelGGL((attn_window_kernel<4, 1, TURN>), dim3(num_tiles, nkv), dim3(256), 0, stream, a);      \
+  else hipLaunchKernelGGL((attn_window_kernel<1, WIDE_CT, TURN>), dim3((num_tiles + 3) / 4, nkv), dim3(256), 0, stream, a)
+  if (turn) { LAUNCH(true); }
+  else { LAUNCH(false); }
+#undef LAUNCH
   return qvl_launch_status();
 }

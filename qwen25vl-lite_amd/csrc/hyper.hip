@@ -1,7 +1,7 @@
 // A residual stream of several copies that every sublayer mixes anew (hyper-connections), and the norm of what the
 // next sublayer reads.  One pass over a token's row:
 //   y   = the pending addend, or factor * (rms(y1) g1 + rms(y2) g2) of two of them (each normed over the row)
-//   x_t = sum_s mix[s, t] x_s + out[t] y          all copies at once from the old ones (skipped without `mix`)
+//   x_t = sum_s mix[s, t] x_s + out[t] y          every copy from the copies as they were (skipped without `mix`)
 //   u   = sum_t read[t] x_t                       (`read` null: the plain sum of the copies)
 //   h   = norm(u): every one of `groups` consecutive parts of the row divided by its own root mean square
 //         (eps inside the root), times w

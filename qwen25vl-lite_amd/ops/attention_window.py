@@ -19,11 +19,11 @@ from .kernels import _check, _fn, _need, _ptr, _stream
 __all__ = ["try_attention", "supports"]
 
 _c_int, _c_float, _c_ptr = ctypes.c_int, ctypes.c_float, ctypes.c_void_p
-# below this many (tile, key/value head) pairs per compute unit the four waves of a block share a tile.  A wave that
-# walks a tile's keys alone waits for each of its fetches, and the longest walk decides while the tiles are few
-# (measured on 256 units, heads of 128, us alone / shared: 2,048 tokens in chunks of 1,024 169 / 109, windows of 1,024
-# 189 / 142; 4,096 tokens 275 / 201 and 349 / 294; 16,384 tokens 1,255 / 1,202)
-SHARE_BELOW_PER_CU = 32
+# below this many (tile, key/value head) pairs per compute unit the four waves of a block share a tile: the longest walk
+# decides while the tiles are few (measured on 256 units, heads of 128, us a wave alone / shared: 1,792 pairs in windows
+# or chunks of 1,024 97 / 62, 2,048 pairs 101 / 86; 3,584 pairs 124 / 141 in windows, 106 / 112 in chunks; 7,168 pairs
+# 238 / 297)
+SHARE_BELOW_PER_CU = 9
 
 
 def supports(head_dim: int, value_dim: int, page_size: int, dtype: torch.dtype) -> bool:

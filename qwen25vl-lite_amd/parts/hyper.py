@@ -1,8 +1,8 @@
 """A layer over several copies of the residual sum that every sublayer mixes anew (hyper-connections).
 
 With copies ``x_1 .. x_s`` (all equal to the embedding's output at the start) a sublayer reads
-``u = sum_s in[s] x_s``, and with its result ``y`` every copy becomes ``x_t <- sum_s mix[s, t] x_s + out[t] y``, all
-at once from the old ones.  What a sublayer gave stays pending, with the weights by which it joins, until the kernel
+``u = sum_s in[s] x_s``, and with its result ``y`` copy t becomes ``sum_s mix[s, t] x_s + out[t] y``, the ``x_s`` being
+the copies as the sublayer found them.  What a sublayer gave stays pending, with the weights by which it joins, until the kernel
 of the next norm in line joins it, forms the next sublayer's ``u`` and norms it in one pass over the copies.
 """
 

@@ -176,7 +176,7 @@ def _copies_case(n, s, width, groups, pending, seed, equal):
 @pytest.mark.parametrize("pending", [None, "float32", "bfloat16", "slabs", "mean"])
 @pytest.mark.parametrize("equal", [False, True])
 def test_copies_joined_read_and_normed_in_one_pass(s, width, groups, pending, equal):
-    """All copies at once from the old ones; the norm in parts of the row; chosen rows of the copies' sum."""
+    """Every copy from the copies as they were; the norm in parts of the row; chosen rows of the copies' sum."""
     from qwen25vl_lite_amd.ops.hyper import join_norm
     t, h, copies, w, y, new, t64 = _copies_case(9, s, width, groups, pending, s + width, equal)
     join = None if pending is None else (t["a.mix"].cuda(), t["a.out"].cuda())
