@@ -175,6 +175,7 @@ extern "C" int qvl_tanh(const void* x, void* out, long long total, int out_dtype
 // ---------------------------------------------------------------------------------------
 // Norm over groups of `span` consecutive channels, then a gate:
 //   y = x / sqrt(mean_group(x^2) + eps) * w[c % wlen] * act(gate[n, c])
+// (gate_first: x stands for x * act(gate[n, c]) and nothing is multiplied behind the norm)
 // x float32 [N, C] (C a multiple of span), or `nslabs` such arrays `slab_stride` apart whose sum, taken
 // in slab order, is x; gate is read from rows of `gate_stride` values starting at its own pointer;
 // act: 0 no gate, 1 sigmoid, 2 silu.  One block per (group, token).
@@ -182,15 +183,21 @@ extern "C" int qvl_tanh(const void* x, void* out, long long total, int out_dtype
 template <typename TG, typename TO>
 __global__ void group_norm_gate_kernel(const float* __restrict__ x, const float* __restrict__ w, int wlen,
                                        const TG* __restrict__ gate, long long gate_stride, TO* __restrict__ out,
-                                       int C, int span, float eps, int act, int nslabs, long long slab_stride) {
+                                       int C, int span, float eps, int act, int gate_first, int nslabs,
+                                       long long slab_stride) {
   __shared__ float red[17];
   const size_t n = blockIdx.y;
   const int c0 = blockIdx.x * span;
   const float* xr = x + n * (size_t)C + c0;
+  const TG* gr = gate ? gate + n * (size_t)gate_stride + c0 : nullptr;
+  auto act_at = [&](int i) {
+    const float g = ldf<TG>(gr + i);
+    return act == 1 ? sigmoid_f(g) : g * sigmoid_f(g);
+  };
   auto x_at = [&](int i) {
     float v = xr[i];
     for (int s = 1; s < nslabs; ++s) v += xr[(size_t)s * slab_stride + i];
-    return v;
+    return act && gate_first ? v * act_at(i) : v;
   };
   float ss = 0.f;
   for (int i = threadIdx.x; i < span; i += blockDim.x) {
@@ -199,13 +206,9 @@ __global__ void group_norm_gate_kernel(const float* __restrict__ x, const float*
   }
   const float rs = 1.0f / sqrtf(block_sum(ss, red) / (float)span + eps);
   TO* o = out + n * (size_t)C + c0;
-  const TG* gr = gate ? gate + n * (size_t)gate_stride + c0 : nullptr;
   for (int i = threadIdx.x; i < span; i += blockDim.x) {
     float y = (x_at(i) * rs) * w[(c0 + i) % wlen];
-    if (act) {
-      const float g = ldf<TG>(gr + i);
-      y *= act == 1 ? sigmoid_f(g) : g * sigmoid_f(g);
-    }
+    if (act && !gate_first) y *= act_at(i);
     stf<TO>(o + i, y);
   }
 }
@@ -218,7 +221,7 @@ __global__ void group_norm_gate_kernel(const float* __restrict__ x, const float*
 template <typename TG, typename TO, int TEAM>
 __global__ __launch_bounds__(256) void group_norm_gate_vec_kernel(
     const float* __restrict__ x, const float* __restrict__ w, int wlen, const TG* __restrict__ gate,
-    long long gate_stride, TO* __restrict__ out, int C, int span, float eps, int act, int nslabs,
+    long long gate_stride, TO* __restrict__ out, int C, int span, float eps, int act, int gate_first, int nslabs,
     long long slab_stride, long long items) {
   __shared__ float red[17];
   const int team = threadIdx.x / TEAM, lane = threadIdx.x % TEAM;
@@ -228,6 +231,13 @@ __global__ __launch_bounds__(256) void group_norm_gate_vec_kernel(
   const size_t n = live ? (size_t)(item / groups) : 0;
   const int c0 = live ? (int)(item % groups) * span : 0;
   const float* xr = x + n * (size_t)C + c0;
+  const TG* gr = gate ? gate + n * (size_t)gate_stride + c0 : nullptr;
+  auto gated = [&](float4 y, int i) {
+    const float4 g = ldv4<TG>(gr + 4 * i);
+    if (act == 1) { y.x *= sigmoid_f(g.x); y.y *= sigmoid_f(g.y); y.z *= sigmoid_f(g.z); y.w *= sigmoid_f(g.w); }
+    else { y.x *= g.x * sigmoid_f(g.x); y.y *= g.y * sigmoid_f(g.y); y.z *= g.z * sigmoid_f(g.z); y.w *= g.w * sigmoid_f(g.w); }
+    return y;
+  };
   const int nvec = span >> 2;
   float4 v[GN_VEC];
   float ss = 0.f;
@@ -241,6 +251,7 @@ __global__ __launch_bounds__(256) void group_norm_gate_vec_kernel(
         const float4 a = ldv4<float>(xr + (size_t)s * slab_stride + 4 * i);
         v[j].x += a.x; v[j].y += a.y; v[j].z += a.z; v[j].w += a.w;
       }
+      if (act && gate_first) v[j] = gated(v[j], i);
       ss += v[j].x * v[j].x + v[j].y * v[j].y + v[j].z * v[j].z + v[j].w * v[j].w;
     }
   }
@@ -255,7 +266,6 @@ __global__ __launch_bounds__(256) void group_norm_gate_vec_kernel(
   if (!live) return;
   const float rs = 1.0f / sqrtf(total / (float)span + eps);
   TO* o = out + n * (size_t)C + c0;
-  const TG* gr = gate ? gate + n * (size_t)gate_stride + c0 : nullptr;
 #pragma unroll
   for (int j = 0; j < GN_VEC; ++j) {
     const int i = lane + TEAM * j;
@@ -263,11 +273,7 @@ __global__ __launch_bounds__(256) void group_norm_gate_vec_kernel(
       const int wc = (c0 + 4 * i) % wlen;       // wlen is a multiple of 4 here, so the four stay in one period
       const float4 ww = ldv4<float>(w + wc);
       float4 y{(v[j].x * rs) * ww.x, (v[j].y * rs) * ww.y, (v[j].z * rs) * ww.z, (v[j].w * rs) * ww.w};
-      if (act) {
-        const float4 g = ldv4<TG>(gr + 4 * i);
-        if (act == 1) { y.x *= sigmoid_f(g.x); y.y *= sigmoid_f(g.y); y.z *= sigmoid_f(g.z); y.w *= sigmoid_f(g.w); }
-        else { y.x *= g.x * sigmoid_f(g.x); y.y *= g.y * sigmoid_f(g.y); y.z *= g.z * sigmoid_f(g.z); y.w *= g.w * sigmoid_f(g.w); }
-      }
+      if (act && !gate_first) y = gated(y, i);
       stv4<TO>(o + 4 * i, y);
     }
   }
@@ -275,7 +281,7 @@ __global__ __launch_bounds__(256) void group_norm_gate_vec_kernel(
 
 extern "C" int qvl_group_norm_gate(const void* x, const void* w, int wlen, const void* gate, long long gate_stride,
                                    int gate_dtype, void* out, int out_dtype, int N, int C, int span, float eps, int act,
-                                   int nslabs, long long slab_stride, hipStream_t stream) {
+                                   int gate_first, int nslabs, long long slab_stride, hipStream_t stream) {
   if (N <= 0 || C <= 0) return QVL_OK;
   if (span <= 0 || C % span || wlen <= 0 || (act && !gate) || act < 0 || act > 2 || nslabs < 1) return QVL_ERR_SHAPE;
   if (C / span > 65535 * 16) return QVL_ERR_LIMIT;
@@ -292,7 +298,7 @@ extern "C" int qvl_group_norm_gate(const void* x, const void* w, int wlen, const
 #define LAUNCHV(TG, TO, TEAM)                                                                                      \
     hipLaunchKernelGGL((group_norm_gate_vec_kernel<TG, TO, TEAM>), dim3((unsigned)blocks), dim3(256), 0, stream,   \
                        (const float*)x, (const float*)w, wlen, (const TG*)gate, gate_stride, (TO*)out, C, span,    \
-                       eps, act, nslabs, slab_stride, items)
+                       eps, act, gate_first, nslabs, slab_stride, items)
 #define BY_TEAM(TG, TO) if (narrow) LAUNCHV(TG, TO, 16); else if (wave) LAUNCHV(TG, TO, 64); else LAUNCHV(TG, TO, 256)
     if (gate_dtype == 0 && out_dtype == 0) { BY_TEAM(float, float); }
     else if (gate_dtype == 1 && out_dtype == 1) { BY_TEAM(bf16_t, bf16_t); }
@@ -309,7 +315,7 @@ extern "C" int qvl_group_norm_gate(const void* x, const void* w, int wlen, const
     hipLaunchKernelGGL((group_norm_gate_kernel<TG, TO>), dim3(C / span, rows), dim3(threads), 0, stream,          \
                        (const float*)x + (size_t)at * C, (const float*)w, wlen,                                   \
                        gate ? (const TG*)gate + (size_t)at * gate_stride : (const TG*)nullptr, gate_stride,       \
-                       (TO*)out + (size_t)at * C, C, span, eps, act, nslabs, slab_stride);                        \
+                       (TO*)out + (size_t)at * C, C, span, eps, act, gate_first, nslabs, slab_stride);                        \
   }
   if (gate_dtype == 0 && out_dtype == 0) { LAUNCH(float, float) }
   else if (gate_dtype == 1 && out_dtype == 1) { LAUNCH(bf16_t, bf16_t) }

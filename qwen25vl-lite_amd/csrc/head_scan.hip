@@ -1,0 +1,639 @@
+// Recurrences over outer products with one decay per head and token, a_t = exp(A_h softplus(raw_t + bias_h)):
+//   plain   S <- a S + step k v^T,                              o = S^T q (+ D v)      (step = the softplus)
+//   delta   S <- a S;  u = beta (v - S^T k);  S <- S + k u^T;   o = S^T q              (beta = sigmoid of another raw column)
+// S is [HS_DIM, vdim] float32 per (request slot, head).  q and k belong to groups of heads (head h reads group
+// h / (H / G)) and may be made unit vectors first, x / sqrt(sum x^2 + unit_eps); q is scaled.  q, k and v are columns of
+// float32 or bfloat16 rows; raw columns, decays, step sizes, unit lengths, states and outputs are float32.
+// Compiled per key size (-DHS_DIM=...).
+//
+// Runs of few tokens: hs_scan_kernel walks a request's tokens in order.  A block of four waves owns 64 value channels of
+// one head; lane = value channel, each wave keeps a quarter of the rows of S in registers.
+//
+// Long runs are cut into chunks of 64 tokens.  With L_ij = a_(j+1) ... a_i (i >= j, from logarithms summed in float64)
+// and S' the state before a chunk
+//   delta: (I + strict lower(diag(beta) L o K K^T)) [Wv | Wk] = diag(beta) [V | diag(L_i0) K],   U = Wv - Wk S'
+//   plain: U = diag(step) V
+//   O = (L o Q K^T) U + diag(L_i0) Q S',     S_end = L_n0 S' + sum_j L_nj k_j u_j^T
+// (L_i0: from the chunk's start up to i.)  Everything but the carry of S runs over chunks side by side, the products
+// through v_mfma_f32_16x16x4_f32 (float32 operands, float32 sums):
+//   hs_prep    sums of logarithms and gates per (chunk, head)
+//   hs_score   Q K^T (and K K^T) per (chunk, group), unit lengths folded in
+//   hs_solve   [Wv | Wk] per (chunk, head), a triangular system in blocks of 16 rows        (delta)
+//   hs_carry   the states, chunk after chunk; a block per (request, head, 16 value channels); leaves S' and U of every chunk
+//   hs_out     O per (chunk, head)
+//
+// Matrix fragments.  Lane l of a wave stands for row (or column) l % 16 and the four inner indices 4 (l / 16) .. + 3 of a
+// block of 16: instruction j of four takes inner index 4 (l / 16) + j of both operands.  A result's lane holds rows
+// 4 (l / 16) .. + 3 of column l % 16, which is the right operand's layout with rows as the inner index, so results
+// are multiplied again without moving.  U and S' lie in memory in that layout: [.., block of 16 rows, lane, 4].
+#include "common.h"
+
+#ifndef HS_DIM
+#define HS_DIM 64
+#endif
+#if HS_DIM < 1 || HS_DIM > 512
+#error "key sizes 1 to 512"
+#endif
+#define HS_ROWS ((HS_DIM + 3) / 4)              // rows of S a wave keeps in hs_scan_kernel
+#define HS_TB (HS_DIM > 256 ? 2 : (HS_DIM > 128 ? 4 : 8))
+#define HS_CHUNK 64
+#define HS_KB ((HS_DIM + 15) / 16)              // blocks of 16 key channels
+#define HS_DIMP (HS_KB * 16)
+#define HS_LD (HS_DIMP + 4)                     // a row of staged keys: columns read down a row block hit different banks
+#define HS_CHUNKED (HS_DIMP <= 256)
+
+struct HeadScan {
+  const void* x;             // rows of x_stride values of TX
+  long long x_stride;
+  int q_off, k_off, v_off;
+  const float* raw;          // rows of raw_stride values: step inputs from a_off, beta inputs from b_off
+  long long raw_stride;
+  int a_off, b_off;
+  const float* bias;         // [H]
+  const float* a_neg;        // [H], -exp(A_log)
+  const float* skip;         // [H] or null: D
+  float q_scale, unit_eps;   // unit_eps < 0: q and k are taken as they are
+  float* state;              // [slots, H, HS_DIM, vdim]
+  const int* bounds;         // [runs + 1] tokens of a run (or chunk)
+  const int* row_of;         // [runs] a request's slot
+  float* out;                // [N, H * vdim]
+  int H, G, vdim;
+  // chunks
+  const int* req_first;      // [R + 1] a request's chunks
+  double* lsum;              // [chunks, H, 64]: sum of the decays' logarithms from the chunk's start, token included
+  float* gate;               // [chunks, H, 64]: beta or step
+  float* qk;                 // [chunks, G, 64, 64]
+  float* kk;                 // [chunks, G, 64, 64]
+  float* unit;               // [chunks, G, 2, 64]: factors on q (its scale included) and k
+  float* wk;                 // [chunks, H, 64, HS_DIMP]
+  float* u;                  // [chunks, H, vtiles, 4, 64, 4]
+  float* s0;                 // [chunks, H, vtiles, HS_KB, 64, 4]
+};
+
+__device__ __forceinline__ float hs_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float hs_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+// ---------------------------------------------------------------------------------------
+// few tokens: one after the other
+// ---------------------------------------------------------------------------------------
+template <typename TX, bool DELTA>
+__global__ __launch_bounds__(256) void hs_scan_kernel(HeadScan a) {
+  __shared__ float qs[HS_TB][4 * HS_ROWS];
+  __shared__ float ks[HS_TB][4 * HS_ROWS];
+  __shared__ float fq[HS_TB], fk[HS_TB], dec[HS_TB], gate[HS_TB];
+  __shared__ float seen[2][4][64];              // a token's S^T k by wave
+  __shared__ float po[HS_TB][4][64];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int head = blockIdx.y, run = blockIdx.z, grp = head / (a.H / a.G);
+  const int vcol = blockIdx.x * 64 + lane;
+  const bool live = vcol < a.vdim;
+  const int begin = a.bounds[run], end = a.bounds[run + 1];
+  if (begin >= end) return;
+  const TX* x = reinterpret_cast<const TX*>(a.x);
+  const int d0 = wave * HS_ROWS;
+  float* srow = a.state + (((size_t)a.row_of[run] * a.H + head) * HS_DIM + d0) * a.vdim + (live ? vcol : 0);
+  float S[HS_ROWS];
+#pragma unroll
+  for (int i = 0; i < HS_ROWS; ++i) S[i] = live && d0 + i < HS_DIM ? srow[(size_t)i * a.vdim] : 0.f;
+  const float bias = a.bias[head], a_neg = a.a_neg[head], skip = a.skip ? a.skip[head] : 0.f;
+
+  for (int t0 = begin; t0 < end; t0 += HS_TB) {
+    const int nt = end - t0 < HS_TB ? end - t0 : HS_TB;
+    for (int idx = tid; idx < nt * 4 * HS_ROWS; idx += 256) {
+      const int t = idx / (4 * HS_ROWS), d = idx % (4 * HS_ROWS);
+      const TX* row = x + (size_t)(t0 + t) * a.x_stride + (size_t)grp * HS_DIM + d;
+      qs[t][d] = d < HS_DIM ? ldf<TX>(row + a.q_off) : 0.f;
+      ks[t][d] = d < HS_DIM ? ldf<TX>(row + a.k_off) : 0.f;
+    }
+    float vt[HS_TB];
+#pragma unroll
+    for (int t = 0; t < HS_TB; ++t)
+      vt[t] = live && t < nt ? ldf<TX>(x + (size_t)(t0 + t) * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol) : 0.f;
+    if (tid < nt) {
+      const float* r = a.raw + (size_t)(t0 + tid) * a.raw_stride;
+      const float step = hs_softplus(r[a.a_off + head] + bias);
+      dec[tid] = expf(a_neg * step);
+      gate[tid] = DELTA ? hs_sigmoid(r[a.b_off + head]) : step;
+    }
+    __syncthreads();
+    for (int t = wave; t < nt; t += 4) {        // a wave's token: its factors on q and k
+      float sq = 0.f, sk = 0.f;
+      if (a.unit_eps >= 0.f) {
+        for (int d = lane; d < HS_DIM; d += 64) {
+          sq += qs[t][d] * qs[t][d];
+          sk += ks[t][d] * ks[t][d];
+        }
+        sq = wave_sum(sq);
+        sk = wave_sum(sk);
+      }
+      if (lane == 0) {
+        fq[t] = a.unit_eps >= 0.f ? a.q_scale / sqrtf(sq + a.unit_eps) : a.q_scale;
+        fk[t] = a.unit_eps >= 0.f ? 1.0f / sqrtf(sk + a.unit_eps) : 1.0f;
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < HS_TB; ++t) {
+      if (t < nt) {                             // the same for the whole block
+        const float g = dec[t], kf = fk[t];
+        float w;                                // what the key writes, its factor included
+        if (DELTA) {
+          float acc = 0.f;
+#pragma unroll
+          for (int i = 0; i < HS_ROWS; ++i) {
+            S[i] *= g;
+            acc += S[i] * ks[t][d0 + i];
+          }
+          seen[t & 1][wave][lane] = acc;
+          __syncthreads();
+          const float sum = (seen[t & 1][0][lane] + seen[t & 1][1][lane]) + (seen[t & 1][2][lane] + seen[t & 1][3][lane]);
+          w = gate[t] * (vt[t] - kf * sum) * kf;
+        } else {
+          w = gate[t] * vt[t] * kf;
+        }
+        float acc = 0.f;
+#pragma unroll
+        for (int i = 0; i < HS_ROWS; ++i) {
+          S[i] = (DELTA ? S[i] : g * S[i]) + ks[t][d0 + i] * w;
+          acc += S[i] * qs[t][d0 + i];
+        }
+        po[t][wave][lane] = acc;
+      }
+    }
+    __syncthreads();
+    for (int t = wave; t < nt; t += 4) {        // vt[t] with t not known at compile time: the value is read again
+      if (live) {
+        float o = ((po[t][0][lane] + po[t][1][lane]) + (po[t][2][lane] + po[t][3][lane])) * fq[t];
+        if (a.skip) o += skip * ldf<TX>(x + (size_t)(t0 + t) * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol);
+        a.out[((size_t)(t0 + t) * a.H + head) * a.vdim + vcol] = o;
+      }
+    }
+    __syncthreads();
+  }
+  if (live) {
+#pragma unroll
+    for (int i = 0; i < HS_ROWS; ++i)
+      if (d0 + i < HS_DIM) srow[(size_t)i * a.vdim] = S[i];
+  }
+}
+
+#if HS_CHUNKED
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+// acc += A B over one block of 16 inner indices
+__device__ __forceinline__ f32x4 mma16(const f32x4 p, const f32x4 q, f32x4 acc) {
+#pragma unroll
+  for (int j = 0; j < 4; ++j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(p[j], q[j], acc, 0, 0, 0);
+  return acc;
+}
+
+// ---------------------------------------------------------------------------------------
+// a wave per (chunk, head), a lane per token
+// ---------------------------------------------------------------------------------------
+template <bool DELTA>
+__global__ __launch_bounds__(256) void hs_prep_kernel(HeadScan a) {
+  const int c = blockIdx.x, head = blockIdx.y * 4 + (threadIdx.x >> 6), t = threadIdx.x & 63;
+  if (head >= a.H) return;
+  const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
+  double l = 0.0;
+  float g = 0.f;
+  if (t < n) {
+    const float* r = a.raw + (size_t)(begin + t) * a.raw_stride;
+    const float step = hs_softplus(r[a.a_off + head] + a.bias[head]);
+    l = (double)(a.a_neg[head] * step);
+    g = DELTA ? hs_sigmoid(r[a.b_off + head]) : step;
+  }
+#pragma unroll
+  for (int o = 1; o < 64; o <<= 1) {
+    const double up = __shfl_up(l, o, 64);
+    if (t >= o) l += up;
+  }
+  const size_t at = ((size_t)c * a.H + head) * HS_CHUNK + t;
+  a.lsum[at] = l;                               // tokens past the chunk's end keep the last sum
+  a.gate[at] = g;
+}
+
+// a row of 16 key blocks from global memory, four channels from d on (zeros past HS_DIM)
+template <typename TX> __device__ __forceinline__ f32x4 ld_keys(const TX* row, int d) {
+  f32x4 v;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v[j] = d + j < HS_DIM ? ldf<TX>(row + d + j) : 0.f;
+  return v;
+}
+
+// ---------------------------------------------------------------------------------------
+// Q K^T and K K^T of a (chunk, group), lower triangle's tiles; factors of the unit lengths folded in
+// ---------------------------------------------------------------------------------------
+template <typename TX, bool DELTA>
+__global__ __launch_bounds__(256) void hs_score_kernel(HeadScan a) {
+  __shared__ __attribute__((aligned(16))) float q[HS_CHUNK * HS_LD], k[HS_CHUNK * HS_LD];
+  __shared__ float f[2][HS_CHUNK];
+  const int c = blockIdx.x, grp = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
+  const TX* x = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride + (size_t)grp * HS_DIM;
+  for (int idx = tid; idx < HS_CHUNK * (HS_DIMP / 4); idx += 256) {
+    const int t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
+    f32x4 qv = {0.f, 0.f, 0.f, 0.f}, kv = qv;
+    if (t < n) {
+      qv = ld_keys<TX>(x + (size_t)t * a.x_stride + a.q_off, d);
+      kv = ld_keys<TX>(x + (size_t)t * a.x_stride + a.k_off, d);
+    }
+    *reinterpret_cast<f32x4*>(q + t * HS_LD + d) = qv;
+    *reinterpret_cast<f32x4*>(k + t * HS_LD + d) = kv;
+  }
+  __syncthreads();
+  {                                             // four threads a token
+    const int t = tid >> 2, part = tid & 3;
+    float sq = 0.f, sk = 0.f;
+    if (a.unit_eps >= 0.f) {
+      for (int d = part * 4; d < HS_DIMP; d += 16) {
+        const f32x4 qv = *reinterpret_cast<const f32x4*>(q + t * HS_LD + d), kv = *reinterpret_cast<const f32x4*>(k + t * HS_LD + d);
+        sq += qv[0] * qv[0] + qv[1] * qv[1] + qv[2] * qv[2] + qv[3] * qv[3];
+        sk += kv[0] * kv[0] + kv[1] * kv[1] + kv[2] * kv[2] + kv[3] * kv[3];
+      }
+      sq += __shfl_xor(sq, 1, 64); sq += __shfl_xor(sq, 2, 64);
+      sk += __shfl_xor(sk, 1, 64); sk += __shfl_xor(sk, 2, 64);
+    }
+    if (part == 0) {
+      f[0][t] = a.unit_eps >= 0.f ? a.q_scale / sqrtf(sq + a.unit_eps) : a.q_scale;
+      f[1][t] = a.unit_eps >= 0.f ? 1.0f / sqrtf(sk + a.unit_eps) : 1.0f;
+    }
+  }
+  __syncthreads();
+  if (tid < 2 * HS_CHUNK) a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + tid] = f[tid >> 6][tid & 63];
+  const int col = lane & 15, lg = lane >> 4;
+  const size_t base = ((size_t)c * a.G + grp) * HS_CHUNK * HS_CHUNK;
+  // ten tiles on or below the diagonal: tile number i is (row, column) of the list, shared among the waves
+  for (int i = wave; i < 10; i += 4) {
+    const int rt = i < 1 ? 0 : (i < 3 ? 1 : (i < 6 ? 2 : 3)), ct = i - rt * (rt + 1) / 2;
+    f32x4 s = {0.f, 0.f, 0.f, 0.f}, w = s;
+#pragma unroll 4
+    for (int b = 0; b < HS_KB; ++b) {
+      const f32x4 kb = *reinterpret_cast<const f32x4*>(k + (ct * 16 + col) * HS_LD + b * 16 + 4 * lg);
+      s = mma16(*reinterpret_cast<const f32x4*>(q + (rt * 16 + col) * HS_LD + b * 16 + 4 * lg), kb, s);
+      if (DELTA) w = mma16(*reinterpret_cast<const f32x4*>(k + (rt * 16 + col) * HS_LD + b * 16 + 4 * lg), kb, w);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = rt * 16 + 4 * lg + r;
+      const size_t at = base + (size_t)row * HS_CHUNK + ct * 16 + col;
+      a.qk[at] = s[r] * f[0][row] * f[1][ct * 16 + col];
+      if (DELTA) a.kk[at] = w[r] * f[1][row] * f[1][ct * 16 + col];
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// [Wv | Wk] of a (chunk, head): a wave owns 16 columns of the right side at a time
+// ---------------------------------------------------------------------------------------
+template <typename TX>
+__global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
+  __shared__ __attribute__((aligned(16))) float A[HS_CHUNK][HS_CHUNK + 4];   // strictly below the diagonal
+  __shared__ __attribute__((aligned(16))) float T[4][16][20];                // inverses of the diagonal blocks
+  __shared__ float rv[HS_CHUNK], rk[HS_CHUNK];                               // factors on the rows of V and K
+  const int c = blockIdx.x, head = blockIdx.y, grp = head / (a.H / a.G);
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, lg = lane >> 4;
+  const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
+  const size_t ch = (size_t)c * a.H + head;
+  const double* ls = a.lsum + ch * HS_CHUNK;
+  const float* beta = a.gate + ch * HS_CHUNK;
+  const float* kk = a.kk + ((size_t)c * a.G + grp) * HS_CHUNK * HS_CHUNK;
+  for (int idx = tid; idx < HS_CHUNK * HS_CHUNK; idx += 256) {
+    const int i = idx >> 6, j = idx & 63;
+    A[i][j] = j < i ? beta[i] * expf((float)(ls[i] - ls[j])) * kk[idx] : 0.f;
+  }
+  if (tid < HS_CHUNK) {
+    rv[tid] = beta[tid];
+    rk[tid] = beta[tid] * expf((float)ls[tid]) * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + HS_CHUNK + tid];
+  }
+  __syncthreads();
+  if (lane < 16) {                              // wave w inverts diagonal block w, a lane per column
+    float xcol[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == lane ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < i; ++j) v -= A[wave * 16 + i][wave * 16 + j] * xcol[j];
+      xcol[i] = v;
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) T[wave][i][lane] = xcol[i];
+  }
+  __syncthreads();
+  f32x4 inv[4], low[6];                         // low[i (i - 1) / 2 + j] = -A's block (i, j)
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    inv[i] = *reinterpret_cast<const f32x4*>(&T[i][col][4 * lg]);
+#pragma unroll
+    for (int j = 0; j < i; ++j) low[i * (i - 1) / 2 + j] = -*reinterpret_cast<const f32x4*>(&A[i * 16 + col][j * 16 + 4 * lg]);
+  }
+  const TX* x = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride;
+  const int vtiles = (a.vdim + 15) / 16;
+  for (int tile = wave; tile < vtiles + HS_KB; tile += 4) {
+    const bool values = tile < vtiles;
+    const int cc = (values ? tile : tile - vtiles) * 16 + col;
+    const bool in = values ? cc < a.vdim : cc < HS_DIM;
+    const TX* src = x + (values ? a.v_off + (size_t)head * a.vdim : a.k_off + (size_t)grp * HS_DIM) + (in ? cc : 0);
+    f32x4 y[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = i * 16 + 4 * lg + r;
+        y[i][r] = in && t < n ? ldf<TX>(src + (size_t)t * a.x_stride) : 0.f;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) y[i][r] *= values ? rv[i * 16 + 4 * lg + r] : rk[i * 16 + 4 * lg + r];
+#pragma unroll
+      for (int j = 0; j < i; ++j) y[i] = mma16(low[i * (i - 1) / 2 + j], y[j], y[i]);
+      y[i] = mma16(inv[i], y[i], f32x4{0.f, 0.f, 0.f, 0.f});
+    }
+    if (values) {
+      float* dst = a.u + ((ch * vtiles + tile) * 4 * 64 + lane) * 4;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) *reinterpret_cast<f32x4*>(dst + i * 256) = y[i];
+    } else {
+      float* dst = a.wk + ch * HS_CHUNK * HS_DIMP + cc;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) dst[(size_t)(i * 16 + 4 * lg + r) * HS_DIMP] = y[i][r];
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// The states from chunk to chunk: a block per (16 value channels, head, request)
+// ---------------------------------------------------------------------------------------
+#define HS_MT ((HS_KB + 3) / 4)                 // row blocks of S a wave keeps: wave w has blocks w, w + 4, ...
+
+template <typename TX, bool DELTA>
+__global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
+  __shared__ __attribute__((aligned(16))) float k[HS_CHUNK * HS_LD];   // the chunk's keys
+  __shared__ f32x4 s[HS_KB * 64];               // S as right operand
+  __shared__ f32x4 us[4 * 64];                  // U, weighted by what is left of it at the chunk's end
+  const int vtile = blockIdx.x, head = blockIdx.y, req = blockIdx.z, grp = head / (a.H / a.G);
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, lg = lane >> 4;
+  const int vtiles = gridDim.x, vcol = vtile * 16 + col;
+  const bool in = vcol < a.vdim;
+  const int first = a.req_first[req], last = a.req_first[req + 1];
+  if (first >= last) return;
+  float* slot = a.state + ((size_t)a.row_of[req] * a.H + head) * HS_DIM * a.vdim + (in ? vcol : 0);
+  f32x4 S[HS_MT];
+#pragma unroll
+  for (int m = 0; m < HS_MT; ++m) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = (wave + 4 * m) * 16 + 4 * lg + r;
+      S[m][r] = in && d < HS_DIM ? slot[(size_t)d * a.vdim] : 0.f;
+    }
+  }
+  const TX* x = reinterpret_cast<const TX*>(a.x);
+  for (int c = first; c < last; ++c) {
+    const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
+    const size_t ch = (size_t)c * a.H + head;
+    const double* ls = a.lsum + ch * HS_CHUNK;
+    const float* gate = a.gate + ch * HS_CHUNK;
+    const float* unit = a.unit + (((size_t)c * a.G + grp) * 2 + 1) * HS_CHUNK;
+    const TX* xr = x + (size_t)begin * a.x_stride;
+    for (int idx = tid; idx < HS_CHUNK * (HS_DIMP / 4); idx += 256) {
+      const int t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
+      f32x4 kv = {0.f, 0.f, 0.f, 0.f};
+      if (t < n) kv = ld_keys<TX>(xr + (size_t)t * a.x_stride + a.k_off + (size_t)grp * HS_DIM, d);
+      *reinterpret_cast<f32x4*>(k + t * HS_LD + d) = kv;
+    }
+    float* s0 = a.s0 + ((ch * vtiles + vtile) * HS_KB * 64 + lane) * 4;
+#pragma unroll
+    for (int m = 0; m < HS_MT; ++m) {
+      const int b = wave + 4 * m;
+      if (b < HS_KB) {
+        s[b * 64 + lane] = S[m];
+        *reinterpret_cast<f32x4*>(s0 + (size_t)b * 256) = S[m];
+      }
+    }
+    float* ug = a.u + ((ch * vtiles + vtile) * 4 + wave) * 256 + lane * 4;
+    f32x4 u;
+    if (DELTA) {
+      u = *reinterpret_cast<const f32x4*>(ug);
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = wave * 16 + 4 * lg + r;
+        u[r] = in && t < n ? gate[t] * ldf<TX>(xr + (size_t)t * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol) : 0.f;
+      }
+    }
+    __syncthreads();
+    if (DELTA) {
+      const float* wk = a.wk + (ch * HS_CHUNK + wave * 16 + col) * HS_DIMP + 4 * lg;
+      f32x4 p0 = {0.f, 0.f, 0.f, 0.f}, p1 = p0;
+#pragma unroll
+      for (int b = 0; b < HS_KB; b += 2) {
+        p0 = mma16(*reinterpret_cast<const f32x4*>(wk + b * 16), s[b * 64 + lane], p0);
+        if (b + 1 < HS_KB) p1 = mma16(*reinterpret_cast<const f32x4*>(wk + b * 16 + 16), s[(b + 1) * 64 + lane], p1);
+      }
+      u -= p0 + p1;
+    }
+    *reinterpret_cast<f32x4*>(ug) = u;
+    const double end = ls[HS_CHUNK - 1];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = wave * 16 + 4 * lg + r;
+      u[r] *= expf((float)(end - ls[t])) * unit[t];
+    }
+    us[wave * 64 + lane] = u;
+    __syncthreads();
+    const float g = expf((float)end);
+#pragma unroll
+    for (int m = 0; m < HS_MT; ++m) {
+      const int b = wave + 4 * m;
+      if (b < HS_KB) {
+        f32x4 acc = S[m] * g;
+#pragma unroll
+        for (int tb = 0; tb < 4; ++tb) {
+          f32x4 kt;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) kt[j] = k[(tb * 16 + 4 * lg + j) * HS_LD + b * 16 + col];
+          acc = mma16(kt, us[tb * 64 + lane], acc);
+        }
+        S[m] = acc;
+      }
+    }
+    __syncthreads();                            // the staged keys, S and U have been read
+  }
+  if (in) {
+#pragma unroll
+    for (int m = 0; m < HS_MT; ++m) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = (wave + 4 * m) * 16 + 4 * lg + r;
+        if (d < HS_DIM) slot[(size_t)d * a.vdim] = S[m][r];
+      }
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// O of a (chunk, head): wave w has the token rows 16 w .. 16 w + 15
+// ---------------------------------------------------------------------------------------
+template <typename TX>
+__global__ __launch_bounds__(256) void hs_out_kernel(HeadScan a) {
+  const int c = blockIdx.x, head = blockIdx.y, grp = head / (a.H / a.G);
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, lg = lane >> 4;
+  const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
+  if (wave * 16 >= n) return;
+  const size_t ch = (size_t)c * a.H + head;
+  const double* ls = a.lsum + ch * HS_CHUNK;
+  const TX* xr = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride;
+  const int row = wave * 16 + col;              // of the left operands
+  const double mine = ls[row];
+  f32x4 p[4];
+#pragma unroll
+  for (int jb = 0; jb < 4; ++jb) {
+    p[jb] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (jb <= wave) {
+      const f32x4 sc = *reinterpret_cast<const f32x4*>(a.qk + (((size_t)c * a.G + grp) * HS_CHUNK + row) * HS_CHUNK + jb * 16 + 4 * lg);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int t = jb * 16 + 4 * lg + j;
+        if (t <= row) p[jb][j] = sc[j] * expf((float)(mine - ls[t]));
+      }
+    }
+  }
+  f32x4 q[HS_KB];
+  {
+    const float f = expf((float)mine) * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + row];
+    const TX* qr = xr + (size_t)(row < n ? row : 0) * a.x_stride + a.q_off + (size_t)grp * HS_DIM;
+#pragma unroll
+    for (int b = 0; b < HS_KB; ++b) {
+      q[b] = ld_keys<TX>(qr, b * 16 + 4 * lg);
+      q[b] *= row < n ? f : 0.f;
+    }
+  }
+  const float skip = a.skip ? a.skip[head] : 0.f;
+  const int vtiles = (a.vdim + 15) / 16;
+  for (int vt = 0; vt < vtiles; ++vt) {
+    const f32x4* s0 = reinterpret_cast<const f32x4*>(a.s0) + (ch * vtiles + vt) * HS_KB * 64 + lane;
+    const f32x4* ug = reinterpret_cast<const f32x4*>(a.u) + (ch * vtiles + vt) * 4 * 64 + lane;
+    f32x4 o0 = {0.f, 0.f, 0.f, 0.f}, o1 = o0;
+#pragma unroll
+    for (int b = 0; b < HS_KB; ++b) o0 = mma16(q[b], s0[b * 64], o0);
+#pragma unroll
+    for (int jb = 0; jb < 4; ++jb)
+      if (jb <= wave) o1 = mma16(p[jb], ug[jb * 64], o1);
+    const int vcol = vt * 16 + col;
+    if (vcol < a.vdim) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = wave * 16 + 4 * lg + r;
+        if (t < n) {
+          float v = o0[r] + o1[r];
+          if (a.skip) v += skip * ldf<TX>(xr + (size_t)t * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol);
+          a.out[((size_t)(begin + t) * a.H + head) * a.vdim + vcol] = v;
+        }
+      }
+    }
+  }
+}
+#endif  // HS_CHUNKED
+
+extern "C" int qvl_head_scan_key_size() { return HS_DIM; }
+extern "C" int qvl_head_scan_chunked() { return HS_CHUNKED; }
+
+static int fill_args(HeadScan& a, const void* x, long long x_stride, int q_off, int k_off, int v_off, const void* raw,
+                     long long raw_stride, int a_off, int b_off, const void* bias, const void* a_neg, const void* skip,
+                     float q_scale, float unit_eps, void* state, const void* bounds, const void* row_of, void* out, int H,
+                     int G, int dim, int vdim) {
+  if (dim != HS_DIM || H <= 0 || G <= 0 || H % G || vdim <= 0) return QVL_ERR_SHAPE;
+  if (!x || !raw || !bias || !a_neg || !state || !bounds || !row_of || !out) return QVL_ERR_SHAPE;
+  if (q_off < 0 || k_off < 0 || v_off < 0 || a_off < 0) return QVL_ERR_SHAPE;
+  if (x_stride < (long long)q_off + (long long)G * HS_DIM || x_stride < (long long)k_off + (long long)G * HS_DIM ||
+      x_stride < (long long)v_off + (long long)H * vdim || raw_stride < (long long)a_off + H || raw_stride < (long long)b_off + H)
+    return QVL_ERR_SHAPE;
+  if (H > 65535) return QVL_ERR_LIMIT;
+  a = HeadScan{};
+  a.x = x; a.x_stride = x_stride; a.q_off = q_off; a.k_off = k_off; a.v_off = v_off; a.raw = (const float*)raw;
+  a.raw_stride = raw_stride; a.a_off = a_off; a.b_off = b_off; a.bias = (const float*)bias; a.a_neg = (const float*)a_neg;
+  a.skip = (const float*)skip; a.q_scale = q_scale; a.unit_eps = unit_eps; a.state = (float*)state;
+  a.bounds = (const int*)bounds; a.row_of = (const int*)row_of; a.out = (float*)out; a.H = H; a.G = G; a.vdim = vdim;
+  return QVL_OK;
+}
+
+// x rows hold q (G * HS_DIM columns from q_off), k (from k_off) and v (H * vdim columns from v_off); raw rows the step
+// inputs (from a_off) and, with the delta rule (b_off >= 0), the beta inputs.  unit_eps < 0: no unit vectors.  bounds
+// [R + 1], row_of [R] (the request's slot); out float32 [N, H * vdim].  dtype: of x.
+extern "C" int qvl_head_scan(const void* x, long long x_stride, int q_off, int k_off, int v_off, const void* raw,
+                             long long raw_stride, int a_off, int b_off, const void* bias, const void* a_neg,
+                             const void* skip, float q_scale, float unit_eps, void* state, const void* bounds,
+                             const void* row_of, void* out, int R, int H, int G, int dim, int vdim, int dtype,
+                             hipStream_t stream) {
+  if (R <= 0) return QVL_OK;
+  if (R > 65535) return QVL_ERR_LIMIT;
+  HeadScan a;
+  const int bad = fill_args(a, x, x_stride, q_off, k_off, v_off, raw, raw_stride, a_off, b_off, bias, a_neg, skip, q_scale,
+                            unit_eps, state, bounds, row_of, out, H, G, dim, vdim);
+  if (bad) return bad;
+  const dim3 grid((vdim + 63) / 64, H, R);
+  const bool delta = b_off >= 0;
+#define LAUNCH(TX, D) hipLaunchKernelGGL((hs_scan_kernel<TX, D>), grid, dim3(256), 0, stream, a)
+  if (dtype == 0) { if (delta) LAUNCH(float, true); else LAUNCH(float, false); }
+  else if (dtype == 1) { if (delta) LAUNCH(bf16_t, true); else LAUNCH(bf16_t, false); }
+  else return QVL_ERR_DTYPE;
+#undef LAUNCH
+  return qvl_launch_status();
+}
+
+// Floats of scratch memory that qvl_head_scan_chunks needs.
+extern "C" long long qvl_head_scan_scratch(int chunks, int H, int G, int vdim, int delta) {
+  const long long vtiles = (vdim + 15) / 16, c = chunks;
+  return c * H * HS_CHUNK * 3 + c * G * (2 * HS_CHUNK + (delta ? 2 : 1) * HS_CHUNK * HS_CHUNK) +
+         (delta ? c * H * HS_CHUNK * HS_DIMP : 0) + c * H * vtiles * (4 + HS_KB) * 256;
+}
+
+// The same in chunks of at most 64 tokens: chunk_cu [chunks + 1], req_first [R + 1] (the first chunk of each request);
+// scratch 16-byte aligned.
+extern "C" int qvl_head_scan_chunks(const void* x, long long x_stride, int q_off, int k_off, int v_off, const void* raw,
+                                    long long raw_stride, int a_off, int b_off, const void* bias, const void* a_neg,
+                                    const void* skip, float q_scale, float unit_eps, void* state, const void* chunk_cu,
+                                    const void* req_first, const void* row_of, void* out, void* scratch, int chunks, int R,
+                                    int H, int G, int dim, int vdim, int dtype, hipStream_t stream) {
+#if HS_CHUNKED
+  if (R <= 0 || chunks <= 0) return QVL_OK;
+  if (R > 65535) return QVL_ERR_LIMIT;
+  HeadScan a;
+  const int bad = fill_args(a, x, x_stride, q_off, k_off, v_off, raw, raw_stride, a_off, b_off, bias, a_neg, skip, q_scale,
+                            unit_eps, state, chunk_cu, row_of, out, H, G, dim, vdim);
+  if (bad) return bad;
+  if (!req_first || !scratch || ((uintptr_t)scratch & 15)) return QVL_ERR_SHAPE;
+  const bool delta = b_off >= 0;
+  const int vtiles = (vdim + 15) / 16;
+  a.req_first = (const int*)req_first;
+  const long long c = chunks;
+  float* at = (float*)scratch;
+  a.lsum = (double*)at; at += c * H * HS_CHUNK * 2;
+  a.gate = at; at += c * H * HS_CHUNK;
+  a.unit = at; at += c * G * 2 * HS_CHUNK;
+  a.qk = at; at += c * G * HS_CHUNK * HS_CHUNK;
+  if (delta) { a.kk = at; at += c * G * HS_CHUNK * HS_CHUNK; }
+  if (delta) { a.wk = at; at += c * H * HS_CHUNK * HS_DIMP; }
+  a.u = at; at += c * H * vtiles * 4 * 256;
+  a.s0 = at;
+#define LAUNCH(TX, D)                                                                                                \
+  {                                                                                                                  \
+    hipLaunchKernelGGL((hs_prep_kernel<D>), dim3(chunks, (H + 3) / 4), dim3(256), 0, stream, a);                     \
+    hipLaunchKernelGGL((hs_score_kernel<TX, D>), dim3(chunks, G), dim3(256), 0, stream, a);                \
+    if (D) hipLaunchKernelGGL((hs_solve_kernel<TX>), dim3(chunks, H), dim3(256), 0, stream, a);                      \
+    hipLaunchKernelGGL((hs_carry_kernel<TX, D>), dim3(vtiles, H, R), dim3(256), 0, stream, a);             \
+    hipLaunchKernelGGL((hs_out_kernel<TX>), dim3(chunks, H), dim3(256), 0, stream, a);                               \
+  }
+  if (dtype == 0) { if (delta) LAUNCH(float, true) else LAUNCH(float, false) }
+  else if (dtype == 1) { if (delta) LAUNCH(bf16_t, true) else LAUNCH(bf16_t, false) }
+  else return QVL_ERR_DTYPE;
+#undef LAUNCH
+  return qvl_launch_status();
+#else
+  return QVL_ERR_LIMIT;
+#endif
+}

@@ -1,7 +1,7 @@
 // Row-wise kernels of layers whose norm stands behind the sublayer, and of feed-forwards whose activation
 // is a sum of normed powers or a squared relu.  float32 and bfloat16 storage; all arithmetic is float32.
 //
-//   layer norm     y = (v - mean(v)) / sqrt(mean((v - mean(v))^2) + eps) * w      (no bias; two passes: the
+//   layer norm     y = (v - mean(v)) / sqrt(mean((v - mean(v))^2) + eps) * w [+ b]  (two passes: the
 //                  deviations are formed from the mean, not from a sum of squares)
 //   normed powers  out = a z / rms(z) + b z^2 / rms(z^2) + c z^3 / rms(z^3) + e,  rms(u) = sqrt(mean(u^2) + eps),
 //                  powers taken element by element over a row
@@ -109,7 +109,8 @@ struct RowValues {
 template <typename TS, typename TO, int PER, int VEC>
 __global__ __launch_bounds__(RN_THREADS) void layer_norm_kernel(const TS* __restrict__ src, int nslabs,
                                                                 long long slab_stride, const float* __restrict__ w,
-                                                                float eps, float* __restrict__ add, TO* __restrict__ out,
+                                                                const float* __restrict__ b, float eps,
+                                                                float* __restrict__ add, TO* __restrict__ out,
                                                                 const int* __restrict__ rows, int H) {
   __shared__ float red[17];
   const size_t m = blockIdx.x;
@@ -129,6 +130,10 @@ __global__ __launch_bounds__(RN_THREADS) void layer_norm_kernel(const TS* __rest
     r.each4([&](float4 x, int c) {
       const float4 g = ld4v<float>(w + c);
       float4 y{(x.x - mean) * inv * g.x, (x.y - mean) * inv * g.y, (x.z - mean) * inv * g.z, (x.w - mean) * inv * g.w};
+      if (b) {
+        const float4 o = ld4v<float>(b + c);
+        y.x += o.x; y.y += o.y; y.z += o.z; y.w += o.w;
+      }
       if (arow) {
         const float4 a = ld4v<float>(arow + c);
         y.x += a.x; y.y += a.y; y.z += a.z; y.w += a.w;
@@ -140,6 +145,7 @@ __global__ __launch_bounds__(RN_THREADS) void layer_norm_kernel(const TS* __rest
   }
   r.each([&](float x, int c) {
     float y = (x - mean) * inv * w[c];
+    if (b) y += b[c];
     if (arow) {
       y += arow[c];
       arow[c] = y;
@@ -151,12 +157,12 @@ __global__ __launch_bounds__(RN_THREADS) void layer_norm_kernel(const TS* __rest
 static inline bool aligned16(const void* p) { return ((uintptr_t)p & 15) == 0; }
 
 template <typename TS, typename TO>
-static int launch_layer_norm(const void* src, int nslabs, long long slab_stride, const void* w, float eps, void* add,
+static int launch_layer_norm(const void* src, int nslabs, long long slab_stride, const void* w, const void* b, float eps, void* add,
                              void* out, const void* rows, int M, int H, hipStream_t stream) {
 #define LN_LAUNCH(PER, VEC)                                                                                           \
   hipLaunchKernelGGL((layer_norm_kernel<TS, TO, PER, VEC>), dim3(M), dim3(RN_THREADS), 0, stream, (const TS*)src,     \
-                     nslabs, slab_stride, (const float*)w, eps, (float*)add, (TO*)out, (const int*)rows, H)
-  if (H % 4 == 0 && H <= RN_THREADS * 4 * 32 && slab_stride % 4 == 0 && aligned16(src) && aligned16(w) && aligned16(add) &&
+                     nslabs, slab_stride, (const float*)w, (const float*)b, eps, (float*)add, (TO*)out, (const int*)rows, H)
+  if (H % 4 == 0 && H <= RN_THREADS * 4 * 32 && slab_stride % 4 == 0 && aligned16(src) && aligned16(w) && aligned16(b) && aligned16(add) &&
       aligned16(out)) {
     const int per = (H / 4 + RN_THREADS - 1) / RN_THREADS;
     if (per <= 1) LN_LAUNCH(1, 4);
@@ -179,20 +185,20 @@ static int launch_layer_norm(const void* src, int nslabs, long long slab_stride,
   return qvl_launch_status();
 }
 
-// src_dtype / out_dtype: 0 float32, 1 bfloat16.  Slabs (nslabs > 1) are float32.  `add` (float32 [rows, H], may
+// b: float32 [H] or null.  src_dtype / out_dtype: 0 float32, 1 bfloat16.  Slabs (nslabs > 1) are float32.  `add` (float32 [rows, H], may
 // be null) and `out` ([M, H], may be null) as above; `rows` (int32 [M], may be null) picks rows of src.
-extern "C" int qvl_layer_norm(const void* src, int src_dtype, int nslabs, long long slab_stride, const void* w, float eps,
-                              void* add, void* out, int out_dtype, const void* rows, int M, int H, hipStream_t stream) {
+extern "C" int qvl_layer_norm(const void* src, int src_dtype, int nslabs, long long slab_stride, const void* w, const void* b,
+                              float eps, void* add, void* out, int out_dtype, const void* rows, int M, int H, hipStream_t stream) {
   if (M <= 0) return QVL_OK;
   if (H <= 0 || !src || !w || nslabs < 1 || (nslabs > 1 && src_dtype != 0) || (!add && !out)) return QVL_ERR_SHAPE;
   if (src_dtype == 0 && (out_dtype == 0 || !out))
-    return launch_layer_norm<float, float>(src, nslabs, slab_stride, w, eps, add, out, rows, M, H, stream);
+    return launch_layer_norm<float, float>(src, nslabs, slab_stride, w, b, eps, add, out, rows, M, H, stream);
   if (src_dtype == 0 && out_dtype == 1)
-    return launch_layer_norm<float, bf16_t>(src, nslabs, slab_stride, w, eps, add, out, rows, M, H, stream);
+    return launch_layer_norm<float, bf16_t>(src, nslabs, slab_stride, w, b, eps, add, out, rows, M, H, stream);
   if (src_dtype == 1 && (out_dtype == 0 || !out))
-    return launch_layer_norm<bf16_t, float>(src, nslabs, slab_stride, w, eps, add, out, rows, M, H, stream);
+    return launch_layer_norm<bf16_t, float>(src, nslabs, slab_stride, w, b, eps, add, out, rows, M, H, stream);
   if (src_dtype == 1 && out_dtype == 1)
-    return launch_layer_norm<bf16_t, bf16_t>(src, nslabs, slab_stride, w, eps, add, out, rows, M, H, stream);
+    return launch_layer_norm<bf16_t, bf16_t>(src, nslabs, slab_stride, w, b, eps, add, out, rows, M, H, stream);
   return QVL_ERR_DTYPE;
 }
 

@@ -104,6 +104,27 @@ class PassMix(Part):
         return ResidualStream(h if h.is_contiguous() else h.contiguous(), pending=first_share)
 
 
+class TokenSideTable(Part):
+    """A table ``[vocab, columns]`` beside the embedding's: every layer of a model that has one reads columns of its own
+    of a token's row."""
+
+    graph_safe = True
+
+    def __init__(self, vocab: int, columns: int, dtype, device):
+        super().__init__(dtype, device)
+        self.vocab, self.columns = int(vocab), int(columns)
+        self.weight: Optional[torch.Tensor] = None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        return {"weight": ParamSpec((self.vocab, self.columns), "table")}
+
+    def load(self, tensors):
+        self.weight = tensors["weight"]
+
+    def named_weights(self) -> Dict[str, torch.Tensor]:
+        return {"weight": self.weight}
+
+
 class DecoderModel:
     """Holds the parts and runs a step over them.  Tensors arrive through :meth:`load_part`."""
 
@@ -127,6 +148,11 @@ class DecoderModel:
             if not spec.pass_mix_name.endswith(".weight"):
                 raise ValueError("the pass-mix matrix is a tensor '<name>.weight'")
             self.pass_mix = PassMix(spec.hidden_size, dtype, self.device)
+        self.token_side: Optional[TokenSideTable] = None
+        if spec.token_side_name is not None:
+            if not spec.token_side_name.endswith(".weight") or spec.token_side_columns <= 0:
+                raise ValueError("the second table of token rows is a tensor '<name>.weight' with at least one column")
+            self.token_side = TokenSideTable(spec.vocab_size, spec.token_side_columns, dtype, self.device)
         for i, entry in enumerate(spec.run):
             if entry.add_vector is not None and not (self.pass_vectors is not None
                                                      and 0 <= entry.add_vector < spec.pass_vectors_rows):
@@ -200,6 +226,8 @@ class DecoderModel:
             _collect(self.pass_vectors, _prefix_of(spec.pass_vectors_name), self.params)
         if self.pass_mix is not None:
             _collect(self.pass_mix, _prefix_of(spec.pass_mix_name), self.params)
+        if self.token_side is not None:
+            _collect(self.token_side, _prefix_of(spec.token_side_name), self.params)
         for ls, block in zip(spec.layers, self.blocks):
             _collect(block, ls.prefix, self.params)
         _collect(self.final_norm, spec.final_norm_prefix, self.params)
@@ -281,6 +309,7 @@ class DecoderModel:
         ``step.logit_rows``."""
         if not self._has_weights:
             raise RuntimeError("the model has no weights yet")
+        step.token_side = None if self.token_side is None else self.token_side.weight
         if self.embed_place is not None:
             stream = ResidualStream(self.embedding.forward(step.token_ids, step, slots[len(self.spec.run)]))
         else:
@@ -295,7 +324,10 @@ class DecoderModel:
                 if stream.row_addend is not None:
                     raise RuntimeError("a block left a pass vector unadded: its first norm must fold the stream")
                 stream.row_addend = self.pass_vectors.weight[entry.add_vector]   # the layer's first norm adds it
-            stream = self.blocks[entry.layer].forward(stream, step, slot)
+            block = self.blocks[entry.layer]
+            stream = block.forward(stream, step, slot)
+            if not block.leaves_rounded:
+                stream.rounded = None
         if step.logit_rows.shape[0] == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=self.device)
         x = self.final_norm.forward(stream, rows=step.logit_rows)

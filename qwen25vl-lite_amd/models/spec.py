@@ -69,3 +69,7 @@ class ModelSpec:
     # the matrix ``[hidden, 2 hidden]`` of the run entries with ``mix_input`` (columns of the running sum first,
     # then those of the embedding's output): the canonical name of the tensor; None: the model has none
     pass_mix_name: Optional[str] = None
+    # a second table of token rows whose columns layers read (``StepContext.token_side``): the canonical name of a
+    # tensor ``[vocab, columns]`` and its number of columns; None: the model has none
+    token_side_name: Optional[str] = None
+    token_side_columns: int = 0

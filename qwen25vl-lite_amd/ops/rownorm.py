@@ -17,7 +17,7 @@ from .kernels import _check, _dev, _fn, _need, _ptr, _stream, dtype_code
 __all__ = ["layer_norm", "layer_norm_add_", "normed_powers", "squared_relu_"]
 
 _c_int, _c_float, _c_ptr, _c_ll = ctypes.c_int, ctypes.c_float, ctypes.c_void_p, ctypes.c_longlong
-_LN_ARGS = [_c_ptr, _c_int, _c_int, _c_ll, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr]
+_LN_ARGS = [_c_ptr, _c_int, _c_int, _c_ll, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr]
 
 
 def _source(y: torch.Tensor, width: int):
@@ -32,13 +32,14 @@ def _source(y: torch.Tensor, width: int):
 
 
 def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,
-               rows: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``(x - mean) / sqrt(mean((x - mean)^2) + eps) * weight`` over each row (of ``x[rows]`` if given), in
+               rows: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``(x - mean) / sqrt(mean((x - mean)^2) + eps) * weight [+ bias]`` over each row (of ``x[rows]`` if given), in
     ``out_dtype``; statistics and arithmetic in float32."""
-    _dev(x, weight, rows)
+    _dev(x, weight, rows, bias)
     width = x.shape[-1]
-    _need(weight.dtype == torch.float32 and weight.shape == (width,) and weight.is_contiguous(),
-          "the norm's weight must be float32 [H]")
+    for v in (weight, bias):
+        _need(v is None or (v.dtype == torch.float32 and v.shape == (width,) and v.is_contiguous()),
+              "the norm's weight and bias must be float32 [H]")
     n, nslabs, stride = _source(x, width)
     m = n
     if rows is not None:
@@ -47,7 +48,7 @@ def layer_norm(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: tor
         m = rows.shape[0]
     out = torch.empty((m, width), dtype=out_dtype, device=x.device)
     fn = _fn("rownorm", "qvl_layer_norm", _LN_ARGS)
-    _check(fn(_ptr(x), dtype_code(x.dtype), nslabs, stride, _ptr(weight), float(eps), None, _ptr(out),
+    _check(fn(_ptr(x), dtype_code(x.dtype), nslabs, stride, _ptr(weight), _ptr(bias), float(eps), None, _ptr(out),
               dtype_code(out_dtype), _ptr(rows), m, width, _stream()), "layer_norm")
     return out
 
@@ -65,7 +66,7 @@ def layer_norm_add_(h: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps:
     _need(rows == n, "the addend must have h's rows")
     out = None if copy_dtype is None else torch.empty((n, width), dtype=copy_dtype, device=h.device)
     fn = _fn("rownorm", "qvl_layer_norm", _LN_ARGS)
-    _check(fn(_ptr(y), dtype_code(y.dtype), nslabs, stride, _ptr(weight), float(eps), _ptr(h), _ptr(out),
+    _check(fn(_ptr(y), dtype_code(y.dtype), nslabs, stride, _ptr(weight), None, float(eps), _ptr(h), _ptr(out),
               dtype_code(copy_dtype) if copy_dtype is not None else 0, None, n, width, _stream()), "layer_norm_add")
     return out
 

@@ -51,7 +51,9 @@ class PagedAttention(Mixer):
     convolution over time, ``y_t = sum_j w[:, j] u_(t - taps + 1 + j)`` per channel with weights ``q_conv`` /
     ``k_conv`` of ``[channels, taps]``, before norm and rotation; keys that are their own values are taken behind
     it; a request's last ``taps - 1`` projected rows are its state), ``sinks`` (True: a tensor ``sink [heads]``
-    whose ``exp`` joins each head's softmax denominator), ``chunk`` (a number: positions are cut into chunks of
+    whose ``exp`` joins each head's softmax denominator), ``plus_one`` (True: one joins each denominator, a sink of zero
+    that no tensor holds), ``retain`` (how many keys back pages are kept, default ``window``: the longest window of the
+    layers that read this cache; None: all), ``chunk`` (a number: positions are cut into chunks of
     that many from the sequence's start and a token sees the keys of its own chunk up to itself), ``value_rotation`` (a
     base: the value of position j is turned by j over all its channels before it is cached, in the position encoding's
     layout of pairs, pair m by ``j base^(-2m/value_dim)``, and each head's output at position i is turned back by i).
@@ -83,6 +85,13 @@ class PagedAttention(Mixer):
         self.qk_norm_scope = str(params.get("qk_norm_scope", "head"))
         self.conv_taps = int(params.get("conv_taps") or 0)
         self.has_sinks = bool(params.get("sinks", False))
+        self.plus_one = bool(params.get("plus_one", False))
+        if self.has_sinks and self.plus_one:
+            raise ValueError("a softmax's denominator takes a sink per head or one, not both")
+        self.retain: Optional[int] = params.get("retain", self.window)
+        if (self.retain is None) != (self.window is None) and self.retain is not None or (
+                self.retain is not None and self.window is not None and self.retain < self.window):
+            raise ValueError("a cache is kept at least as far back as its layer sees")
         self.chunk: Optional[int] = None if params.get("chunk") is None else int(params["chunk"])
         if self.chunk is not None and self.chunk < 1:
             raise ValueError("a chunk holds at least one position")
@@ -133,7 +142,7 @@ class PagedAttention(Mixer):
         self.sink: Optional[torch.Tensor] = None
 
     def cache_need(self) -> CacheNeed:
-        return CacheNeed(self.nkv, self.hd, self.window, self.keep_first, None if self.vd == self.hd else self.vd, self.chunk)
+        return CacheNeed(self.nkv, self.hd, self.retain, self.keep_first, None if self.vd == self.hd else self.vd, self.chunk)
 
     @property
     def conv_channels(self) -> int:
@@ -206,6 +215,8 @@ class PagedAttention(Mixer):
                 taps.append(tensors[f"{n['k_conv']}.weight"])
             self.w_conv = torch.cat(taps, dim=0).t().contiguous()
         self.sink = tensors.get(f"{n['sink']}.weight")
+        if self.plus_one:
+            self.sink = torch.zeros(self.nq, dtype=torch.float32, device=self.w_out.device)
 
     def named_weights(self) -> Dict[str, torch.Tensor]:
         """Views of the stacked tensors under their checkpoint names."""
@@ -228,7 +239,7 @@ class PagedAttention(Mixer):
             out[f"{n['q_conv']}.weight"] = self.w_conv[:, :self.nq * self.hd].t()
             if not self.kv_shared:
                 out[f"{n['k_conv']}.weight"] = self.w_conv[:, self.nq * self.hd:].t()
-        if self.sink is not None:
+        if self.has_sinks:
             out[f"{n['sink']}.weight"] = self.sink
         out[f"{n['o']}.weight"] = self.w_out
         return out

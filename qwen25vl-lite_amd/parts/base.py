@@ -36,7 +36,7 @@ import torch
 
 __all__ = [
     "ParamSpec", "PartSpec", "CacheNeed", "StateNeed", "LayerSlot", "GroupStep", "StepContext", "ResidualStream",
-    "NormedMean",
+    "NormedMean", "SumTerm", "ScaledSum",
     "Part", "Norm", "Mixer", "FeedForward", "Filter", "PositionEncoding", "Block", "register_part", "build_part",
     "known_parts", "Embedding", "Head",
 ]
@@ -161,6 +161,8 @@ class StepContext:
     max_ctx_len: int = 0
     dtype: torch.dtype = torch.float32
     residual: Optional[torch.Tensor] = None   # set by a block while a part may add its result in place
+    # the model's second table of token rows [vocab, columns], where it has one: layers read columns of their own
+    token_side: Optional[torch.Tensor] = None
     derived: Dict[Any, Any] = field(default_factory=dict)   # per-step arrays kernels derive once (tile lists)
     # tensors computed from the step's values once per forward pass (rotation tables): a context
     # that is run again with new values (a captured step) starts each pass with this empty
@@ -184,6 +186,9 @@ class ResidualStream:
     copies: Optional[torch.Tensor] = None
     # (mix [copies, copies], out [copies]) float32: how the pending addend joins the copies
     pending_join: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
+    # ``h`` rounded to the run dtype, where the kernel that wrote ``h`` last wrote that too (a block that leaves it
+    # says so: ``Block.leaves_rounded``)
+    rounded: Optional[torch.Tensor] = None
 
 
 @dataclass
@@ -198,6 +203,38 @@ class NormedMean:
     gain_second: torch.Tensor
     eps: float
     factor: float
+
+
+@dataclass
+class ScaledSum:
+    """A sublayer's result ``factor_first * first + factor_second * second`` that has not been computed yet (addends as
+    in :class:`NormedMean`)."""
+
+    first: torch.Tensor
+    second: torch.Tensor
+    factor_first: float
+    factor_second: float
+
+
+@dataclass
+class SumTerm:
+    """One term of a residual sum: ``factor * value``, or with a gain ``factor * rmsnorm(value) * gain``.  ``value`` is
+    ``[N, hidden]`` (float32 or bfloat16) or float32 slabs ``[slabs, N, hidden]`` that are added in order."""
+
+    value: torch.Tensor
+    factor: float = 1.0
+    gain: Optional[torch.Tensor] = None
+    eps: float = 0.0
+
+    @staticmethod
+    def of(result) -> List["SumTerm"]:
+        """The terms of what a sublayer returned."""
+        if isinstance(result, NormedMean):
+            return [SumTerm(result.first, result.factor, result.gain_first, result.eps),
+                    SumTerm(result.second, result.factor, result.gain_second, result.eps)]
+        if isinstance(result, ScaledSum):
+            return [SumTerm(result.first, result.factor_first), SumTerm(result.second, result.factor_second)]
+        return [SumTerm(result)]
 
 
 class Part:
@@ -279,6 +316,8 @@ class PositionEncoding(Part):
 
 
 class Block(Part):
+    leaves_rounded: bool = False    # forward leaves ``stream.rounded`` equal to the ``stream.h`` it leaves
+
     def forward(self, stream: ResidualStream, step: StepContext, slot: LayerSlot) -> ResidualStream:
         raise NotImplementedError
 

@@ -6,9 +6,9 @@ from typing import Dict, Optional
 
 import torch
 
-from .base import Block, LayerSlot, Part, PartSpec, ResidualStream, StepContext, build_part, register_part
+from .base import Block, LayerSlot, Part, PartSpec, ResidualStream, StepContext, SumTerm, build_part, register_part
 
-__all__ = ["PreNormBlock", "ParallelBlock", "SandwichBlock", "PostNormBlock"]
+__all__ = ["PreNormBlock", "ParallelBlock", "SandwichBlock", "PostNormBlock", "SumNormBlock"]
 
 
 class PreNormBlock(Block):
@@ -215,6 +215,74 @@ class PostNormBlock(Block):
         return stream
 
 
+class SumNormBlock(Block):
+    """``h = norm1(alpha h + mixer(h)); h = norm2(alpha h + ffn(h))``: the sublayers read the sum itself and the norm
+    stands behind the sum; then, with a side input, ``h += side_norm(side(h))``.
+
+    params: ``alpha``, ``mixer``, ``norm1`` (:class:`PartSpec` each; the norm must offer ``norm_sum``, as a layer norm
+    with a bias does), ``ffn`` and ``norm2`` (or ``ffn`` None for a layer without a feed-forward, whose ``norm2`` is then
+    not built), ``side`` (a :class:`PartSpec` of category ``ffn``, or None) and ``side_norm`` (of an RMS norm), and
+    ``names``, the checkpoint sub-name of each.  The sum stays float32; the kernel that forms it also writes the rounded
+    rows that the next sublayer reads.
+    """
+
+    graph_safe = True
+    leaves_rounded = True
+
+    def __init__(self, params, dtype, device):
+        super().__init__(dtype, device)
+        self.names: Dict[str, str] = dict(params["names"])
+        self.alpha = float(params["alpha"])
+        self.mixer = build_part("mixer", params["mixer"], dtype, device)
+        self.norm1 = build_part("norm", params["norm1"], dtype, device)
+        self.ffn: Optional[Part] = None
+        self.norm2: Optional[Part] = None
+        if params.get("ffn") is not None:
+            self.ffn = build_part("ffn", params["ffn"], dtype, device)
+            self.norm2 = build_part("norm", params["norm2"], dtype, device)
+        self.side: Optional[Part] = None
+        self.side_norm: Optional[Part] = None
+        if params.get("side") is not None:
+            self.side = build_part("ffn", params["side"], dtype, device)
+            self.side_norm = build_part("norm", params["side_norm"], dtype, device)
+        for norm in (self.norm1, self.norm2):
+            if norm is not None and not hasattr(norm, "norm_sum"):
+                raise ValueError("the norm behind the sum must be able to form it")
+
+    def sub_parts(self) -> Dict[str, Part]:
+        parts = {self.names["mixer"]: self.mixer, self.names["norm1"]: self.norm1}
+        if self.ffn is not None:
+            parts.update({self.names["ffn"]: self.ffn, self.names["norm2"]: self.norm2})
+        if self.side is not None:
+            parts.update({self.names["side"]: self.side, self.names["side_norm"]: self.side_norm})
+        return parts
+
+    def forward(self, stream: ResidualStream, step: StepContext, slot: LayerSlot) -> ResidualStream:
+        from ..ops.sum_norm import sum_norm_
+
+        if stream.pending is not None or stream.pending_norm is not None or stream.row_addend is not None:
+            raise RuntimeError("this block reads the sum itself: nothing may be pending")
+        h = stream.h
+        # rows a sublayer reads: the sum itself in a float32 run, else its rounded copy
+        copy = None if self.dtype == h.dtype else self.dtype
+        x = h if copy is None else (stream.rounded if stream.rounded is not None else h.to(copy))
+
+        def read(rounded):
+            return h if copy is None else rounded
+
+        step.residual = None                 # a sublayer's result joins the sum under the norm
+        y = self.mixer.forward(x, step, slot.of(self.names["mixer"]))
+        x = read(self.norm1.norm_sum(h, self.alpha, y, copy))
+        if self.ffn is not None:
+            x = read(self.norm2.norm_sum(h, self.alpha, self.ffn.forward(x, step), copy))
+        if self.side is not None:
+            y = SumTerm(self.side.forward(x, step), gain=self.side_norm.weight, eps=self.side_norm.eps)
+            x = read(sum_norm_(h, 1.0, [y], copy_dtype=copy))
+        stream.rounded = None if copy is None else x
+        return stream
+
+
+register_part("block", "sum_norm", SumNormBlock)
 register_part("block", "sandwich", SandwichBlock)
 register_part("block", "post_norm", PostNormBlock)
 register_part("block", "pre_norm", PreNormBlock)

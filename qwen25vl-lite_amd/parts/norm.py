@@ -8,7 +8,7 @@ import torch
 
 from ..ops import kernels, skinny
 from ..ops.linear import NormedRows
-from .base import Norm, ParamSpec, ResidualStream, register_part
+from .base import Norm, ParamSpec, ResidualStream, SumTerm, register_part
 
 __all__ = ["RMSNorm", "LayerNorm"]
 
@@ -70,10 +70,10 @@ class RMSNorm(Norm):
 
 
 class LayerNorm(Norm):
-    """``(x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * weight``: the mean is taken off, there is no
-    bias; statistics in float32, the deviations formed from the mean (two passes).
+    """``(x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * weight [+ bias]``: the mean is taken off;
+    statistics in float32, the deviations formed from the mean (two passes).
 
-    params: ``size`` (row width), ``eps``.
+    params: ``size`` (row width), ``eps``, ``bias`` (default False: there is none).
     """
 
     graph_safe = True
@@ -82,13 +82,19 @@ class LayerNorm(Norm):
         super().__init__(dtype, device)
         self.size = int(params["size"])
         self.eps = float(params["eps"])
+        self.has_bias = bool(params.get("bias", False))
         self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
 
     def param_specs(self) -> Dict[str, ParamSpec]:
-        return {"weight": ParamSpec((self.size,), "vector", init="around_one")}
+        specs = {"weight": ParamSpec((self.size,), "vector", init="around_one")}
+        if self.has_bias:
+            specs["bias"] = ParamSpec((self.size,), "vector")
+        return specs
 
     def load(self, tensors):
         self.weight = tensors["weight"]
+        self.bias = tensors.get("bias")
 
     def forward(self, stream: ResidualStream, rows: Optional[torch.Tensor] = None, lazy: bool = False):
         from ..ops import rownorm
@@ -99,13 +105,24 @@ class LayerNorm(Norm):
         if stream.pending is not None:
             residual_add(stream.h, stream.pending)
             stream.pending = None
-        return rownorm.layer_norm(stream.h, self.weight, self.eps, self.dtype, rows=rows)
+        return rownorm.layer_norm(stream.h, self.weight, self.eps, self.dtype, rows=rows, bias=self.bias)
 
     def add_normed(self, h: torch.Tensor, y: torch.Tensor, copy_dtype: Optional[torch.dtype] = None):
         """``h += norm(y)`` in float32, in place; with ``copy_dtype`` the new ``h`` is also returned in it."""
         from ..ops import rownorm
 
+        if self.bias is not None:
+            raise RuntimeError("a norm on what joins the sum has no bias here")
         return rownorm.layer_norm_add_(h, y, self.weight, self.eps, copy_dtype)
+
+    def norm_sum(self, h: torch.Tensor, alpha: float, result, copy_dtype: Optional[torch.dtype] = None):
+        """``h = norm(alpha h + result)`` in float32, in place (``result``: what a sublayer returned); with
+        ``copy_dtype`` the new ``h`` is also returned in it."""
+        from ..ops.sum_norm import sum_norm_
+
+        if self.bias is None:
+            raise RuntimeError("a norm behind the sum has a weight and a bias")
+        return sum_norm_(h, alpha, SumTerm.of(result), self.weight, self.bias, self.eps, copy_dtype)
 
 
 register_part("norm", "rms_norm", RMSNorm)
