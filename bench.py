@@ -194,6 +194,44 @@ def zaposun_config(layers, size="7b", order=ZAPOSUN_ORDER, chunk=1024, streams=4
                        for i in range(int(layers))]}
 
 
+VEZIDRA_ORDER = ("attention", "parallel", "parallel_2", "attention_shared")
+
+
+def vezidra_config(layers, size="7b", order=VEZIDRA_ORDER, window=1024, taps=4, side_dim=256):
+    """A Vezidra decoder with the width, head counts and vocabulary of one of SIZES and attention heads of 128 channels.
+    Layers in the given order (repeated): ``attention`` (the last ``window`` keys), ``attention_shared`` (the same, reading
+    the keys and values of the nearest ``attention`` layer before it), ``parallel`` (attention over all keys beside the
+    delta rule with heads of 128 by 128, queries and keys shared by pairs of heads), ``parallel_2`` (attention over all keys
+    beside a state space of twice the width, heads of 64 channels with 128 states, 8 groups).  Every layer has a
+    feed-forward of 3/2 of the size's width, so that its two matrices weigh what three of a gated one do."""
+    s = SIZES[size]
+    nh, nkv, hd, width = s["num_attention_heads"], s["num_key_value_heads"], 128, s["hidden_size"]
+    heads = {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5}
+    inner_heads = 2 * width // 64
+    mixers = {
+        "attention": {**heads, "mask": {"size": window}, "rot": {"base": 10000.0, "dims": hd // 2}},
+        "parallel": {"left": {**heads, "rot": {"base": 500000.0, "dims": hd, "scaling": {
+                         "factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+                     "right": {"heads": nh, "kv_heads": nh // 2, "dim": hd, "vdim": hd, "conv": taps},
+                     "left_scale": 0.75, "right_scale": 1.25},
+        "parallel_2": {"left": {**heads, "rot": {"base": 1000000.0, "dims": hd, "scaling": {
+                           "factor": 4.0, "original": 8192, "fast": 16.0, "slow": 2.0}}},
+                       "right": {"heads": inner_heads, "vdim": 64, "state": 128, "groups": 8, "norm_groups": 8, "conv": taps}},
+    }
+    mlp = {"kind": "dense", "ff": s["intermediate_size"] * 3 // 2 // 16 * 16}
+    out, owner = [], None
+    for i in range(int(layers)):
+        kind = order[i % len(order)]
+        m = dict(mixers["attention" if kind == "attention_shared" else kind])
+        if kind == "attention_shared" and owner is not None:
+            m["kv_from"] = owner
+        elif kind.startswith("attention"):
+            owner = i
+        out.append({"type": "attention" if kind.startswith("attention") else kind, "mixer": m, "mlp": mlp})
+    return {"architecture": "Vezidra", "width": width, "vocab": s["vocab_size"], "norm": {"eps": 1e-5},
+            "embedding": {"scale": 8.0}, "postln_alpha": 2.0, "token_side": {"dim": side_dim}, "layers": out}
+
+
 def step_bytes(t, batch, ctx, bytes_per_value=2):
     """Bytes a decode step has to read: every weight it uses once (all layers and the head; of the
     embedding only the rows looked up) and the keys and values of the live requests."""
@@ -348,15 +386,15 @@ def main(argv=None) -> int:
     ap.add_argument("--attention", type=int, nargs="+", metavar="TOKENS",
                     help="instead: the prefill attention alone (one request of that many tokens in one step, the "
                          "chosen size's heads, bfloat16, pages in shuffled order), microseconds and TFLOP/s for each length")
-    ap.add_argument("--design", choices=["gogudra", "dazapel", "rapisun", "rofapel", "zaposun"],
+    ap.add_argument("--design", choices=["gogudra", "dazapel", "rapisun", "rofapel", "zaposun", "vezidra"],
                     help="instead: prefill (2,048 tokens) and decode throughput of this design at the chosen size's "
                          "width, heads and feed-forward (random weights), beside the Qwen2.5-VL decoder with as many layers")
-    ap.add_argument("--beside", choices=["qwen25vl", "gogudra", "dazapel", "rapisun", "rofapel"], default="qwen25vl",
+    ap.add_argument("--beside", choices=["qwen25vl", "gogudra", "dazapel", "rapisun", "rofapel", "zaposun"], default="qwen25vl",
                     help="with --design: the model the design is measured beside, at the same sizes")
     ap.add_argument("--order", default=None,
-                    help="with --design gogudra, rapisun, rofapel or zaposun: the mixers of successive layers, repeated "
+                    help="with --design gogudra, rapisun, rofapel, zaposun or vezidra: the mixers of successive layers, repeated "
                          "(gogudra: gla,gla,lightning,attention; rapisun: " + ",".join(RAPISUN_ORDER) + "; rofapel: "
-                         + ",".join(ROFAPEL_ORDER) + "; zaposun: " + ",".join(ZAPOSUN_ORDER) + ")")
+                         + ",".join(ROFAPEL_ORDER) + "; zaposun: " + ",".join(ZAPOSUN_ORDER) + "; vezidra: " + ",".join(VEZIDRA_ORDER) + ")")
     ap.add_argument("--loop", default=None, metavar="START,STOP,TIMES",
                     help="with --design rofapel: layers START .. STOP-1 run TIMES times in a row (default: no loop)")
     ap.add_argument("--no-graph", action="store_true", help="do not replay decode steps from a HIP graph")
@@ -385,7 +423,7 @@ def main(argv=None) -> int:
     if args.design and not args.layers:
         args.layers = 8
     if args.order is None:
-        args.order = ",".join({"rapisun": RAPISUN_ORDER, "rofapel": ROFAPEL_ORDER, "zaposun": ZAPOSUN_ORDER}.get(
+        args.order = ",".join({"rapisun": RAPISUN_ORDER, "rofapel": ROFAPEL_ORDER, "zaposun": ZAPOSUN_ORDER, "vezidra": VEZIDRA_ORDER}.get(
             args.design, ("gla", "gla", "lightning", "attention")))
     cfg = Qwen25VLConfig.from_dict(decoder_config(args.layers, args.size))
     t = cfg.text_config
@@ -461,7 +499,7 @@ def main(argv=None) -> int:
         beside = "the Qwen2.5-VL decoder" if args.beside == "qwen25vl" else args.beside
         out = {"metric": f"prefill and decode tok/s, {args.design} beside {beside} "
                          f"({args.size} sizes, {args.layers} layers, {args.dtype})", "unit": "tokens/s",
-               "order": args.order.split(",") if args.design in ("gogudra", "rapisun", "rofapel", "zaposun") else None,
+               "order": args.order.split(",") if args.design in ("gogudra", "rapisun", "rofapel", "zaposun", "vezidra") else None,
                "batch": args.batch, "prompt_tokens": args.prompt_tokens, "data": "synthetic"}
         if args.design == "rofapel" and args.loop:
             out["loop"] = [int(v) for v in args.loop.split(",")]
@@ -476,7 +514,10 @@ def main(argv=None) -> int:
                 return rofapel_config(args.layers, args.size, tuple(args.order.split(",")) if name == args.design
                                       else ROFAPEL_ORDER, loop=[int(v) for v in args.loop.split(",")] if args.loop else None)
             if name == "zaposun":
-                return zaposun_config(args.layers, args.size, tuple(args.order.split(",")))
+                return zaposun_config(args.layers, args.size, tuple(args.order.split(",")) if name == args.design
+                                      else ZAPOSUN_ORDER)
+            if name == "vezidra":
+                return vezidra_config(args.layers, args.size, tuple(args.order.split(",")))
             return gogudra_config(args.layers, args.size, tuple(args.order.split(",")) if name == args.design
                                   else ("gla", "gla", "lightning", "attention"))
 

@@ -337,10 +337,35 @@ __global__ void head_gate_kernel(T* __restrict__ o, const float* __restrict__ ga
   for (int i = threadIdx.x; i < nh * hd; i += blockDim.x) stf<T>(orow + i, ldf<T>(orow + i) * sigmoid_f(g[i / hd]));
 }
 
+// the same with four values a thread, which belong to one head (hd a multiple of 4)
+template <typename T>
+__global__ __launch_bounds__(256) void head_gate_vec_kernel(T* __restrict__ o, const float* __restrict__ gate,
+                                                            long long gate_stride, int groups, int per_head, long long total) {
+  const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= total) return;
+  const long long n = i / groups;
+  const float g = sigmoid_f(gate[n * gate_stride + (int)(i % groups) / per_head]);
+  float4 v = ldv4<T>(o + 4 * i);
+  stv4<T>(o + 4 * i, float4{v.x * g, v.y * g, v.z * g, v.w * g});
+}
+
 extern "C" int qvl_head_gate(void* o, const void* gate, long long gate_stride, int N, int nh, int hd, int dtype,
                              hipStream_t stream) {
   if (N <= 0) return QVL_OK;
   if (nh <= 0 || hd <= 0 || gate_stride < nh) return QVL_ERR_SHAPE;
+  const long long total = (long long)N * nh * (hd / 4);
+  if (hd % 4 == 0 && (uintptr_t)o % 16 == 0 && (total + 255) / 256 <= 0x7fffffffLL) {
+    const dim3 grid((unsigned)((total + 255) / 256));
+    if (dtype == 0)
+      hipLaunchKernelGGL(head_gate_vec_kernel<float>, grid, dim3(256), 0, stream, (float*)o, (const float*)gate,
+                         gate_stride, nh * (hd / 4), hd / 4, total);
+    else if (dtype == 1)
+      hipLaunchKernelGGL(head_gate_vec_kernel<bf16_t>, grid, dim3(256), 0, stream, (bf16_t*)o, (const float*)gate,
+                         gate_stride, nh * (hd / 4), hd / 4, total);
+    else
+      return QVL_ERR_DTYPE;
+    return qvl_launch_status();
+  }
   if (dtype == 0)
     hipLaunchKernelGGL(head_gate_kernel<float>, dim3(N), dim3(256), 0, stream, (float*)o, (const float*)gate,
                        gate_stride, nh, hd);

@@ -89,6 +89,7 @@ extern "C" void qvl_gemm_resident_timeline(void* p) { timeline_buffer = (unsigne
 
 enum { PRO_PLAIN = 0, PRO_NORM = 1 };
 enum { EPI_STORE = 0, EPI_RESIDUAL = 1, EPI_SWIGLU = 2, EPI_ROPE = 3 };
+#define ACT_RELU2 2
 
 struct ResidentArgs {
   const bf16_t* X;       // PRO_PLAIN: [M, K]
@@ -122,7 +123,7 @@ struct ResidentArgs {
   // is cut into `parts` tiles of `pairs` gate rows and their up rows, so that the last round of
   // tiles is as even as the rounds before it
   int whole_tiles, parts, pairs;
-  int gelu;              // EPI_SWIGLU: the activation is the tanh form of gelu
+  int gelu;              // EPI_SWIGLU: 1: the activation is the tanh form of gelu; EPI_STORE: ACT_RELU2: max(product, 0)^2 is stored
   // Several products of the same sizes side by side (EPI_STORE, one block a team): product i has the blocks
   // i * stack_blocks .. and its operands and result lie i strides further on (in elements)
   int stack_blocks;      // 0: one product
@@ -368,6 +369,10 @@ __global__ __launch_bounds__(64 * RW) void gemm_resident_kernel(ResidentArgs p) 
         }
       } else if (m < p.M && nl < p.rows && n < p.N) {
         sum += epi.bias;
+        if (EPI == EPI_STORE && p.gelu == ACT_RELU2) {
+          sum = fmaxf(sum, 0.f);
+          sum *= sum;
+        }
         if (EPI == EPI_RESIDUAL) {
           float* o = reinterpret_cast<float*>(p.out);
           o[(size_t)m * p.ldo + n] = epi.old + sum;
@@ -574,14 +579,16 @@ extern "C" int qvl_gemm_resident_two_tile_k() { return 32 * XHI_STEPS; }
 
 // x: bfloat16 [M, K] (h null), or h: float32 [M, K] with norm_w [K] and eps (x null): X = rmsnorm(h) * norm_w.
 // epilogue 0: out[M, N] in out_dtype (0 float32, 1 bfloat16); 1: out (float32 [M, N]) += product;
-// 2: out[M, N/2] bfloat16 = silu(gate) * up for W rows in groups of 8 gate, 8 up; 4: the same with gelu's tanh form.
+// 2: out[M, N/2] bfloat16 = silu(gate) * up for W rows in groups of 8 gate, 8 up; 4: the same with gelu's tanh form;
+// 5: out[M, N] in out_dtype = max(product (+ bias), 0)^2.
 // max_blocks: blocks to launch at most (the number of compute units).
 extern "C" int qvl_gemm_resident(const void* x, int ldx, const void* h, int ldh, const void* norm_w, float eps,
                                  const void* W, int ldw, const void* bias, void* out, int ldo, int M, int N, int K,
                                  int out_dtype, int epilogue, int max_blocks, hipStream_t stream) {
   if (M <= 0 || N <= 0) return QVL_OK;
-  const int gelu = epilogue == 4;
-  if (gelu) epilogue = EPI_SWIGLU;
+  const int gelu = epilogue == 4 ? 1 : (epilogue == 5 ? ACT_RELU2 : 0);
+  if (epilogue == 4) epilogue = EPI_SWIGLU;
+  if (epilogue == 5) epilogue = EPI_STORE;
   if (M > 64) return QVL_ERR_LIMIT;
   if (M > 32 && K > PASS_K) return QVL_ERR_LIMIT;   // teams of more than two keep their rows for a single pass
   if (K <= 0 || K % 8 || ldw % 8 || ldw < K || max_blocks <= 0 || !W || !out) return QVL_ERR_SHAPE;

@@ -62,6 +62,8 @@ struct HeadScan {
   const int* req_first;      // [R + 1] a request's chunks
   double* lsum;              // [chunks, H, 64]: sum of the decays' logarithms from the chunk's start, token included
   float* gate;               // [chunks, H, 64]: beta or step
+  float* head;               // [chunks, H, 64]: the decays' product from the chunk's start, token included
+  float* tail;               // [chunks, H, 64]: the decays' product behind the token to the chunk's end
   float* qk;                 // [chunks, G, 64, 64]
   float* kk;                 // [chunks, G, 64, 64]
   float* unit;               // [chunks, G, 2, 64]: factors on q (its scale included) and k
@@ -211,35 +213,59 @@ __global__ __launch_bounds__(256) void hs_prep_kernel(HeadScan a) {
   const size_t at = ((size_t)c * a.H + head) * HS_CHUNK + t;
   a.lsum[at] = l;                               // tokens past the chunk's end keep the last sum
   a.gate[at] = g;
+  a.head[at] = expf((float)l);
+  a.tail[at] = expf((float)(__shfl(l, 63, 64) - l));
 }
 
-// a row of 16 key blocks from global memory, four channels from d on (zeros past HS_DIM)
-template <typename TX> __device__ __forceinline__ f32x4 ld_keys(const TX* row, int d) {
-  f32x4 v;
+// Four channels of a row as they lie in memory.  VEC: HS_DIM, strides and offsets are multiples of four and rows lie on
+// boundaries of four values, so that one load fetches them.
+template <typename TX, bool VEC> struct Four {
+  TX v[4];
+  __device__ __forceinline__ void fetch(const TX* row, int d) {
 #pragma unroll
-  for (int j = 0; j < 4; ++j) v[j] = d + j < HS_DIM ? ldf<TX>(row + d + j) : 0.f;
-  return v;
-}
+    for (int j = 0; j < 4; ++j) v[j] = row[d + j < HS_DIM ? d + j : 0];
+  }
+  __device__ __forceinline__ f32x4 value(int d, bool live) const {
+    f32x4 o;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = live && d + j < HS_DIM ? ldf<TX>(v + j) : 0.f;
+    return o;
+  }
+};
+template <> struct Four<bf16_t, true> {
+  uint2 v;
+  __device__ __forceinline__ void fetch(const bf16_t* row, int d) { v = *reinterpret_cast<const uint2*>(row + (d < HS_DIM ? d : 0)); }
+  __device__ __forceinline__ f32x4 value(int d, bool live) const {
+    if (!live || d >= HS_DIM) return f32x4{0.f, 0.f, 0.f, 0.f};
+    return f32x4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
+                 __uint_as_float(v.y & 0xffff0000u)};
+  }
+};
+template <> struct Four<float, true> {
+  f32x4 v;
+  __device__ __forceinline__ void fetch(const float* row, int d) { v = *reinterpret_cast<const f32x4*>(row + (d < HS_DIM ? d : 0)); }
+  __device__ __forceinline__ f32x4 value(int d, bool live) const { return live && d < HS_DIM ? v : f32x4{0.f, 0.f, 0.f, 0.f}; }
+};
 
 // ---------------------------------------------------------------------------------------
 // Q K^T and K K^T of a (chunk, group), lower triangle's tiles; factors of the unit lengths folded in
 // ---------------------------------------------------------------------------------------
-template <typename TX, bool DELTA>
+template <typename TX, bool DELTA, bool VEC>
 __global__ __launch_bounds__(256) void hs_score_kernel(HeadScan a) {
   __shared__ __attribute__((aligned(16))) float q[HS_CHUNK * HS_LD], k[HS_CHUNK * HS_LD];
   __shared__ float f[2][HS_CHUNK];
   const int c = blockIdx.x, grp = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
   const TX* x = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride + (size_t)grp * HS_DIM;
-  for (int idx = tid; idx < HS_CHUNK * (HS_DIMP / 4); idx += 256) {
-    const int t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
-    f32x4 qv = {0.f, 0.f, 0.f, 0.f}, kv = qv;
-    if (t < n) {
-      qv = ld_keys<TX>(x + (size_t)t * a.x_stride + a.q_off, d);
-      kv = ld_keys<TX>(x + (size_t)t * a.x_stride + a.k_off, d);
-    }
-    *reinterpret_cast<f32x4*>(q + t * HS_LD + d) = qv;
-    *reinterpret_cast<f32x4*>(k + t * HS_LD + d) = kv;
+#pragma unroll 4
+  for (int i = 0; i < HS_KB; ++i) {             // 64 tokens of HS_KB * 4 groups of four channels
+    const int idx = tid + 256 * i, t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
+    Four<TX, VEC> qv, kv;
+    const TX* row = x + (size_t)(t < n ? t : 0) * a.x_stride;
+    qv.fetch(row + a.q_off, d);
+    kv.fetch(row + a.k_off, d);
+    *reinterpret_cast<f32x4*>(q + t * HS_LD + d) = qv.value(d, t < n);
+    *reinterpret_cast<f32x4*>(k + t * HS_LD + d) = kv.value(d, t < n);
   }
   __syncthreads();
   {                                             // four threads a token
@@ -291,20 +317,33 @@ __global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
   __shared__ __attribute__((aligned(16))) float A[HS_CHUNK][HS_CHUNK + 4];   // strictly below the diagonal
   __shared__ __attribute__((aligned(16))) float T[4][16][20];                // inverses of the diagonal blocks
   __shared__ float rv[HS_CHUNK], rk[HS_CHUNK];                               // factors on the rows of V and K
+  __shared__ double ls[HS_CHUNK];
   const int c = blockIdx.x, head = blockIdx.y, grp = head / (a.H / a.G);
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, lg = lane >> 4;
   const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
   const size_t ch = (size_t)c * a.H + head;
-  const double* ls = a.lsum + ch * HS_CHUNK;
-  const float* beta = a.gate + ch * HS_CHUNK;
   const float* kk = a.kk + ((size_t)c * a.G + grp) * HS_CHUNK * HS_CHUNK;
-  for (int idx = tid; idx < HS_CHUNK * HS_CHUNK; idx += 256) {
-    const int i = idx >> 6, j = idx & 63;
-    A[i][j] = j < i ? beta[i] * expf((float)(ls[i] - ls[j])) * kk[idx] : 0.f;
-  }
+  f32x4 prod[4];                                // a thread has four neighbouring columns of the rows tid / 16 + 16 i
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    prod[i] = (tid & 15) * 4 < 16 * i + 16 ? *reinterpret_cast<const f32x4*>(kk + (tid + 256 * i) * 4) : f32x4{0.f, 0.f, 0.f, 0.f};
   if (tid < HS_CHUNK) {
-    rv[tid] = beta[tid];
-    rk[tid] = beta[tid] * expf((float)ls[tid]) * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + HS_CHUNK + tid];
+    const float beta = a.gate[ch * HS_CHUNK + tid];
+    ls[tid] = a.lsum[ch * HS_CHUNK + tid];
+    rv[tid] = beta;
+    rk[tid] = beta * a.head[ch * HS_CHUNK + tid] * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + HS_CHUNK + tid];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int row = (tid >> 4) + 16 * i, j0 = (tid & 15) * 4;
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    if (j0 < row) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (j0 + j < row) v[j] = rv[row] * expf((float)(ls[row] - ls[j0 + j])) * prod[i][j];
+    }
+    *reinterpret_cast<f32x4*>(&A[row][j0]) = v;
   }
   __syncthreads();
   if (lane < 16) {                              // wave w inverts diagonal block w, a lane per column
@@ -370,106 +409,154 @@ __global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
 // ---------------------------------------------------------------------------------------
 #define HS_MT ((HS_KB + 3) / 4)                 // row blocks of S a wave keeps: wave w has blocks w, w + 4, ...
 
-template <typename TX, bool DELTA>
+// What a block reads of a chunk, asked for a chunk ahead: nothing here is waited for before it is used.
+template <typename TX, bool DELTA, bool VEC, int NV> struct CarryLoads {
+  Four<TX, VEC> k[HS_KB];
+  f32x4 wk[DELTA ? HS_KB : 1];
+  f32x4 u[DELTA ? NV : 1];
+  TX v[DELTA ? 1 : NV][4];
+  f32x4 gate, tail, unit;
+  float end;
+  int n;
+};
+
+// NV neighbouring tiles of 16 value channels a block
+template <typename TX, bool DELTA, bool VEC, int NV>
 __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
   __shared__ __attribute__((aligned(16))) float k[HS_CHUNK * HS_LD];   // the chunk's keys
-  __shared__ f32x4 s[HS_KB * 64];               // S as right operand
-  __shared__ f32x4 us[4 * 64];                  // U, weighted by what is left of it at the chunk's end
-  const int vtile = blockIdx.x, head = blockIdx.y, req = blockIdx.z, grp = head / (a.H / a.G);
+  __shared__ f32x4 s[NV][HS_KB * 64];           // S as right operand
+  __shared__ f32x4 us[NV][4 * 64];              // U, weighted by what is left of it at the chunk's end
+  const int head = blockIdx.y, req = blockIdx.z, grp = head / (a.H / a.G);
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, lg = lane >> 4;
-  const int vtiles = gridDim.x, vcol = vtile * 16 + col;
-  const bool in = vcol < a.vdim;
+  const int vtiles = (a.vdim + 15) / 16, vt0 = blockIdx.x * NV;
   const int first = a.req_first[req], last = a.req_first[req + 1];
   if (first >= last) return;
-  float* slot = a.state + ((size_t)a.row_of[req] * a.H + head) * HS_DIM * a.vdim + (in ? vcol : 0);
-  f32x4 S[HS_MT];
+  float* slot = a.state + ((size_t)a.row_of[req] * a.H + head) * HS_DIM * a.vdim;
+  f32x4 S[NV][HS_MT];
 #pragma unroll
-  for (int m = 0; m < HS_MT; ++m) {
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int d = (wave + 4 * m) * 16 + 4 * lg + r;
-      S[m][r] = in && d < HS_DIM ? slot[(size_t)d * a.vdim] : 0.f;
-    }
-  }
-  const TX* x = reinterpret_cast<const TX*>(a.x);
-  for (int c = first; c < last; ++c) {
-    const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
-    const size_t ch = (size_t)c * a.H + head;
-    const double* ls = a.lsum + ch * HS_CHUNK;
-    const float* gate = a.gate + ch * HS_CHUNK;
-    const float* unit = a.unit + (((size_t)c * a.G + grp) * 2 + 1) * HS_CHUNK;
-    const TX* xr = x + (size_t)begin * a.x_stride;
-    for (int idx = tid; idx < HS_CHUNK * (HS_DIMP / 4); idx += 256) {
-      const int t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
-      f32x4 kv = {0.f, 0.f, 0.f, 0.f};
-      if (t < n) kv = ld_keys<TX>(xr + (size_t)t * a.x_stride + a.k_off + (size_t)grp * HS_DIM, d);
-      *reinterpret_cast<f32x4*>(k + t * HS_LD + d) = kv;
-    }
-    float* s0 = a.s0 + ((ch * vtiles + vtile) * HS_KB * 64 + lane) * 4;
-#pragma unroll
-    for (int m = 0; m < HS_MT; ++m) {
-      const int b = wave + 4 * m;
-      if (b < HS_KB) {
-        s[b * 64 + lane] = S[m];
-        *reinterpret_cast<f32x4*>(s0 + (size_t)b * 256) = S[m];
-      }
-    }
-    float* ug = a.u + ((ch * vtiles + vtile) * 4 + wave) * 256 + lane * 4;
-    f32x4 u;
-    if (DELTA) {
-      u = *reinterpret_cast<const f32x4*>(ug);
-    } else {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = wave * 16 + 4 * lg + r;
-        u[r] = in && t < n ? gate[t] * ldf<TX>(xr + (size_t)t * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol) : 0.f;
-      }
-    }
-    __syncthreads();
-    if (DELTA) {
-      const float* wk = a.wk + (ch * HS_CHUNK + wave * 16 + col) * HS_DIMP + 4 * lg;
-      f32x4 p0 = {0.f, 0.f, 0.f, 0.f}, p1 = p0;
-#pragma unroll
-      for (int b = 0; b < HS_KB; b += 2) {
-        p0 = mma16(*reinterpret_cast<const f32x4*>(wk + b * 16), s[b * 64 + lane], p0);
-        if (b + 1 < HS_KB) p1 = mma16(*reinterpret_cast<const f32x4*>(wk + b * 16 + 16), s[(b + 1) * 64 + lane], p1);
-      }
-      u -= p0 + p1;
-    }
-    *reinterpret_cast<f32x4*>(ug) = u;
-    const double end = ls[HS_CHUNK - 1];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = wave * 16 + 4 * lg + r;
-      u[r] *= expf((float)(end - ls[t])) * unit[t];
-    }
-    us[wave * 64 + lane] = u;
-    __syncthreads();
-    const float g = expf((float)end);
-#pragma unroll
-    for (int m = 0; m < HS_MT; ++m) {
-      const int b = wave + 4 * m;
-      if (b < HS_KB) {
-        f32x4 acc = S[m] * g;
-#pragma unroll
-        for (int tb = 0; tb < 4; ++tb) {
-          f32x4 kt;
-#pragma unroll
-          for (int j = 0; j < 4; ++j) kt[j] = k[(tb * 16 + 4 * lg + j) * HS_LD + b * 16 + col];
-          acc = mma16(kt, us[tb * 64 + lane], acc);
-        }
-        S[m] = acc;
-      }
-    }
-    __syncthreads();                            // the staged keys, S and U have been read
-  }
-  if (in) {
+  for (int v = 0; v < NV; ++v) {
+    const int vcol = (vt0 + v) * 16 + col;
 #pragma unroll
     for (int m = 0; m < HS_MT; ++m) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int d = (wave + 4 * m) * 16 + 4 * lg + r;
-        if (d < HS_DIM) slot[(size_t)d * a.vdim] = S[m][r];
+        S[v][m][r] = vcol < a.vdim && d < HS_DIM ? slot[(size_t)d * a.vdim + vcol] : 0.f;
+      }
+    }
+  }
+  const TX* x = reinterpret_cast<const TX*>(a.x);
+  const int t_own = wave * 16 + 4 * lg;         // the first of this lane's four rows of U
+  CarryLoads<TX, DELTA, VEC, NV> l;
+  auto ask_keys = [&](int c) {
+    const int begin = a.bounds[c];
+    l.n = a.bounds[c + 1] - begin;
+    const TX* row0 = x + (size_t)begin * a.x_stride + a.k_off + (size_t)grp * HS_DIM;
+#pragma unroll
+    for (int i = 0; i < HS_KB; ++i) {
+      const int idx = tid + 256 * i, t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
+      l.k[i].fetch(row0 + (size_t)(t < l.n ? t : 0) * a.x_stride, d);
+    }
+  };
+  auto ask_rest = [&](int c) {
+    const size_t ch = (size_t)c * a.H + head;
+    l.tail = *reinterpret_cast<const f32x4*>(a.tail + ch * HS_CHUNK + t_own);
+    l.unit = *reinterpret_cast<const f32x4*>(a.unit + (((size_t)c * a.G + grp) * 2 + 1) * HS_CHUNK + t_own);
+    l.end = a.head[ch * HS_CHUNK + HS_CHUNK - 1];
+    if (DELTA) {
+      const float* wk = a.wk + (ch * HS_CHUNK + wave * 16 + col) * HS_DIMP + 4 * lg;
+#pragma unroll
+      for (int b = 0; b < HS_KB; ++b) l.wk[DELTA ? b : 0] = *reinterpret_cast<const f32x4*>(wk + b * 16);
+#pragma unroll
+      for (int v = 0; v < NV; ++v)
+        if (vt0 + v < vtiles) l.u[DELTA ? v : 0] = *reinterpret_cast<const f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4);
+    } else {
+      l.gate = *reinterpret_cast<const f32x4*>(a.gate + ch * HS_CHUNK + t_own);
+      const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
+#pragma unroll
+      for (int v = 0; v < NV; ++v) {
+        const int vcol = (vt0 + v) * 16 + col;
+        const TX* src = x + (size_t)begin * a.x_stride + a.v_off + (size_t)head * a.vdim + (vcol < a.vdim ? vcol : 0);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) l.v[DELTA ? 0 : v][r] = src[(size_t)(t_own + r < n ? t_own + r : 0) * a.x_stride];
+      }
+    }
+  };
+  ask_keys(first);
+  ask_rest(first);
+  for (int c = first; c < last; ++c) {
+    const size_t ch = (size_t)c * a.H + head;
+    const int n = l.n;
+#pragma unroll
+    for (int i = 0; i < HS_KB; ++i) {
+      const int idx = tid + 256 * i, t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
+      *reinterpret_cast<f32x4*>(k + t * HS_LD + d) = l.k[i].value(d, t < n);
+    }
+    if (c + 1 < last) ask_keys(c + 1);
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+      float* s0 = a.s0 + ((ch * vtiles + vt0 + v) * HS_KB * 64 + lane) * 4;
+#pragma unroll
+      for (int m = 0; m < HS_MT; ++m) {
+        const int b = wave + 4 * m;
+        if (b < HS_KB) {
+          if (DELTA) s[v][b * 64 + lane] = S[v][m];
+          if (vt0 + v < vtiles) *reinterpret_cast<f32x4*>(s0 + (size_t)b * 256) = S[v][m];
+        }
+      }
+    }
+    if (DELTA) __syncthreads();
+    f32x4 u[NV];
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+      if (DELTA) {
+        f32x4 p0 = {0.f, 0.f, 0.f, 0.f}, p1 = p0;
+#pragma unroll
+        for (int b = 0; b < HS_KB; b += 2) {
+          p0 = mma16(l.wk[DELTA ? b : 0], s[v][b * 64 + lane], p0);
+          if (b + 1 < HS_KB) p1 = mma16(l.wk[DELTA ? b + 1 : 0], s[v][(b + 1) * 64 + lane], p1);
+        }
+        u[v] = l.u[DELTA ? v : 0] - (p0 + p1);
+      } else {
+        const bool in = (vt0 + v) * 16 + col < a.vdim;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) u[v][r] = in && t_own + r < n ? l.gate[r] * ldf<TX>(&l.v[DELTA ? 0 : v][r]) : 0.f;
+      }
+      if (vt0 + v < vtiles) *reinterpret_cast<f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4) = u[v];
+      us[v][wave * 64 + lane] = u[v] * l.tail * l.unit;
+    }
+    const float g = l.end;
+    if (c + 1 < last) ask_rest(c + 1);
+    __syncthreads();
+#pragma unroll
+    for (int m = 0; m < HS_MT; ++m) {
+      const int b = wave + 4 * m;
+      if (b < HS_KB) {
+#pragma unroll
+        for (int v = 0; v < NV; ++v) S[v][m] *= g;
+#pragma unroll
+        for (int tb = 0; tb < 4; ++tb) {
+          f32x4 kt;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) kt[j] = k[(tb * 16 + 4 * lg + j) * HS_LD + b * 16 + col];
+#pragma unroll
+          for (int v = 0; v < NV; ++v) S[v][m] = mma16(kt, us[v][tb * 64 + lane], S[v][m]);
+        }
+      }
+    }
+    __syncthreads();                            // the staged keys, S and U have been read
+  }
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int vcol = (vt0 + v) * 16 + col;
+    if (vcol < a.vdim) {
+#pragma unroll
+      for (int m = 0; m < HS_MT; ++m) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int d = (wave + 4 * m) * 16 + 4 * lg + r;
+          if (d < HS_DIM) slot[(size_t)d * a.vdim + vcol] = S[v][m][r];
+        }
       }
     }
   }
@@ -478,7 +565,7 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
 // ---------------------------------------------------------------------------------------
 // O of a (chunk, head): wave w has the token rows 16 w .. 16 w + 15
 // ---------------------------------------------------------------------------------------
-template <typename TX>
+template <typename TX, bool VEC>
 __global__ __launch_bounds__(256) void hs_out_kernel(HeadScan a) {
   const int c = blockIdx.x, head = blockIdx.y, grp = head / (a.H / a.G);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, lg = lane >> 4;
@@ -488,6 +575,11 @@ __global__ __launch_bounds__(256) void hs_out_kernel(HeadScan a) {
   const double* ls = a.lsum + ch * HS_CHUNK;
   const TX* xr = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride;
   const int row = wave * 16 + col;              // of the left operands
+  Four<TX, VEC> qraw[HS_KB];
+  const TX* qr = xr + (size_t)(row < n ? row : 0) * a.x_stride + a.q_off + (size_t)grp * HS_DIM;
+#pragma unroll
+  for (int b = 0; b < HS_KB; ++b) qraw[b].fetch(qr, b * 16 + 4 * lg);
+  const float f = a.head[ch * HS_CHUNK + row] * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + row];
   const double mine = ls[row];
   f32x4 p[4];
 #pragma unroll
@@ -503,35 +595,48 @@ __global__ __launch_bounds__(256) void hs_out_kernel(HeadScan a) {
     }
   }
   f32x4 q[HS_KB];
-  {
-    const float f = expf((float)mine) * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + row];
-    const TX* qr = xr + (size_t)(row < n ? row : 0) * a.x_stride + a.q_off + (size_t)grp * HS_DIM;
 #pragma unroll
-    for (int b = 0; b < HS_KB; ++b) {
-      q[b] = ld_keys<TX>(qr, b * 16 + 4 * lg);
-      q[b] *= row < n ? f : 0.f;
-    }
-  }
+  for (int b = 0; b < HS_KB; ++b) q[b] = qraw[b].value(b * 16 + 4 * lg, row < n) * f;
   const float skip = a.skip ? a.skip[head] : 0.f;
   const int vtiles = (a.vdim + 15) / 16;
-  for (int vt = 0; vt < vtiles; ++vt) {
-    const f32x4* s0 = reinterpret_cast<const f32x4*>(a.s0) + (ch * vtiles + vt) * HS_KB * 64 + lane;
-    const f32x4* ug = reinterpret_cast<const f32x4*>(a.u) + (ch * vtiles + vt) * 4 * 64 + lane;
-    f32x4 o0 = {0.f, 0.f, 0.f, 0.f}, o1 = o0;
+  const f32x4* s0 = reinterpret_cast<const f32x4*>(a.s0) + ch * vtiles * HS_KB * 64 + lane;
+  const f32x4* ug = reinterpret_cast<const f32x4*>(a.u) + ch * vtiles * 4 * 64 + lane;
+  // two tiles of value channels at a time; the last of an odd number is formed twice
+  for (int vt = 0; vt < vtiles; vt += 2) {
+    const int other = vt + 1 < vtiles ? vt + 1 : vt;
+    f32x4 o[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-    for (int b = 0; b < HS_KB; ++b) o0 = mma16(q[b], s0[b * 64], o0);
+    for (int b = 0; b < HS_KB; ++b) {
+      const f32x4 s_a = s0[(vt * HS_KB + b) * 64], s_b = s0[(other * HS_KB + b) * 64];
 #pragma unroll
-    for (int jb = 0; jb < 4; ++jb)
-      if (jb <= wave) o1 = mma16(p[jb], ug[jb * 64], o1);
-    const int vcol = vt * 16 + col;
-    if (vcol < a.vdim) {
+      for (int j = 0; j < 4; ++j) {
+        o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[b][j], s_a[j], o[0], 0, 0, 0);
+        o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[b][j], s_b[j], o[1], 0, 0, 0);
+      }
+    }
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = wave * 16 + 4 * lg + r;
-        if (t < n) {
-          float v = o0[r] + o1[r];
-          if (a.skip) v += skip * ldf<TX>(xr + (size_t)t * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol);
-          a.out[((size_t)(begin + t) * a.H + head) * a.vdim + vcol] = v;
+    for (int jb = 0; jb < 4; ++jb) {
+      if (jb <= wave) {
+        const f32x4 u_a = ug[(vt * 4 + jb) * 64], u_b = ug[(other * 4 + jb) * 64];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[jb][j], u_a[j], o[0], 0, 0, 0);
+          o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[jb][j], u_b[j], o[1], 0, 0, 0);
+        }
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int vcol = (vt + i) * 16 + col;
+      if (vcol < a.vdim) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = wave * 16 + 4 * lg + r;
+          if (t < n) {
+            float v = o[i][r];
+            if (a.skip) v += skip * ldf<TX>(xr + (size_t)t * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol);
+            a.out[((size_t)(begin + t) * a.H + head) * a.vdim + vcol] = v;
+          }
         }
       }
     }
@@ -588,7 +693,7 @@ extern "C" int qvl_head_scan(const void* x, long long x_stride, int q_off, int k
 // Floats of scratch memory that qvl_head_scan_chunks needs.
 extern "C" long long qvl_head_scan_scratch(int chunks, int H, int G, int vdim, int delta) {
   const long long vtiles = (vdim + 15) / 16, c = chunks;
-  return c * H * HS_CHUNK * 3 + c * G * (2 * HS_CHUNK + (delta ? 2 : 1) * HS_CHUNK * HS_CHUNK) +
+  return c * H * HS_CHUNK * 5 + c * G * (2 * HS_CHUNK + (delta ? 2 : 1) * HS_CHUNK * HS_CHUNK) +
          (delta ? c * H * HS_CHUNK * HS_DIMP : 0) + c * H * vtiles * (4 + HS_KB) * 256;
 }
 
@@ -614,24 +719,34 @@ extern "C" int qvl_head_scan_chunks(const void* x, long long x_stride, int q_off
   float* at = (float*)scratch;
   a.lsum = (double*)at; at += c * H * HS_CHUNK * 2;
   a.gate = at; at += c * H * HS_CHUNK;
+  a.head = at; at += c * H * HS_CHUNK;
+  a.tail = at; at += c * H * HS_CHUNK;
   a.unit = at; at += c * G * 2 * HS_CHUNK;
   a.qk = at; at += c * G * HS_CHUNK * HS_CHUNK;
   if (delta) { a.kk = at; at += c * G * HS_CHUNK * HS_CHUNK; }
   if (delta) { a.wk = at; at += c * H * HS_CHUNK * HS_DIMP; }
   a.u = at; at += c * H * vtiles * 4 * 256;
   a.s0 = at;
-#define LAUNCH(TX, D)                                                                                                \
+  const bool vec = HS_DIM % 4 == 0 && x_stride % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0 && ((uintptr_t)x & 15) == 0;
+  // plain: a chunk's keys are staged once for two tiles of value channels
+  const int wide = delta || vtiles < 2 ? 1 : 2;
+#define CARRY(TX, D, V, NV)                                                                                          \
+  hipLaunchKernelGGL((hs_carry_kernel<TX, D, V, NV>), dim3((vtiles + NV - 1) / NV, H, R), dim3(256), 0, stream, a)
+#define LAUNCH(TX, D, V)                                                                                             \
   {                                                                                                                  \
     hipLaunchKernelGGL((hs_prep_kernel<D>), dim3(chunks, (H + 3) / 4), dim3(256), 0, stream, a);                     \
-    hipLaunchKernelGGL((hs_score_kernel<TX, D>), dim3(chunks, G), dim3(256), 0, stream, a);                \
+    hipLaunchKernelGGL((hs_score_kernel<TX, D, V>), dim3(chunks, G), dim3(256), 0, stream, a);                       \
     if (D) hipLaunchKernelGGL((hs_solve_kernel<TX>), dim3(chunks, H), dim3(256), 0, stream, a);                      \
-    hipLaunchKernelGGL((hs_carry_kernel<TX, D>), dim3(vtiles, H, R), dim3(256), 0, stream, a);             \
-    hipLaunchKernelGGL((hs_out_kernel<TX>), dim3(chunks, H), dim3(256), 0, stream, a);                               \
+    if (D || wide == 1) CARRY(TX, D, V, 1); else CARRY(TX, false, V, 2);                                             \
+    hipLaunchKernelGGL((hs_out_kernel<TX, V>), dim3(chunks, H), dim3(256), 0, stream, a);                            \
   }
-  if (dtype == 0) { if (delta) LAUNCH(float, true) else LAUNCH(float, false) }
-  else if (dtype == 1) { if (delta) LAUNCH(bf16_t, true) else LAUNCH(bf16_t, false) }
+#define BY_VEC(TX, D) { if (vec) LAUNCH(TX, D, true) else LAUNCH(TX, D, false) }
+  if (dtype == 0) { if (delta) BY_VEC(float, true) else BY_VEC(float, false) }
+  else if (dtype == 1) { if (delta) BY_VEC(bf16_t, true) else BY_VEC(bf16_t, false) }
   else return QVL_ERR_DTYPE;
+#undef BY_VEC
 #undef LAUNCH
+#undef CARRY
   return qvl_launch_status();
 #else
   return QVL_ERR_LIMIT;

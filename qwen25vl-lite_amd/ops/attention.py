@@ -17,21 +17,21 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     turn: Optional[torch.Tensor] = None, turn_pairs: bool = False) -> torch.Tensor:
     """Attention of the step's tokens over their requests' pages.
 
-    bfloat16 with a head size in steps of 16 runs on the matrix cores;
-    bfloat16 with a window that keeps the first keys, values of another width than the keys, or ``sinks``
-    (float32 ``[heads]``: one more term ``exp(sink)`` in each head's softmax denominator), chunks of positions
+    bfloat16 with a head size in steps of 16 runs on the matrix cores, with ``sinks`` (float32 ``[heads]``: one more term
+    ``exp(sink)`` in each head's softmax denominator) or without;
+    bfloat16 with a window that keeps the first keys, values of another width than the keys, sinks with a head size in
+    steps of 8, chunks of positions
     that see only themselves (``chunk``) or values turned by their positions (``turn``: the angles by which each
     token's output is turned back) has a matrix-core kernel of its own; everything else (float32, other head sizes) runs through the
     float32-arithmetic kernel.
     """
-    plain = (not (window and keep_first) and v_cache.shape[2] == k_cache.shape[3] and sinks is None and chunk is None
-             and turn is None)
+    plain = not (window and keep_first) and v_cache.shape[2] == k_cache.shape[3] and chunk is None and turn is None
     if q.dtype == torch.bfloat16 and plain:
         from . import attention_mfma
-        out = attention_mfma.try_attention(q, k_cache, v_cache, block_table, step, num_q_heads, window, scale)
+        out = attention_mfma.try_attention(q, k_cache, v_cache, block_table, step, num_q_heads, window, scale, sinks=sinks)
         if out is not None:
             return out
-    elif q.dtype == torch.bfloat16:
+    if q.dtype == torch.bfloat16 and (not plain or sinks is not None):
         from . import attention_window
         out = attention_window.try_attention(q, k_cache, v_cache, block_table, step, num_q_heads, window, keep_first,
                                              scale, sinks=sinks, chunk=chunk, turn=turn, turn_pairs=turn_pairs)

@@ -187,8 +187,10 @@ def block_groups(walks: int, places: int, head_dim: int) -> int:
 
 
 def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, window: Optional[int],
-                  scale: float, force_groups: Optional[int] = None, force_wide: Optional[bool] = None) -> Optional[torch.Tensor]:
-    """The attention through the matrix-core kernel, or None if it does not take this shape.
+                  scale: float, force_groups: Optional[int] = None, force_wide: Optional[bool] = None,
+                  sinks: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """The attention through the matrix-core kernel, or None if it does not take this shape.  ``sinks`` (float32
+    ``[heads]``): one more term ``exp(sink)`` in each query head's softmax denominator.
     Calls on one device must not overlap (one stream): the kernel for prompt portions keeps its
     work-queue counters in memory that all calls on the device share.
     ``force_groups``, ``force_wide`` (tests): the workgroup kind of the kernel for prompt portions and
@@ -203,6 +205,8 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
     _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.is_contiguous()
           and block_table.shape[0] == step.num_reqs, "block_table must be int32 [R, width]")
     _need(nq % nkv == 0, "query heads must be a multiple of key/value heads")
+    _need(sinks is None or (sinks.is_cuda and sinks.dtype == torch.float32 and sinks.shape == (nq,)
+                            and sinks.is_contiguous()), "sinks must be float32 [nq] on the GPU")
     tile_req, tile_ct, num_tiles = _step_tiles(step, nq // nkv, 1, q.device)
     out = torch.empty_like(q)
     defines = {"HD": hd}
@@ -219,7 +223,7 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
         if wide:
             tile_req, tile_ct, num_tiles = _step_tiles(step, nq // nkv, block_tiles(hd, True), q.device, by_length=True, only=only)
         fn = _fn("attention_mfma", "qvl_attn_mfma_block",
-                 [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr] + [_c_int] * 4
+                 [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr] + [_c_int] * 4
                  + [_c_float, _c_ptr, _c_int, _c_int, _c_ptr], defines)
         queue, cus = _work_queue(q.device)
         per_cu = int(_fn("attention_mfma", "qvl_attn_mfma_block_per_cu", [], defines)())
@@ -227,7 +231,7 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
         groups = block_groups(num_tiles * nkv, cus * per_cu, hd) if force_groups is None else force_groups
         groups = min(groups, most) if force_groups is None else groups
         code = fn(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(step.cu_q),
-                  _ptr(step.ctx_len), _ptr(tile_req), _ptr(tile_ct), num_tiles, _ptr(out), nq, nkv, ps, int(window or 0),
+                  _ptr(step.ctx_len), _ptr(tile_req), _ptr(tile_ct), num_tiles, _ptr(out), _ptr(sinks), nq, nkv, ps, int(window or 0),
                   float(scale), _ptr(queue), cus * (per_cu if groups == 1 else 1), groups, _stream())
         if code:
             # whatever a launch that went wrong did to the counters, the next one starts from zero
@@ -247,19 +251,21 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
             floats = _fn("attention_mfma", "qvl_attn_mfma_scratch_floats", [_c_int] * 3, defines)
             floats.restype = ctypes.c_longlong
             scratch = torch.empty(int(floats(num_tiles, nkv, nsplit)), dtype=torch.float32, device=q.device)
-        if nsplit > 1 and num_tiles * nkv <= MERGE_COUNTERS:
+        merged = nsplit > 1 and num_tiles * nkv <= MERGE_COUNTERS
+        if merged or sinks is not None:
             # the block of each (tile, head) that finishes last merges the splits: one launch
-            counters = _counters(q.device)
+            counters = _counters(q.device) if merged else None
             fn = _fn("attention_mfma", "qvl_attn_mfma_coop_merged",
-                     [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr, _c_ptr] + [_c_int] * 4
+                     [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr] + [_c_int] * 4
                      + [_c_float, _c_int, _c_int, _c_ptr], defines)
             code = fn(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(cu_q),
                       _ptr(step.ctx_len), _ptr(tile_req), _ptr(tile_ct), num_tiles, _ptr(out), _ptr(scratch),
-                      _ptr(counters), nq, nkv, ps, int(window or 0), float(scale), nsplit, per, _stream())
-            if code:
+                      _ptr(counters), _ptr(sinks), nq, nkv, ps, int(window or 0), float(scale), nsplit, per, _stream())
+            if code and merged:
                 counters.zero_()
             _check(code, "paged_attention (matrix cores, shared tiles, merged)")
-            taken["shared tiles, keys split among blocks, merged in the launch"] += 1
+            taken["shared tiles, keys split among blocks, merged in the launch" if merged else "shared tiles"
+                  + (", keys split among blocks, merged by a second launch" if nsplit > 1 else "")] += 1
             return
         fn = _fn("attention_mfma", "qvl_attn_mfma_coop",
                  [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr] + [_c_int] * 4

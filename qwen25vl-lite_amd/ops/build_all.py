@@ -29,6 +29,9 @@ LIBRARIES = [
     # size; these are what the tests and the benchmark use
     *[("hyper", {"HC_S": s}) for s in (1, 2, 3, 4, 5)],
     *[("selective_scan", {"SSM_STATE": n}) for n in (1, 3, 8, 16, 35, 40)],
+    ("sum_norm", {}),
+    # the recurrences with one decay per head, compiled per key size (these are what the tests and the benchmark use)
+    *[("head_scan", {"HS_DIM": d}) for d in (1, 8, 12, 16, 24, 32, 37, 48, 64, 80, 128, 256, 272)],
     # the linear-attention kernels are compiled per key size (the sizes the tests and the benchmark
     # use; any other size up to 512 is compiled at its first use)
     *[("linear_attention", {"LA_DIM": d}) for d in (5, 6, 8, 12, 16, 20, 32, 64, 128, 320)],

@@ -15,7 +15,7 @@ import torch
 
 from . import kernels, skinny
 
-__all__ = ["NormedRows", "linear", "linear_into", "linear_stack", "gate_up_swiglu", "tune_library_products"]
+__all__ = ["NormedRows", "linear", "linear_into", "linear_stack", "linear_relu2", "gate_up_swiglu", "tune_library_products"]
 
 
 class NormedRows:
@@ -88,6 +88,18 @@ def linear_stack(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
         else:
             _library(x[i], weight[i], None, torch.bfloat16, out=out[i])
     return out
+
+
+def linear_relu2(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """``max(x @ weight.T, 0)^2`` in the run dtype: inside the product's kernel for few bfloat16 rows, else by a kernel
+    behind it."""
+    m, k = x.shape
+    if (weight.dtype == torch.bfloat16 and weight.is_cuda and x.dtype == torch.bfloat16 and m <= skinny.ONE_BLOCK_ROWS
+            and skinny.takes_resident(m, k, weight) and _aligned(x)):
+        return skinny.resident_product(weight, x=x, epilogue=skinny.RELU2, out_dtype=torch.bfloat16)
+    from .rownorm import squared_relu_
+    z = linear(x, weight)
+    return squared_relu_(z if z.is_contiguous() else z.contiguous())
 
 
 def _aligned(x: torch.Tensor) -> bool:

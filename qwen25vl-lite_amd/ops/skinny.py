@@ -16,7 +16,7 @@ import torch
 from .kernels import _check, _fn, _ptr, _stream, dtype_code
 
 __all__ = ["resident_product", "takes_resident", "qkv_rope_product", "takes_qkv_rope", "RESIDENT_ROWS", "resident_norm_k", "resident_two_tile_k", "folds_norm", "ONE_BLOCK_ROWS", "split_product", "takes_split", "prefers_split", "SPLIT_ROWS",
-           "takes_stack", "stack_product", "STORE", "RESIDUAL", "SWIGLU", "GEGLU", "GATED"]
+           "takes_stack", "stack_product", "STORE", "RESIDUAL", "SWIGLU", "GEGLU", "RELU2", "GATED"]
 
 RESIDENT_ROWS = 64       # up to here the resident kernel runs
 ONE_TILE_ROWS = 16       # the rows of one column tile of the matrix instruction
@@ -25,7 +25,7 @@ ONE_BLOCK_ROWS = 32      # up to here one block carries all rows: beyond, teams 
 _MAX_WEIGHT_BYTES = 0xffffff00   # qvl_gemm_resident_max_weight_bytes() + 1
 _pass_k = None
 _two_tile_k = None
-STORE, RESIDUAL, SWIGLU, GEGLU = 0, 1, 2, 4
+STORE, RESIDUAL, SWIGLU, GEGLU, RELU2 = 0, 1, 2, 4, 5
 GATED = {"silu": SWIGLU, "gelu_tanh": GEGLU}
 _c_int, _c_float, _c_ptr = ctypes.c_int, ctypes.c_float, ctypes.c_void_p
 _cu_count = {}
@@ -109,7 +109,8 @@ def resident_product(weight: torch.Tensor, *, x: Optional[torch.Tensor] = None, 
     formed inside the kernel from the float32 rows ``h``.  ``epilogue``: ``STORE`` writes the product
     (plus ``bias``) to ``out``, or to a new tensor, of ``out_dtype``; ``RESIDUAL`` adds it to ``out`` (float32) in
     place; ``SWIGLU`` takes ``weight``'s rows as groups of 8 gate, 8 up rows and returns
-    ``silu(gate) * up`` as bfloat16 ``[M, N/2]`` (``GEGLU``: with the tanh form of gelu)."""
+    ``silu(gate) * up`` as bfloat16 ``[M, N/2]`` (``GEGLU``: with the tanh form of gelu);
+    ``RELU2`` stores the square of relu of the product."""
     src = x if x is not None else h
     m, k = src.shape
     n = weight.shape[0]

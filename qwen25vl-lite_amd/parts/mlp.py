@@ -168,13 +168,13 @@ class PlainFF(FeedForward):
 
     def forward(self, x, step: StepContext):
         from ..ops import rownorm
-        from ..ops.linear import linear
+        from ..ops.linear import linear, linear_relu2
 
-        z = linear(x, self.w_up)
-        z = z if z.is_contiguous() else z.contiguous()
         if self.activation == "relu2":
-            act = rownorm.squared_relu_(z)
+            act = linear_relu2(x, self.w_up)
         else:
+            z = linear(x, self.w_up)
+            z = z if z.is_contiguous() else z.contiguous()
             act = rownorm.normed_powers(z, self.coeff, self.eps, self.dtype)
         return linear_into(step.residual if step is not None else None, act, self.w_down)
 
