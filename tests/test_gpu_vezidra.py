@@ -406,15 +406,18 @@ def test_one_key_just_inside_and_just_outside_a_window(shape, dtype, tmp_path):
     m = vu.heads(2, 1, d, dv, 50.0, 0, 1.0, window=window)
 
     def edit(t):
+        # every query is one direction; a key has it where the input's second channel says so
         t["l0.mix.sink"] = torch.full((2,), -40.0).to(torch.bfloat16)
+        t["l0.mix.q"].zero_()
+        t["l0.mix.q"][::d, 0] = 1.0
+        t["l0.mix.k"][:, :2] = 0.0
+        t["l0.mix.k"][::d, 1] = 20.0
     runner, model, cfg, t = _one_layer(tmp_path, vu.layer(vu.attention(m)), dtype, tensors_edit=edit)
     torch.manual_seed(3)
     n = 60
-    x = 0.1 * torch.randn(n, 56)
-    # every query looks for the loud token's key: all inputs share the direction that makes it, the loud one by far the most
-    direction = torch.linalg.pinv(t["l0.mix.q"]) @ t["l0.mix.k"].mean(dim=1).repeat(2)
-    x = x + (direction / direction.norm()).float()
-    x[loud] = torch.randn(56) * 3
+    x = torch.randn(n, 56)
+    x[:, 0], x[:, 1] = 1.0, 0.0
+    x[loud, 1] = 1.0
     mixer = model.blocks[0].mixer
     store = plain._keep if dtype == torch.float32 else plain.to_bfloat16_and_back
     call = lambda x, step, slot: mixer.forward(x, step, slot.of("mix"))
@@ -423,11 +426,11 @@ def test_one_key_just_inside_and_just_outside_a_window(shape, dtype, tmp_path):
                     + [_run_mixer(runner, call, [("a", 1, p)], x[p:p + 1]) for p in range(20, n)])
     tol = (2e-5 if dtype == torch.float32 else 4e-2) * want.abs().max().item()
     assert torch.allclose(got, want, atol=tol)
-    # a window one token shorter or longer moves exactly the rows at its edge
+    # a window one token shorter or longer moves the row at its edge
     for other in (window - 1, window + 1):
         off = plain.attention(store(x.double()), torch.arange(n), t, "l0.mix.", {**m, "mask": {"size": other}}, 1e-4, store)
         edge = loud + min(window, other)
-        assert (off - want).abs().amax(dim=1)[edge] > 4 * tol, other
+        assert (off - want).abs().amax(dim=1)[edge] > 8 * tol, other
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
@@ -488,11 +491,21 @@ def test_float32_every_schedule_against_the_plain_model(name, folders):
     reqs = _requests(cfg["vocab"], seed=20)
     want = {rid: _oracle(folder, toks) for rid, toks in reqs.items()}
     mixed, peak = mixed_trace(reqs, seed=4, max_live=4)
+    # a root mean square over one value is a sign: with heads of one channel float32 arithmetic itself is visible, and the
+    # measure is the plain model run in float32
+    rounding = None
+    if name == "ones":
+        cfg, t32 = plain.vezidra_read(folder, torch.float32)
+        rounding = torch.cat([_rel_rows(plain.vezidra_forward(cfg, t32, toks), want[rid]) for rid, toks in reqs.items()])
     holders = {}
     for steps, size in ((whole_trace(reqs), 192), (tail_trace(reqs, 50), 192), (portion_trace(reqs), 192), (mixed, peak)):
         got = run_steps(_replayer(folder, "float32", size), steps, holders if steps is mixed else None)
-        for rid, toks in reqs.items():
-            assert _rel(_rows(got, rid, len(toks)), want[rid]) < 2e-5, (name, rid)
+        errors = torch.cat([_rel_rows(_rows(got, rid, len(toks)), want[rid]) for rid, toks in reqs.items()])
+        if rounding is None:
+            assert errors.max() < 2e-5, (name, errors.max())
+        else:
+            assert _like_rounding(errors, rounding, 1e-6), (errors.median(), rounding.median(), errors.quantile(0.9), rounding.quantile(0.9))
+            assert errors.max() < 4 * rounding.max() + 1e-5, (errors.max(), rounding.max())
     assert any(len(who) > 1 for who in holders.values()), "no page was used by two requests"
 
 
@@ -681,7 +694,7 @@ def test_the_replay_program_and_the_command_line(dtype, folders, tmp_path):
     s0 = torch.from_numpy(np.fromfile(out / "0.f32", dtype="<f4").reshape(2, vocab))
     s2 = torch.from_numpy(np.fromfile(out / "2.f32", dtype="<f4").reshape(2, vocab))
     rounding = _rel_rows(_oracle(folder, toks, plain.to_bfloat16_and_back), want)[[0, 18, 44, 2]]
-    limit = torch.full((4,), 2e-5) if dtype == "float32" else 2 * rounding + 4e-3
+    limit = torch.full((4,), 2e-5) if dtype == "float32" else 3 * rounding + 4e-3
     assert (_rel_rows(torch.cat([s0, s2]), want[[0, 18, 44, 2]]) < limit).all()
     if dtype == "float32":
         prompt = toks[:12]
