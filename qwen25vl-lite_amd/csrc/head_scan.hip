@@ -19,7 +19,7 @@
 //   hs_prep    sums of logarithms and gates per (chunk, head)
 //   hs_score   Q K^T (and K K^T) per (chunk, group), unit lengths folded in
 //   hs_solve   [Wv | Wk] per (chunk, head), a triangular system in blocks of 16 rows        (delta)
-//   hs_carry   the states, chunk after chunk; a block per (request, head, 16 value channels); leaves S' and U of every chunk
+//   hs_carry   the states, chunk after chunk; a block per (request, head, 16 value channels); leaves S' (delta: and U) of every chunk
 //   hs_out     O per (chunk, head)
 //
 // Matrix fragments.  Lane l of a wave stands for row (or column) l % 16 and the four inner indices 4 (l / 16) .. + 3 of a
@@ -66,9 +66,10 @@ struct HeadScan {
   float* tail;               // [chunks, H, 64]: the decays' product behind the token to the chunk's end
   float* qk;                 // [chunks, G, 64, 64]
   float* kk;                 // [chunks, G, 64, 64]
+  void* kt;                  // [chunks, G, HS_KB, 4, 64, 4] of TX: K as left operand with channels as rows
   float* unit;               // [chunks, G, 2, 64]: factors on q (its scale included) and k
   float* wk;                 // [chunks, H, 64, HS_DIMP]
-  float* u;                  // [chunks, H, vtiles, 4, 64, 4]
+  float* u;                  // [chunks, H, vtiles, 4, 64, 4] (delta)
   float* s0;                 // [chunks, H, vtiles, HS_KB, 64, 4]
 };
 
@@ -110,7 +111,7 @@ __global__ __launch_bounds__(256) void hs_scan_kernel(HeadScan a) {
     float vt[HS_TB];
 #pragma unroll
     for (int t = 0; t < HS_TB; ++t)
-      vt[t] = live && t < nt ? ldf<TX>(x + (size_t)(t0 + t) * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol) : 0.f;
+      vt[t] = ldf<TX>(x + (size_t)(t0 + (t < nt ? t : 0)) * a.x_stride + a.v_off + (size_t)head * a.vdim + (live ? vcol : 0));
     if (tid < nt) {
       const float* r = a.raw + (size_t)(t0 + tid) * a.raw_stride;
       const float step = hs_softplus(r[a.a_off + head] + bias);
@@ -182,6 +183,14 @@ __global__ __launch_bounds__(256) void hs_scan_kernel(HeadScan a) {
 #if HS_CHUNKED
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
+// exp(l) of a difference of sums of logarithms, which is not positive where it counts.  Formed whether or not it is
+// used: a branch around it would wait for its operands one by one.
+__device__ __forceinline__ float decay_of(double l) {
+  float e = expf(fminf((float)l, 0.f));
+  asm volatile("" : "+v"(e));
+  return e;
+}
+
 // acc += A B over one block of 16 inner indices
 __device__ __forceinline__ f32x4 mma16(const f32x4 p, const f32x4 q, f32x4 acc) {
 #pragma unroll
@@ -219,12 +228,14 @@ __global__ __launch_bounds__(256) void hs_prep_kernel(HeadScan a) {
 
 // Four channels of a row as they lie in memory.  VEC: HS_DIM, strides and offsets are multiples of four and rows lie on
 // boundaries of four values, so that one load fetches them.
+// `at`: where channel d lies, or channel 0 with d past the last one.
 template <typename TX, bool VEC> struct Four {
   TX v[4];
-  __device__ __forceinline__ void fetch(const TX* row, int d) {
+  __device__ __forceinline__ void fetch_at(const TX* at, int d) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) v[j] = row[d + j < HS_DIM ? d + j : 0];
+    for (int j = 0; j < 4; ++j) v[j] = at[d + j < HS_DIM ? j : 0];
   }
+  __device__ __forceinline__ void fetch(const TX* row, int d) { fetch_at(row + (d < HS_DIM ? d : 0), d); }
   __device__ __forceinline__ f32x4 value(int d, bool live) const {
     f32x4 o;
 #pragma unroll
@@ -234,16 +245,30 @@ template <typename TX, bool VEC> struct Four {
 };
 template <> struct Four<bf16_t, true> {
   uint2 v;
-  __device__ __forceinline__ void fetch(const bf16_t* row, int d) { v = *reinterpret_cast<const uint2*>(row + (d < HS_DIM ? d : 0)); }
-  __device__ __forceinline__ f32x4 value(int d, bool live) const {
-    if (!live || d >= HS_DIM) return f32x4{0.f, 0.f, 0.f, 0.f};
+  // of values that are bfloat16 already
+  __device__ __forceinline__ void set(const f32x4& w) {
+    v.x = (__float_as_uint(w[0]) >> 16) | (__float_as_uint(w[1]) & 0xffff0000u);
+    v.y = (__float_as_uint(w[2]) >> 16) | (__float_as_uint(w[3]) & 0xffff0000u);
+  }
+  __device__ __forceinline__ f32x4 all() const {
     return f32x4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
                  __uint_as_float(v.y & 0xffff0000u)};
+  }
+  __device__ __forceinline__ void store(bf16_t* at) const { *reinterpret_cast<uint2*>(at) = v; }
+  __device__ __forceinline__ void fetch_at(const bf16_t* at, int) { v = *reinterpret_cast<const uint2*>(at); }
+  __device__ __forceinline__ void fetch(const bf16_t* row, int d) { fetch_at(row + (d < HS_DIM ? d : 0), d); }
+  __device__ __forceinline__ f32x4 value(int d, bool live) const {
+    if (!live || d >= HS_DIM) return f32x4{0.f, 0.f, 0.f, 0.f};
+    return all();
   }
 };
 template <> struct Four<float, true> {
   f32x4 v;
-  __device__ __forceinline__ void fetch(const float* row, int d) { v = *reinterpret_cast<const f32x4*>(row + (d < HS_DIM ? d : 0)); }
+  __device__ __forceinline__ void set(const f32x4& w) { v = w; }
+  __device__ __forceinline__ f32x4 all() const { return v; }
+  __device__ __forceinline__ void store(float* at) const { *reinterpret_cast<f32x4*>(at) = v; }
+  __device__ __forceinline__ void fetch_at(const float* at, int) { v = *reinterpret_cast<const f32x4*>(at); }
+  __device__ __forceinline__ void fetch(const float* row, int d) { fetch_at(row + (d < HS_DIM ? d : 0), d); }
   __device__ __forceinline__ f32x4 value(int d, bool live) const { return live && d < HS_DIM ? v : f32x4{0.f, 0.f, 0.f, 0.f}; }
 };
 
@@ -289,6 +314,16 @@ __global__ __launch_bounds__(256) void hs_score_kernel(HeadScan a) {
   if (tid < 2 * HS_CHUNK) a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + tid] = f[tid >> 6][tid & 63];
   const int col = lane & 15, lg = lane >> 4;
   const size_t base = ((size_t)c * a.G + grp) * HS_CHUNK * HS_CHUNK;
+  TX* kt = reinterpret_cast<TX*>(a.kt) + (((size_t)c * a.G + grp) * HS_KB * 4 * 64 + lane) * 4;
+#pragma unroll 4
+  for (int i = wave; i < HS_KB * 4; i += 4) {   // a block of 16 channels and a block of 16 tokens
+    Four<TX, true> o;
+    f32x4 v;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = k[((i & 3) * 16 + 4 * lg + j) * HS_LD + (i >> 2) * 16 + col];
+    o.set(v);
+    o.store(kt + (size_t)i * 256);
+  }
   // ten tiles on or below the diagonal: tile number i is (row, column) of the list, shared among the waves
   for (int i = wave; i < 10; i += 4) {
     const int rt = i < 1 ? 0 : (i < 3 ? 1 : (i < 6 ? 2 : 3)), ct = i - rt * (rt + 1) / 2;
@@ -316,10 +351,10 @@ template <typename TX>
 __global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
   __shared__ __attribute__((aligned(16))) float A[HS_CHUNK][HS_CHUNK + 4];   // strictly below the diagonal
   __shared__ __attribute__((aligned(16))) float T[4][16][20];                // inverses of the diagonal blocks
-  __shared__ float rv[HS_CHUNK], rk[HS_CHUNK];                               // factors on the rows of V and K
+  __shared__ __attribute__((aligned(16))) float rv[HS_CHUNK], rk[HS_CHUNK];                               // factors on the rows of V and K
   __shared__ double ls[HS_CHUNK];
   const int c = blockIdx.x, head = blockIdx.y, grp = head / (a.H / a.G);
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, lg = lane >> 4;
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, lg = lane >> 4;
   const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
   const size_t ch = (size_t)c * a.H + head;
   const float* kk = a.kk + ((size_t)c * a.G + grp) * HS_CHUNK * HS_CHUNK;
@@ -337,12 +372,10 @@ __global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int row = (tid >> 4) + 16 * i, j0 = (tid & 15) * 4;
-    f32x4 v = {0.f, 0.f, 0.f, 0.f};
-    if (j0 < row) {
+    f32x4 v;
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (j0 + j < row) v[j] = rv[row] * expf((float)(ls[row] - ls[j0 + j])) * prod[i][j];
-    }
+    for (int j = 0; j < 4; ++j)
+      v[j] = j0 + j < row ? rv[row] * decay_of(ls[row] - ls[j0 + j]) * prod[i][j] : 0.f;
     *reinterpret_cast<f32x4*>(&A[row][j0]) = v;
   }
   __syncthreads();
@@ -367,25 +400,39 @@ __global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
     for (int j = 0; j < i; ++j) low[i * (i - 1) / 2 + j] = -*reinterpret_cast<const f32x4*>(&A[i * 16 + col][j * 16 + 4 * lg]);
   }
   const TX* x = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride;
-  const int vtiles = (a.vdim + 15) / 16;
-  for (int tile = wave; tile < vtiles + HS_KB; tile += 4) {
+  const int vtiles = (a.vdim + 15) / 16, tiles = vtiles + HS_KB;
+  // a tile's values as they lie in memory, asked for a tile ahead; what lies outside is read from inside and not counted
+  TX raw[16];
+  auto ask = [&](int tile) {
     const bool values = tile < vtiles;
     const int cc = (values ? tile : tile - vtiles) * 16 + col;
-    const bool in = values ? cc < a.vdim : cc < HS_DIM;
-    const TX* src = x + (values ? a.v_off + (size_t)head * a.vdim : a.k_off + (size_t)grp * HS_DIM) + (in ? cc : 0);
+    const TX* src = x + (values ? a.v_off + (size_t)head * a.vdim : a.k_off + (size_t)grp * HS_DIM) +
+                    (cc < (values ? a.vdim : HS_DIM) ? cc : 0);
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const int t = (i >> 2) * 16 + 4 * lg + (i & 3);
+      raw[i] = src[(size_t)(t < n ? t : 0) * a.x_stride];
+    }
+  };
+  if (wave < tiles) ask(wave);
+  for (int tile = wave; tile < tiles; tile += 4) {
+    const bool values = tile < vtiles;
+    const int cc = (values ? tile : tile - vtiles) * 16 + col;
+    const bool in = cc < (values ? a.vdim : HS_DIM);
+    const float* factor = values ? rv : rk;
     f32x4 y[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
+      y[i] = *reinterpret_cast<const f32x4*>(factor + i * 16 + 4 * lg);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int t = i * 16 + 4 * lg + r;
-        y[i][r] = in && t < n ? ldf<TX>(src + (size_t)t * a.x_stride) : 0.f;
+        const float v = y[i][r] * ldf<TX>(raw + i * 4 + r);
+        y[i][r] = in && i * 16 + 4 * lg + r < n ? v : 0.f;
       }
     }
+    if (tile + 4 < tiles) ask(tile + 4);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) y[i][r] *= values ? rv[i * 16 + 4 * lg + r] : rk[i * 16 + 4 * lg + r];
 #pragma unroll
       for (int j = 0; j < i; ++j) y[i] = mma16(low[i * (i - 1) / 2 + j], y[j], y[i]);
       y[i] = mma16(inv[i], y[i], f32x4{0.f, 0.f, 0.f, 0.f});
@@ -407,11 +454,14 @@ __global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
 // ---------------------------------------------------------------------------------------
 // The states from chunk to chunk: a block per (16 value channels, head, request)
 // ---------------------------------------------------------------------------------------
+#ifndef HS_WIDE_CARRY
+#define HS_WIDE_CARRY 0                         // plain rule: 1 stages a chunk's keys once for two tiles of value channels
+#endif
 #define HS_MT ((HS_KB + 3) / 4)                 // row blocks of S a wave keeps: wave w has blocks w, w + 4, ...
 
-// What a block reads of a chunk, asked for a chunk ahead: nothing here is waited for before it is used.
-template <typename TX, bool DELTA, bool VEC, int NV> struct CarryLoads {
-  Four<TX, VEC> k[HS_KB];
+// What a block reads of a chunk, asked for two chunks ahead: nothing here is waited for before it is used.
+template <typename TX, bool DELTA, int NV> struct CarryLoads {
+  Four<TX, true> k[HS_MT][4];
   f32x4 wk[DELTA ? HS_KB : 1];
   f32x4 u[DELTA ? NV : 1];
   TX v[DELTA ? 1 : NV][4];
@@ -421,16 +471,23 @@ template <typename TX, bool DELTA, bool VEC, int NV> struct CarryLoads {
 };
 
 // NV neighbouring tiles of 16 value channels a block
-template <typename TX, bool DELTA, bool VEC, int NV>
+template <typename TX, bool DELTA, int NV>
 __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
-  __shared__ __attribute__((aligned(16))) float k[HS_CHUNK * HS_LD];   // the chunk's keys
+  __shared__ f32x4 us_place[2][NV][4 * 64];     // U, weighted by what is left of it at the chunk's end; two places, taken in turn
   __shared__ f32x4 s[NV][HS_KB * 64];           // S as right operand
-  __shared__ f32x4 us[NV][4 * 64];              // U, weighted by what is left of it at the chunk's end
-  const int head = blockIdx.y, req = blockIdx.z, grp = head / (a.H / a.G);
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, lg = lane >> 4;
-  const int vtiles = (a.vdim + 15) / 16, vt0 = blockIdx.x * NV;
-  const int first = a.req_first[req], last = a.req_first[req + 1];
+  __shared__ float left[2];                     // what a chunk leaves of the state before it
+  // Workgroups go to the 8 XCDs in turn: numbered so that an XCD gets neighbouring tiles and heads, whose blocks read the
+  // same keys and Wk, so that these come into its L2 once.
+  const int vtiles = (a.vdim + 15) / 16, across = (vtiles + NV - 1) / NV;
+  const int item = (blockIdx.x & 7) * (gridDim.x >> 3) + (blockIdx.x >> 3);
+  if (item >= across * a.H) return;
+  const int head = item / across, vt0 = item % across * NV, req = blockIdx.y, grp = head / (a.H / a.G);
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, lg = lane >> 4;
+  const int first = __builtin_amdgcn_readfirstlane(a.req_first[req]), last = __builtin_amdgcn_readfirstlane(a.req_first[req + 1]);
   if (first >= last) return;
+  // a run's chunks follow one another and all but the last are full
+  const int run_begin = __builtin_amdgcn_readfirstlane(a.bounds[first]), run_end = __builtin_amdgcn_readfirstlane(a.bounds[last]);
+  static_assert(HS_CHUNK == 64, "four blocks of 16 tokens");
   float* slot = a.state + ((size_t)a.row_of[req] * a.H + head) * HS_DIM * a.vdim;
   f32x4 S[NV][HS_MT];
 #pragma unroll
@@ -447,18 +504,25 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
   }
   const TX* x = reinterpret_cast<const TX*>(a.x);
   const int t_own = wave * 16 + 4 * lg;         // the first of this lane's four rows of U
-  CarryLoads<TX, DELTA, VEC, NV> l;
-  auto ask_keys = [&](int c) {
-    const int begin = a.bounds[c];
-    l.n = a.bounds[c + 1] - begin;
-    const TX* row0 = x + (size_t)begin * a.x_stride + a.k_off + (size_t)grp * HS_DIM;
+  typedef CarryLoads<TX, DELTA, NV> Loads;
+  // places of values within a chunk, in bytes from its first token's: the same for every chunk
+  unsigned v_at[NV][4];
 #pragma unroll
-    for (int i = 0; i < HS_KB; ++i) {
-      const int idx = tid + 256 * i, t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
-      l.k[i].fetch(row0 + (size_t)(t < l.n ? t : 0) * a.x_stride, d);
+  for (int v = 0; v < NV; ++v) {
+    const int vcol = (vt0 + v) * 16 + col;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) v_at[v][r] = (unsigned)(((t_own + r) * (int)a.x_stride + (vcol < a.vdim ? vcol : 0)) * (int)sizeof(TX));
+  }
+  auto ask_keys = [&](Loads& l, int c) {
+    const TX* kt = reinterpret_cast<const TX*>(a.kt) + (((size_t)c * a.G + grp) * HS_KB * 4 * 64 + lane) * 4;
+#pragma unroll
+    for (int m = 0; m < HS_MT; ++m) {
+      const int b = wave + 4 * m;
+#pragma unroll
+      for (int tb = 0; tb < 4; ++tb) l.k[m][tb].fetch_at(kt + (size_t)((HS_KB % 4 == 0 || b < HS_KB ? b : 0) * 4 + tb) * 256, 0);
     }
   };
-  auto ask_rest = [&](int c) {
+  auto ask_rest = [&](Loads& l, int c) {
     const size_t ch = (size_t)c * a.H + head;
     l.tail = *reinterpret_cast<const f32x4*>(a.tail + ch * HS_CHUNK + t_own);
     l.unit = *reinterpret_cast<const f32x4*>(a.unit + (((size_t)c * a.G + grp) * 2 + 1) * HS_CHUNK + t_own);
@@ -469,43 +533,33 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
       for (int b = 0; b < HS_KB; ++b) l.wk[DELTA ? b : 0] = *reinterpret_cast<const f32x4*>(wk + b * 16);
 #pragma unroll
       for (int v = 0; v < NV; ++v)
-        if (vt0 + v < vtiles) l.u[DELTA ? v : 0] = *reinterpret_cast<const f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4);
+        if (NV == 1 || vt0 + v < vtiles) l.u[DELTA ? v : 0] = *reinterpret_cast<const f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4);
     } else {
       l.gate = *reinterpret_cast<const f32x4*>(a.gate + ch * HS_CHUNK + t_own);
-      const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
+      const int begin = run_begin + (c - first) * HS_CHUNK, n = run_end - begin < HS_CHUNK ? run_end - begin : HS_CHUNK;
+      l.n = n;
+      const char* base = reinterpret_cast<const char*>(x + (size_t)begin * a.x_stride + a.v_off + (size_t)head * a.vdim);
 #pragma unroll
-      for (int v = 0; v < NV; ++v) {
-        const int vcol = (vt0 + v) * 16 + col;
-        const TX* src = x + (size_t)begin * a.x_stride + a.v_off + (size_t)head * a.vdim + (vcol < a.vdim ? vcol : 0);
+      for (int v = 0; v < NV; ++v)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) l.v[DELTA ? 0 : v][r] = src[(size_t)(t_own + r < n ? t_own + r : 0) * a.x_stride];
-      }
+        for (int r = 0; r < 4; ++r)
+          l.v[DELTA ? 0 : v][r] = *reinterpret_cast<const TX*>(base + (t_own + r < n ? v_at[v][r] : 0u));
     }
   };
-  ask_keys(first);
-  ask_rest(first);
-  for (int c = first; c < last; ++c) {
+  // The order of a step's memory operations is that in which they are waited for: what the next step needs first is asked
+  // for first, and the stores, which nobody waits for, come last.
+  auto step = [&](Loads& l, int c) {
     const size_t ch = (size_t)c * a.H + head;
-    const int n = l.n;
+    const int n = DELTA ? 0 : l.n, next = c + 2 < last ? c + 2 : last - 1;      // the last two ask for the last chunk again
+    f32x4 (*us)[4 * 64] = us_place[c & 1];
+    if (DELTA) {
 #pragma unroll
-    for (int i = 0; i < HS_KB; ++i) {
-      const int idx = tid + 256 * i, t = idx / (HS_DIMP / 4), d = idx % (HS_DIMP / 4) * 4;
-      *reinterpret_cast<f32x4*>(k + t * HS_LD + d) = l.k[i].value(d, t < n);
+      for (int v = 0; v < NV; ++v)
+#pragma unroll
+        for (int m = 0; m < HS_MT; ++m)
+          if (HS_KB % 4 == 0 || wave + 4 * m < HS_KB) s[v][(wave + 4 * m) * 64 + lane] = S[v][m];
+      __syncthreads();
     }
-    if (c + 1 < last) ask_keys(c + 1);
-#pragma unroll
-    for (int v = 0; v < NV; ++v) {
-      float* s0 = a.s0 + ((ch * vtiles + vt0 + v) * HS_KB * 64 + lane) * 4;
-#pragma unroll
-      for (int m = 0; m < HS_MT; ++m) {
-        const int b = wave + 4 * m;
-        if (b < HS_KB) {
-          if (DELTA) s[v][b * 64 + lane] = S[v][m];
-          if (vt0 + v < vtiles) *reinterpret_cast<f32x4*>(s0 + (size_t)b * 256) = S[v][m];
-        }
-      }
-    }
-    if (DELTA) __syncthreads();
     f32x4 u[NV];
 #pragma unroll
     for (int v = 0; v < NV; ++v) {
@@ -522,29 +576,53 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) u[v][r] = in && t_own + r < n ? l.gate[r] * ldf<TX>(&l.v[DELTA ? 0 : v][r]) : 0.f;
       }
-      if (vt0 + v < vtiles) *reinterpret_cast<f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4) = u[v];
       us[v][wave * 64 + lane] = u[v] * l.tail * l.unit;
     }
-    const float g = l.end;
-    if (c + 1 < last) ask_rest(c + 1);
-    __syncthreads();
+    if (tid == 0) left[c & 1] = l.end;
+    ask_rest(l, next);
 #pragma unroll
-    for (int m = 0; m < HS_MT; ++m) {
-      const int b = wave + 4 * m;
-      if (b < HS_KB) {
+    for (int v = 0; v < NV; ++v) {
+      if (NV > 1 && vt0 + v >= vtiles) continue;
+      float* s0 = a.s0 + ((ch * vtiles + vt0 + v) * HS_KB * 64 + lane) * 4;
 #pragma unroll
-        for (int v = 0; v < NV; ++v) S[v][m] *= g;
-#pragma unroll
-        for (int tb = 0; tb < 4; ++tb) {
-          f32x4 kt;
-#pragma unroll
-          for (int j = 0; j < 4; ++j) kt[j] = k[(tb * 16 + 4 * lg + j) * HS_LD + b * 16 + col];
-#pragma unroll
-          for (int v = 0; v < NV; ++v) S[v][m] = mma16(kt, us[v][tb * 64 + lane], S[v][m]);
-        }
-      }
+      for (int m = 0; m < HS_MT; ++m)
+        if (HS_KB % 4 == 0 || wave + 4 * m < HS_KB) *reinterpret_cast<f32x4*>(s0 + (size_t)(wave + 4 * m) * 256) = S[v][m];
+      if (DELTA) *reinterpret_cast<f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4) = u[v];
     }
-    __syncthreads();                            // the staged keys, S and U have been read
+    __syncthreads();
+    f32x4 ur[NV][4];
+#pragma unroll
+    for (int v = 0; v < NV; ++v)
+#pragma unroll
+      for (int tb = 0; tb < 4; ++tb) ur[v][tb] = us[v][tb * 64 + lane];
+    const float g = left[c & 1];
+#pragma unroll
+    for (int m = 0; m < HS_MT; ++m)
+#pragma unroll
+      for (int v = 0; v < NV; ++v) S[v][m] *= g;
+#pragma unroll
+    for (int tb = 0; tb < 4; ++tb) {
+      f32x4 kt[HS_MT];
+#pragma unroll
+      for (int m = 0; m < HS_MT; ++m) kt[m] = l.k[m][tb].all();
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int m = 0; m < HS_MT; ++m)
+#pragma unroll
+          for (int v = 0; v < NV; ++v) S[v][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[m][j], ur[v][tb][j], S[v][m], 0, 0, 0);
+    }
+    ask_keys(l, next);
+  };
+  Loads even, odd;
+  ask_keys(even, first);
+  ask_rest(even, first);
+  ask_keys(odd, first + 1 < last ? first + 1 : first);
+  ask_rest(odd, first + 1 < last ? first + 1 : first);
+  for (int c = first; c < last; c += 2) {
+    step(even, c);
+    if (c + 1 >= last) break;
+    step(odd, c + 1);
   }
 #pragma unroll
   for (int v = 0; v < NV; ++v) {
@@ -563,80 +641,103 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
 }
 
 // ---------------------------------------------------------------------------------------
-// O of a (chunk, head): wave w has the token rows 16 w .. 16 w + 15
+// O of a (chunk, head): wave w forms the tiles of 16 value channels w, w + 4, ... of all 64 tokens, so that S' and U are
+// read once; the left operands, the same for all tiles, lie in LDS as fragments.
 // ---------------------------------------------------------------------------------------
-template <typename TX, bool VEC>
-__global__ __launch_bounds__(256) void hs_out_kernel(HeadScan a) {
+template <typename TX, bool DELTA, bool VEC>
+__global__ __launch_bounds__(256, HS_DIMP <= 128 ? 3 : 2) void hs_out_kernel(HeadScan a) {
+  __shared__ f32x4 qf[4][HS_KB][64];            // diag(L_i0) Q
+  __shared__ f32x4 pf[10][64];                  // L o Q K^T, tile (row, column) at row (row + 1) / 2 + column
+  __shared__ double ls[HS_CHUNK];
   const int c = blockIdx.x, head = blockIdx.y, grp = head / (a.H / a.G);
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, col = lane & 15, lg = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, col = lane & 15, lg = lane >> 4;
   const int begin = a.bounds[c], n = a.bounds[c + 1] - begin;
-  if (wave * 16 >= n) return;
   const size_t ch = (size_t)c * a.H + head;
-  const double* ls = a.lsum + ch * HS_CHUNK;
-  const TX* xr = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride;
-  const int row = wave * 16 + col;              // of the left operands
-  Four<TX, VEC> qraw[HS_KB];
-  const TX* qr = xr + (size_t)(row < n ? row : 0) * a.x_stride + a.q_off + (size_t)grp * HS_DIM;
-#pragma unroll
-  for (int b = 0; b < HS_KB; ++b) qraw[b].fetch(qr, b * 16 + 4 * lg);
-  const float f = a.head[ch * HS_CHUNK + row] * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + row];
-  const double mine = ls[row];
-  f32x4 p[4];
-#pragma unroll
-  for (int jb = 0; jb < 4; ++jb) {
-    p[jb] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (jb <= wave) {
-      const f32x4 sc = *reinterpret_cast<const f32x4*>(a.qk + (((size_t)c * a.G + grp) * HS_CHUNK + row) * HS_CHUNK + jb * 16 + 4 * lg);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int t = jb * 16 + 4 * lg + j;
-        if (t <= row) p[jb][j] = sc[j] * expf((float)(mine - ls[t]));
-      }
-    }
-  }
-  f32x4 q[HS_KB];
-#pragma unroll
-  for (int b = 0; b < HS_KB; ++b) q[b] = qraw[b].value(b * 16 + 4 * lg, row < n) * f;
-  const float skip = a.skip ? a.skip[head] : 0.f;
-  const int vtiles = (a.vdim + 15) / 16;
+  const int vtiles = (a.vdim + 15) / 16, row_tiles = (n + 15) / 16;
   const f32x4* s0 = reinterpret_cast<const f32x4*>(a.s0) + ch * vtiles * HS_KB * 64 + lane;
   const f32x4* ug = reinterpret_cast<const f32x4*>(a.u) + ch * vtiles * 4 * 64 + lane;
-  // two tiles of value channels at a time; the last of an odd number is formed twice
-  for (int vt = 0; vt < vtiles; vt += 2) {
-    const int other = vt + 1 < vtiles ? vt + 1 : vt;
-    f32x4 o[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+  const TX* xr = reinterpret_cast<const TX*>(a.x) + (size_t)begin * a.x_stride;
+  const float* gate = a.gate + ch * HS_CHUNK;
+  constexpr int AHEAD = HS_KB <= 4 ? HS_KB : 4; // blocks of S' asked for together
+  f32x4 sv[AHEAD];
 #pragma unroll
-    for (int b = 0; b < HS_KB; ++b) {
-      const f32x4 s_a = s0[(vt * HS_KB + b) * 64], s_b = s0[(other * HS_KB + b) * 64];
+  for (int b = 0; b < AHEAD; ++b) sv[b] = s0[((wave < vtiles ? wave : 0) * HS_KB + b) * 64];
+  {
+    const int row = wave * 16 + col;
+    const TX* qr = xr + (size_t)(row < n ? row : 0) * a.x_stride + a.q_off + (size_t)grp * HS_DIM;
+    Four<TX, VEC> qraw[HS_KB];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[b][j], s_a[j], o[0], 0, 0, 0);
-        o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[b][j], s_b[j], o[1], 0, 0, 0);
-      }
-    }
+    for (int b = 0; b < HS_KB; ++b) qraw[b].fetch(qr, b * 16 + 4 * lg);
+    const float f = a.head[ch * HS_CHUNK + row] * a.unit[((size_t)c * a.G + grp) * 2 * HS_CHUNK + row];
+    const float* qk = a.qk + (((size_t)c * a.G + grp) * HS_CHUNK + row) * HS_CHUNK + 4 * lg;
+    f32x4 sc[4];
+#pragma unroll
+    for (int jb = 0; jb < 4; ++jb) sc[jb] = *reinterpret_cast<const f32x4*>(qk + (jb <= wave ? jb : 0) * 16);
+    if (threadIdx.x < HS_CHUNK) ls[threadIdx.x] = a.lsum[ch * HS_CHUNK + threadIdx.x];
+    __syncthreads();
+    const double mine = ls[row];
 #pragma unroll
     for (int jb = 0; jb < 4; ++jb) {
       if (jb <= wave) {
-        const f32x4 u_a = ug[(vt * 4 + jb) * 64], u_b = ug[(other * 4 + jb) * 64];
+        f32x4 p;
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[jb][j], u_a[j], o[0], 0, 0, 0);
-          o[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[jb][j], u_b[j], o[1], 0, 0, 0);
+          const int t = jb * 16 + 4 * lg + j;
+          p[j] = t <= row ? sc[jb][j] * decay_of(mine - ls[t]) : 0.f;
         }
+        pf[wave * (wave + 1) / 2 + jb][lane] = p;
       }
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int vcol = (vt + i) * 16 + col;
-      if (vcol < a.vdim) {
+    for (int b = 0; b < HS_KB; ++b) qf[wave][b][lane] = qraw[b].value(b * 16 + 4 * lg, row < n) * f;
+  }
+  const float skip = a.skip ? a.skip[head] : 0.f;
+  __syncthreads();
+  for (int vt = wave; vt < vtiles; vt += 4) {
+    asm volatile("" ::: "memory");              // the fragments are read from LDS for every tile, not kept in registers
+    const int vcol = vt * 16 + col;
+    const bool in = vcol < a.vdim;
+    const TX* vr = xr + a.v_off + (size_t)head * a.vdim + (in ? vcol : 0);
+    f32x4 u[4], v[4], o[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+      v[i] = o[i];
+      if (DELTA) u[i] = ug[(vt * 4 + i) * 64];
+      if (!DELTA || a.skip) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int t = wave * 16 + 4 * lg + r;
-          if (t < n) {
-            float v = o[i][r];
-            if (a.skip) v += skip * ldf<TX>(xr + (size_t)t * a.x_stride + a.v_off + (size_t)head * a.vdim + vcol);
-            a.out[((size_t)(begin + t) * a.H + head) * a.vdim + vcol] = v;
-          }
+          const int t = i * 16 + 4 * lg + r;
+          const float x = ldf<TX>(vr + (size_t)(t < n ? t : 0) * a.x_stride);
+          v[i][r] = in && t < n ? x : 0.f;
+        }
+      }
+      if (!DELTA) u[i] = v[i] * *reinterpret_cast<const f32x4*>(gate + i * 16 + 4 * lg);
+    }
+#pragma unroll
+    for (int b = 0; b < HS_KB; ++b) {
+      const f32x4 sb = sv[b % AHEAD];
+      if (b + AHEAD < HS_KB) sv[b % AHEAD] = s0[(vt * HS_KB + b + AHEAD) * 64];
+      else if (vt + 4 < vtiles) sv[b % AHEAD] = s0[((vt + 4) * HS_KB + b + AHEAD - HS_KB) * 64];
+      f32x4 q[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) q[i] = qf[i][b][lane];
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[i][j], sb[j], o[i], 0, 0, 0);
+    }
+#pragma unroll
+    for (int jb = 0; jb < 4; ++jb)
+#pragma unroll
+      for (int i = jb; i < 4; ++i) o[i] = mma16(pf[i * (i + 1) / 2 + jb][lane], u[jb], o[i]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      if (i < row_tiles && in) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = i * 16 + 4 * lg + r;
+          if (t < n) a.out[((size_t)(begin + t) * a.H + head) * a.vdim + vcol] = o[i][r] + skip * v[i][r];
         }
       }
     }
@@ -655,7 +756,7 @@ static int fill_args(HeadScan& a, const void* x, long long x_stride, int q_off, 
   if (!x || !raw || !bias || !a_neg || !state || !bounds || !row_of || !out) return QVL_ERR_SHAPE;
   if (q_off < 0 || k_off < 0 || v_off < 0 || a_off < 0) return QVL_ERR_SHAPE;
   if (x_stride < (long long)q_off + (long long)G * HS_DIM || x_stride < (long long)k_off + (long long)G * HS_DIM ||
-      x_stride < (long long)v_off + (long long)H * vdim || raw_stride < (long long)a_off + H || raw_stride < (long long)b_off + H)
+      x_stride < (long long)v_off + (long long)H * vdim || x_stride > 0x7fffffffLL / (HS_CHUNK * 8) || raw_stride < (long long)a_off + H || raw_stride < (long long)b_off + H)
     return QVL_ERR_SHAPE;
   if (H > 65535) return QVL_ERR_LIMIT;
   a = HeadScan{};
@@ -693,8 +794,8 @@ extern "C" int qvl_head_scan(const void* x, long long x_stride, int q_off, int k
 // Floats of scratch memory that qvl_head_scan_chunks needs.
 extern "C" long long qvl_head_scan_scratch(int chunks, int H, int G, int vdim, int delta) {
   const long long vtiles = (vdim + 15) / 16, c = chunks;
-  return c * H * HS_CHUNK * 5 + c * G * (2 * HS_CHUNK + (delta ? 2 : 1) * HS_CHUNK * HS_CHUNK) +
-         (delta ? c * H * HS_CHUNK * HS_DIMP : 0) + c * H * vtiles * (4 + HS_KB) * 256;
+  return c * H * HS_CHUNK * 5 + c * G * (2 * HS_CHUNK + HS_CHUNK * HS_DIMP + (delta ? 2 : 1) * HS_CHUNK * HS_CHUNK) +
+         (delta ? c * H * HS_CHUNK * HS_DIMP : 0) + c * H * vtiles * ((delta ? 4 : 0) + HS_KB) * 256;
 }
 
 // The same in chunks of at most 64 tokens: chunk_cu [chunks + 1], req_first [R + 1] (the first chunk of each request);
@@ -722,23 +823,23 @@ extern "C" int qvl_head_scan_chunks(const void* x, long long x_stride, int q_off
   a.head = at; at += c * H * HS_CHUNK;
   a.tail = at; at += c * H * HS_CHUNK;
   a.unit = at; at += c * G * 2 * HS_CHUNK;
+  a.kt = at; at += c * G * HS_CHUNK * HS_DIMP;
   a.qk = at; at += c * G * HS_CHUNK * HS_CHUNK;
   if (delta) { a.kk = at; at += c * G * HS_CHUNK * HS_CHUNK; }
   if (delta) { a.wk = at; at += c * H * HS_CHUNK * HS_DIMP; }
-  a.u = at; at += c * H * vtiles * 4 * 256;
+  if (delta) { a.u = at; at += c * H * vtiles * 4 * 256; }
   a.s0 = at;
   const bool vec = HS_DIM % 4 == 0 && x_stride % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0 && ((uintptr_t)x & 15) == 0;
-  // plain: a chunk's keys are staged once for two tiles of value channels
-  const int wide = delta || vtiles < 2 ? 1 : 2;
-#define CARRY(TX, D, V, NV)                                                                                          \
-  hipLaunchKernelGGL((hs_carry_kernel<TX, D, V, NV>), dim3((vtiles + NV - 1) / NV, H, R), dim3(256), 0, stream, a)
+  const int wide = HS_WIDE_CARRY && !delta && vtiles > 1 ? 2 : 1;
+#define CARRY(TX, D, NV)                                                                                          \
+  hipLaunchKernelGGL((hs_carry_kernel<TX, D, NV>), dim3((((vtiles + NV - 1) / NV) * H + 7) / 8 * 8, R), dim3(256), 0, stream, a)
 #define LAUNCH(TX, D, V)                                                                                             \
   {                                                                                                                  \
     hipLaunchKernelGGL((hs_prep_kernel<D>), dim3(chunks, (H + 3) / 4), dim3(256), 0, stream, a);                     \
     hipLaunchKernelGGL((hs_score_kernel<TX, D, V>), dim3(chunks, G), dim3(256), 0, stream, a);                       \
     if (D) hipLaunchKernelGGL((hs_solve_kernel<TX>), dim3(chunks, H), dim3(256), 0, stream, a);                      \
-    if (D || wide == 1) CARRY(TX, D, V, 1); else CARRY(TX, false, V, 2);                                             \
-    hipLaunchKernelGGL((hs_out_kernel<TX, V>), dim3(chunks, H), dim3(256), 0, stream, a);                            \
+    if (D || wide == 1) CARRY(TX, D, 1); else CARRY(TX, false, 2);                                             \
+    hipLaunchKernelGGL((hs_out_kernel<TX, D, V>), dim3(chunks, H), dim3(256), 0, stream, a);                            \
   }
 #define BY_VEC(TX, D) { if (vec) LAUNCH(TX, D, true) else LAUNCH(TX, D, false) }
   if (dtype == 0) { if (delta) BY_VEC(float, true) else BY_VEC(float, false) }
