@@ -535,9 +535,17 @@ struct TileInfo {
   int lo_tile, hi_tile;
 };
 
-// One more term in a softmax's denominator, exp(sink) of the query head, relative to the reference m (base 2).
-__device__ __forceinline__ float sink_term(const float* __restrict__ sinks, int head, float m) {
-  return sinks ? __builtin_amdgcn_exp2f(sinks[head] * LOG2E - m) : 0.f;
+// What a head's sums are multiplied by when they are written: one over the denominator `total`, in which a sink may stand
+// (sinks[head], relative to the reference m in base 2), times the sigmoid of the head's gate if there is one.
+struct HeadEnd {
+  const float* sinks;        // [nq] or null
+  const float* gates;        // rows of gate_stride values, one per token: [.., nq], or null
+  long long gate_stride;
+};
+__device__ __forceinline__ float head_end(const HeadEnd& e, int token, int head, float total, float m) {
+  if (e.sinks) total += __builtin_amdgcn_exp2f(e.sinks[head] * LOG2E - m);
+  if (e.gates) total *= 1.0f + __builtin_amdgcn_exp2f(-LOG2E * e.gates[(size_t)token * e.gate_stride + head]);
+  return 1.0f / total;
 }
 
 // A request's run of tokens in this step.  Without the array of run starts every request brings one
@@ -772,7 +780,7 @@ __device__ __forceinline__ void attend_block(BlockShared<GROUPS>& sh, int item, 
                                              const int* __restrict__ cu_q, const int* __restrict__ ctx_len,
                                              const int* __restrict__ blk_req, const int* __restrict__ blk_cb,
                                              bf16_t* __restrict__ out, int nq, int nkv, int ps, int window,
-                                             float scale, const float* __restrict__ sinks) {
+                                             float scale, const HeadEnd& end) {
   const int g = nq / nkv;
   const int wave_of_all = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int group = wave_of_all / BLK_WAVES, wave = wave_of_all % BLK_WAVES;
@@ -930,8 +938,7 @@ __device__ __forceinline__ void attend_block(BlockShared<GROUPS>& sh, int item, 
 #pragma unroll
   for (int i = 0; i < BLK_CT; ++i) {
     if (!t[i].valid) continue;
-    const float total = st[i].acc[NT][0] + sink_term(sinks, t[i].head, st[i].m);
-    const float inv = 1.0f / total;
+    const float inv = head_end(end, t[i].token, t[i].head, st[i].acc[NT][0], st[i].m);
     bf16_t* orow = out + ((size_t)t[i].token * nq + t[i].head) * HD;
 #pragma unroll
     for (int dt = 0; dt < NT; ++dt) {
@@ -964,7 +971,7 @@ __global__ __launch_bounds__(64 * BLK_WAVES * GROUPS, GROUPS == 1 ? BLK_PER_CU :
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
     const int* __restrict__ bt, int table_width, const int* __restrict__ cu_q, const int* __restrict__ ctx_len,
     const int* __restrict__ blk_req, const int* __restrict__ blk_cb, int num_blocks, bf16_t* __restrict__ out, int nq,
-    int nkv, int ps, int window, float scale, int* __restrict__ queue, const float* __restrict__ sinks) {
+    int nkv, int ps, int window, float scale, int* __restrict__ queue, HeadEnd end) {
   __shared__ BlockShared<GROUPS> sh;
   const bool per_head = 8 % nkv == 0;
   const int queues = per_head ? nkv : 1;
@@ -978,7 +985,7 @@ __global__ __launch_bounds__(64 * BLK_WAVES * GROUPS, GROUPS == 1 ? BLK_PER_CU :
       const int work = __builtin_amdgcn_readfirstlane(sh.work);   // the same for all: keep it scalar
       if (work >= per_queue) break;  // uniform over the block; every workgroup gets here for every queue
       attend_block(sh, per_head ? work : work / nkv, per_head ? qi : work % nkv, q, kc, vc, bt, table_width, cu_q,
-                   ctx_len, blk_req, blk_cb, out, nq, nkv, ps, window, scale, sinks);
+                   ctx_len, blk_req, blk_cb, out, nq, nkv, ps, window, scale, end);
       __syncthreads();               // everybody has read sh.work and is done with the stages
     }
     __syncthreads();
@@ -1025,7 +1032,7 @@ __device__ __forceinline__ float load_device_scope(const float* p) {
 template <bool ACROSS>
 __device__ __forceinline__ void merge_splits(const float* __restrict__ base, int nsplit, int r, int ct, int kvh, int g,
                                              const int* __restrict__ cu_q, bf16_t* __restrict__ out, int nq,
-                                             const float* __restrict__ sinks) {
+                                             const HeadEnd& end) {
   const Run run = run_of(cu_q, r);
   const int q0 = run.q0, qlen = run.qlen;
   for (int idx = threadIdx.x; idx < 16 * (HD / 4); idx += blockDim.x) {
@@ -1065,7 +1072,7 @@ __device__ __forceinline__ void merge_splits(const float* __restrict__ base, int
         den += wgt * pl[j];
       }
     }
-    const float inv = 1.0f / (den + sink_term(sinks, kvh * g + gh, m));
+    const float inv = head_end(end, q0 + i, kvh * g + gh, den, m);
     uint2 wv;
     wv.x = pack2(num.x * inv, num.y * inv);
     wv.y = pack2(num.z * inv, num.w * inv);
@@ -1078,7 +1085,7 @@ __global__ __launch_bounds__(64 * COOP_WAVES) void attn_mfma_coop_kernel(
     const int* __restrict__ bt, int table_width, const int* __restrict__ cu_q, const int* __restrict__ ctx_len,
     const int* __restrict__ tile_req, const int* __restrict__ tile_ct, bf16_t* __restrict__ out,
     float* __restrict__ scratch, int* __restrict__ counters, int nq, int nkv, int ps, int window, float scale,
-    int nsplit, int keys_per_split, const float* __restrict__ sinks) {
+    int nsplit, int keys_per_split, HeadEnd end) {
   __shared__ __attribute__((aligned(16))) float sm[COOP_WAVES][PART_STRIDE];
   __shared__ __attribute__((aligned(16))) char second_place[K_VIA_LDS ? COOP_WAVES : 1][K_VIA_LDS ? 32 * HD * 2 : 16];   // of staged keys
   __shared__ int is_last;
@@ -1159,7 +1166,7 @@ __global__ __launch_bounds__(64 * COOP_WAVES) void attn_mfma_coop_kernel(
         }
       }
     } else if (i < qlen) {
-      const float inv = 1.0f / (den + sink_term(sinks, kvh * g + gh, m));
+      const float inv = head_end(end, q0 + i, kvh * g + gh, den, m);
       uint2 wv;
       wv.x = pack2(num.x * inv, num.y * inv);
       wv.y = pack2(num.z * inv, num.w * inv);
@@ -1178,18 +1185,18 @@ __global__ __launch_bounds__(64 * COOP_WAVES) void attn_mfma_coop_kernel(
     }
     __syncthreads();
     if (is_last)
-      merge_splits<true>(scratch + ((size_t)tile * nkv + kvh) * nsplit * PART_STRIDE, nsplit, r, ct, kvh, g, cu_q, out, nq, sinks);
+      merge_splits<true>(scratch + ((size_t)tile * nkv + kvh) * nsplit * PART_STRIDE, nsplit, r, ct, kvh, g, cu_q, out, nq, end);
   }
 }
 
 __global__ void attn_mfma_merge_kernel(const float* __restrict__ scratch, const int* __restrict__ cu_q,
                                        const int* __restrict__ tile_req, const int* __restrict__ tile_ct,
                                        bf16_t* __restrict__ out, int nq, int nkv, int nsplit,
-                                       const float* __restrict__ sinks) {
+                                       HeadEnd end) {
   // one block per (tile, kv head)
   const int tile = blockIdx.x, kvh = blockIdx.y;
   merge_splits<false>(scratch + ((size_t)tile * nkv + kvh) * nsplit * PART_STRIDE, nsplit, tile_req ? tile_req[tile] : tile,
-                      tile_req ? tile_ct[tile] : 0, kvh, nq / nkv, cu_q, out, nq, sinks);
+                      tile_req ? tile_ct[tile] : 0, kvh, nq / nkv, cu_q, out, nq, end);
 }
 
 static int check_common(int num_tiles, int nq, int nkv, int ps, int table_width) {
@@ -1208,9 +1215,10 @@ extern "C" int qvl_attn_mfma_queue_ints() { return QUEUE_INTS; }
 
 extern "C" int qvl_attn_mfma_block(const void* q, const void* kc, const void* vc, const void* bt, int table_width,
                                    const void* cu_q, const void* ctx_len, const void* blk_req, const void* blk_cb,
-                                   int num_blocks, void* out, const void* sinks, int nq, int nkv, int ps, int window,
-                                   float scale, void* queue, int max_workgroups, int groups, hipStream_t stream) {
+                                   int num_blocks, void* out, const void* sinks, const void* gates,
+                                   long long gate_stride, int nq, int nkv, int ps, int window, float scale, void* queue, int max_workgroups, int groups, hipStream_t stream) {
   // sinks: float32 [nq] or null: one more term exp(sink) in each query head's softmax denominator.
+  // gates: float32, a row of gate_stride values per token, or null: head h's output times sigmoid(row[h]).
   // queue: qvl_attn_mfma_queue_ints() ints, zero before the first launch that uses them.
   // groups: wave groups per workgroup, 1 .. qvl_attn_mfma_block_max_groups(); max_workgroups should
   // be what the device holds at a time (qvl_attn_mfma_block_per_cu() per compute unit with one group, one with two).
@@ -1221,11 +1229,12 @@ extern "C" int qvl_attn_mfma_block(const void* q, const void* kc, const void* vc
   const long long total = (long long)num_blocks * nkv;
   if (total > 0x7fffffffLL) return QVL_ERR_LIMIT;
   const unsigned grid = (unsigned)(total < max_workgroups ? total : max_workgroups);
+  const HeadEnd end{(const float*)sinks, (const float*)gates, gate_stride};
 #define QVL_BLOCK_LAUNCH(G)                                                                                          \
   hipLaunchKernelGGL(attn_mfma_block_kernel<G>, dim3(grid), dim3(64 * BLK_WAVES * G), 0, stream, (const bf16_t*)q,    \
                      (const bf16_t*)kc, (const bf16_t*)vc, (const int*)bt, table_width, (const int*)cu_q,              \
                      (const int*)ctx_len, (const int*)blk_req, (const int*)blk_cb, num_blocks, (bf16_t*)out, nq, nkv, \
-                     ps, window, scale, (int*)queue, (const float*)sinks)
+                     ps, window, scale, (int*)queue, end)
   if (groups == 1) QVL_BLOCK_LAUNCH(1);
 #if BLK_MAX_GROUPS > 1
   else QVL_BLOCK_LAUNCH(2);
@@ -1241,7 +1250,7 @@ extern "C" long long qvl_attn_mfma_scratch_floats(int num_tiles, int nkv, int ns
 
 static int launch_coop(const void* q, const void* kc, const void* vc, const void* bt, int table_width,
                        const void* cu_q, const void* ctx_len, const void* tile_req, const void* tile_ct,
-                       int num_tiles, void* out, void* scratch, void* counters, const void* sinks, int nq, int nkv,
+                       int num_tiles, void* out, void* scratch, void* counters, const HeadEnd& end, int nq, int nkv,
                        int ps, int window, float scale, int nsplit, int keys_per_split, hipStream_t stream) {
   const int c = check_common(num_tiles, nq, nkv, ps, table_width);
   if (c >= 0) return c;
@@ -1252,12 +1261,11 @@ static int launch_coop(const void* q, const void* kc, const void* vc, const void
                      (const bf16_t*)q, (const bf16_t*)kc, (const bf16_t*)vc, (const int*)bt, table_width,
                      (const int*)cu_q, (const int*)ctx_len, (const int*)tile_req, (const int*)tile_ct, (bf16_t*)out,
                      (float*)scratch, nsplit > 1 ? (int*)counters : nullptr, nq, nkv, ps, window, scale, nsplit,
-                     keys_per_split, (const float*)sinks);
+                     keys_per_split, end);
   if (hipGetLastError() != hipSuccess) return QVL_ERR_LAUNCH;
   if (nsplit > 1 && !counters)
     hipLaunchKernelGGL(attn_mfma_merge_kernel, dim3(num_tiles, nkv), dim3(256), 0, stream, (const float*)scratch,
-                       (const int*)cu_q, (const int*)tile_req, (const int*)tile_ct, (bf16_t*)out, nq, nkv, nsplit,
-                       (const float*)sinks);
+                       (const int*)cu_q, (const int*)tile_req, (const int*)tile_ct, (bf16_t*)out, nq, nkv, nsplit, end);
   return qvl_launch_status();
 }
 
@@ -1265,20 +1273,21 @@ extern "C" int qvl_attn_mfma_coop(const void* q, const void* kc, const void* vc,
                                   const void* cu_q, const void* ctx_len, const void* tile_req, const void* tile_ct,
                                   int num_tiles, void* out, void* scratch, int nq, int nkv, int ps, int window,
                                   float scale, int nsplit, int keys_per_split, hipStream_t stream) {
-  return launch_coop(q, kc, vc, bt, table_width, cu_q, ctx_len, tile_req, tile_ct, num_tiles, out, scratch, nullptr, nullptr, nq,
+  return launch_coop(q, kc, vc, bt, table_width, cu_q, ctx_len, tile_req, tile_ct, num_tiles, out, scratch, nullptr, HeadEnd{nullptr, nullptr, 0}, nq,
                      nkv, ps, window, scale, nsplit, keys_per_split, stream);
 }
 
 // The same with the splits merged inside the one kernel, by the block of each (tile, kv head) that
 // finishes last.  counters: num_tiles * nkv ints, zero before the launch; the launch leaves them at
-// zero (null: a second launch merges).  sinks: float32 [nq] or null, as above.  Launches that share counters or scratch must not overlap.
+// zero (null: a second launch merges).  sinks and gates as above.  Launches that share counters or scratch must not overlap.
 extern "C" int qvl_attn_mfma_coop_merged(const void* q, const void* kc, const void* vc, const void* bt, int table_width,
                                          const void* cu_q, const void* ctx_len, const void* tile_req,
                                          const void* tile_ct, int num_tiles, void* out, void* scratch, void* counters,
-                                         const void* sinks, int nq, int nkv, int ps, int window, float scale, int nsplit,
+                                         const void* sinks, const void* gates, long long gate_stride, int nq, int nkv,
+                                         int ps, int window, float scale, int nsplit,
                                          int keys_per_split, hipStream_t stream) {
   return launch_coop(q, kc, vc, bt, table_width, cu_q, ctx_len, tile_req, tile_ct, num_tiles, out, scratch, counters,
-                     sinks, nq, nkv, ps, window, scale, nsplit, keys_per_split, stream);
+                     HeadEnd{(const float*)sinks, (const float*)gates, gate_stride}, nq, nkv, ps, window, scale, nsplit, keys_per_split, stream);
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -1335,6 +1344,6 @@ extern "C" int qvl_attn_mfma_coop_static(const void* q, const void* kc, const vo
   if (!ptr) return err;
   // Every (tile, head, split) block writes all of its part before the merge kernel reads it, so
   // nothing of the array has to start at zero, whatever the call before left there.
-  return launch_coop(q, kc, vc, bt, table_width, cu_q, ctx_len, tile_req, tile_ct, num_tiles, out, ptr, nullptr, nullptr, nq, nkv,
+  return launch_coop(q, kc, vc, bt, table_width, cu_q, ctx_len, tile_req, tile_ct, num_tiles, out, ptr, nullptr, HeadEnd{nullptr, nullptr, 0}, nq, nkv,
                      ps, window, scale, nsplit, keys_per_split, stream);
 }

@@ -387,7 +387,8 @@ extern "C" int qvl_head_gate(void* o, const void* gate, long long gate_stride, i
 //   cosines and sines are cs[n, f]: pair (2f, 2f+1) if `interleaved`, else (f, f + rot_half).
 //   norm_mode 0: no norm; 1: the norm comes before the rotation; 2: after it; 3: before it and over all
 //   query heads of a token together (and all its key heads together): the two inverse root mean squares
-//   come in `row_rs` [N, 2] (row_inv_rms below forms them) and the weights span all heads' columns.
+//   come in `row_rs` [N, 2] (row_inv_rms below forms them), or every wave forms its own from the whole row (row_rs null:
+//   for few rows), and the weights span all heads' columns.
 //   Queries go to q_out [N, nq hd]; keys into k_cache [pages, nkv, ps, hd] at slots[n]; values
 //   (the key head before norm and rotation, or the value head) into v_cache [pages, nkv, vd, ps].
 //   `vcs` [N, vd/2, 2] (or null): value heads are turned by these angles over all their channels, channel c with
@@ -452,7 +453,21 @@ __global__ __launch_bounds__(256) void qk_norm_rope_write_kernel(
     const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)hd + eps);
     for (int c = lane; c < hd; c += 64) mine[c] = nw ? (mine[c] * rs) * nw[c] : mine[c] * rs;
   } else if (norm_mode == 3) {
-    const float rs = row_rs[2 * (size_t)n + kind];
+    float rs;
+    if (row_rs) {
+      rs = row_rs[2 * (size_t)n + kind];
+    } else {
+      const int width = (kind == 0 ? nq : nkv) * hd;
+      const float* all = x + (size_t)n * x_stride + (kind == 0 ? 0 : (size_t)nq * hd);
+      const float* ball = bias ? bias + (kind == 0 ? 0 : (size_t)nq * hd) : nullptr;
+      float sum = 0.f;
+#pragma unroll 8
+      for (int c = lane; c < width; c += 64) {
+        const float v = all[c] + (ball ? ball[c] : 0.f);
+        sum += v * v;
+      }
+      rs = 1.0f / sqrtf(wave_sum(sum) / (float)width + eps);
+    }
     const float* nwh = nw ? nw + (size_t)(kind == 0 ? head : head - nq) * hd : nullptr;
     for (int c = lane; c < hd; c += 64) mine[c] = nwh ? (mine[c] * rs) * nwh[c] : mine[c] * rs;
   }
@@ -501,7 +516,7 @@ extern "C" int qvl_qk_norm_rope_write(const void* x, long long x_stride, const v
   if (N <= 0) return QVL_OK;
   if (nq <= 0 || nkv < 0 || hd <= 0 || vd <= 0 || rot_half < 0 || 2 * rot_half > hd || ps <= 0) return QVL_ERR_SHAPE;
   if (write_kv && (!slots || !k_cache || !v_cache || nkv <= 0)) return QVL_ERR_SHAPE;
-  if (norm_mode < 0 || norm_mode > 3 || (norm_mode == 3 && !row_rs) || (v_from_k && vd != hd)) return QVL_ERR_SHAPE;
+  if (norm_mode < 0 || norm_mode > 3 || (v_from_k && vd != hd)) return QVL_ERR_SHAPE;
   if (vcs && (v_from_k || vd % 2)) return QVL_ERR_SHAPE;
   if (hd > QKN_MAX_HD || vd > QKN_MAX_HD) return QVL_ERR_LIMIT;
   const int heads = nq + (write_kv ? (v_from_k ? nkv : 2 * nkv) : 0);

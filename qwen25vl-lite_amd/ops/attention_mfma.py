@@ -18,7 +18,7 @@ from .kernels import _check, _fn, _need, _ptr, _stream
 
 __all__ = ["try_attention", "supports", "tiles_for", "plan_splits"]
 
-_c_int, _c_float, _c_ptr = ctypes.c_int, ctypes.c_float, ctypes.c_void_p
+_c_int, _c_float, _c_ptr, _c_ll = ctypes.c_int, ctypes.c_float, ctypes.c_void_p, ctypes.c_longlong
 _MAX_HD = 256
 # Thresholds that follow the device: counts per compute unit (measured on 256 of them); the names below
 # them hold a number instead of None where a caller (a test) fixes the count itself.
@@ -188,9 +188,11 @@ def block_groups(walks: int, places: int, head_dim: int) -> int:
 
 def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, window: Optional[int],
                   scale: float, force_groups: Optional[int] = None, force_wide: Optional[bool] = None,
-                  sinks: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+                  sinks: Optional[torch.Tensor] = None,
+                  gate: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """The attention through the matrix-core kernel, or None if it does not take this shape.  ``sinks`` (float32
-    ``[heads]``): one more term ``exp(sink)`` in each query head's softmax denominator.
+    ``[heads]``): one more term ``exp(sink)`` in each query head's softmax denominator.  ``gate`` (float32 ``[N, heads]``,
+    rows any distance apart): each head's output times the sigmoid of its number.
     Calls on one device must not overlap (one stream): the kernel for prompt portions keeps its
     work-queue counters in memory that all calls on the device share.
     ``force_groups``, ``force_wide`` (tests): the workgroup kind of the kernel for prompt portions and
@@ -207,6 +209,9 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
     _need(nq % nkv == 0, "query heads must be a multiple of key/value heads")
     _need(sinks is None or (sinks.is_cuda and sinks.dtype == torch.float32 and sinks.shape == (nq,)
                             and sinks.is_contiguous()), "sinks must be float32 [nq] on the GPU")
+    _need(gate is None or (gate.is_cuda and gate.dtype == torch.float32 and gate.shape == (n, nq) and gate.stride(1) == 1),
+          "gate must be float32 [N, nq] on the GPU with contiguous rows")
+    gate_args = (_ptr(gate), 0 if gate is None else gate.stride(0))
     tile_req, tile_ct, num_tiles = _step_tiles(step, nq // nkv, 1, q.device)
     out = torch.empty_like(q)
     defines = {"HD": hd}
@@ -223,7 +228,7 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
         if wide:
             tile_req, tile_ct, num_tiles = _step_tiles(step, nq // nkv, block_tiles(hd, True), q.device, by_length=True, only=only)
         fn = _fn("attention_mfma", "qvl_attn_mfma_block",
-                 [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr] + [_c_int] * 4
+                 [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr, _c_ptr, _c_ll] + [_c_int] * 4
                  + [_c_float, _c_ptr, _c_int, _c_int, _c_ptr], defines)
         queue, cus = _work_queue(q.device)
         per_cu = int(_fn("attention_mfma", "qvl_attn_mfma_block_per_cu", [], defines)())
@@ -231,7 +236,7 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
         groups = block_groups(num_tiles * nkv, cus * per_cu, hd) if force_groups is None else force_groups
         groups = min(groups, most) if force_groups is None else groups
         code = fn(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(step.cu_q),
-                  _ptr(step.ctx_len), _ptr(tile_req), _ptr(tile_ct), num_tiles, _ptr(out), _ptr(sinks), nq, nkv, ps, int(window or 0),
+                  _ptr(step.ctx_len), _ptr(tile_req), _ptr(tile_ct), num_tiles, _ptr(out), _ptr(sinks), *gate_args, nq, nkv, ps, int(window or 0),
                   float(scale), _ptr(queue), cus * (per_cu if groups == 1 else 1), groups, _stream())
         if code:
             # whatever a launch that went wrong did to the counters, the next one starts from zero
@@ -252,15 +257,15 @@ def try_attention(q, k_cache, v_cache, block_table, step, num_q_heads: int, wind
             floats.restype = ctypes.c_longlong
             scratch = torch.empty(int(floats(num_tiles, nkv, nsplit)), dtype=torch.float32, device=q.device)
         merged = nsplit > 1 and num_tiles * nkv <= MERGE_COUNTERS
-        if merged or sinks is not None:
+        if merged or sinks is not None or gate is not None:
             # the block of each (tile, head) that finishes last merges the splits: one launch
             counters = _counters(q.device) if merged else None
             fn = _fn("attention_mfma", "qvl_attn_mfma_coop_merged",
-                     [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr] + [_c_int] * 4
+                     [_c_ptr] * 4 + [_c_int] + [_c_ptr] * 4 + [_c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll] + [_c_int] * 4
                      + [_c_float, _c_int, _c_int, _c_ptr], defines)
             code = fn(_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1], _ptr(cu_q),
                       _ptr(step.ctx_len), _ptr(tile_req), _ptr(tile_ct), num_tiles, _ptr(out), _ptr(scratch),
-                      _ptr(counters), _ptr(sinks), nq, nkv, ps, int(window or 0), float(scale), nsplit, per, _stream())
+                      _ptr(counters), _ptr(sinks), *gate_args, nq, nkv, ps, int(window or 0), float(scale), nsplit, per, _stream())
             if code and merged:
                 counters.zero_()
             _check(code, "paged_attention (matrix cores, shared tiles, merged)")

@@ -17,6 +17,7 @@ __all__ = ["residual_add", "gated_act", "softcap_", "group_norm_gate", "head_gat
            "row_inv_rms", "tanh_to"]
 
 _c_int, _c_float, _c_ptr, _c_ll = ctypes.c_int, ctypes.c_float, ctypes.c_void_p, ctypes.c_longlong
+WHOLE_NORM_ROWS = 16      # up to here the kernel that rotates forms a whole projection's root mean square by itself
 GATE_ACTS = {None: 0, "sigmoid": 1, "silu": 2}
 
 
@@ -162,7 +163,7 @@ def qk_norm_rope_write(x: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: 
                             and w.is_contiguous()),
               "a head norm's weight must be float32 [head_dim], a whole projection's [heads head_dim]")
     row_rs = None
-    if norm == "whole":
+    if norm == "whole" and n > WHOLE_NORM_ROWS:
         row_rs = row_inv_rms(x, nq * hd, nkv * hd if write else 0, eps, bias)
     _need(bias is None or (bias.dtype == torch.float32 and bias.dim() == 1 and bias.shape[0] >= cols
                            and bias.is_contiguous()), "the bias must be float32 over the heads' columns")

@@ -295,13 +295,12 @@ class PagedAttention(Mixer):
             self.nq, self.nkv, self.hd, group.page_size, self.dtype, interleaved=self.interleaved,
             values_are_keys=self.values_are_keys, norm=norm, bias=self.b_in, value_dim=self.vd,
             value_cs=value_cs)
+        gate = proj[:, self.w_in.shape[0] - self.gate_rows:] if self.gate_rows else None
         o = paged_attention(q, slot.k_cache, slot.v_cache, group.block_table, step, self.nq, self.window, self.scale,
                             keep_first=self.keep_first, sinks=self.sink, chunk=self.chunk, turn=value_cs,
-                            turn_pairs=self.interleaved)
-        if self.gate_rows:
-            # one gate per head, or one per element (a "head" of one channel)
-            at = self.w_in.shape[0] - self.gate_rows
-            gated.head_gate_(o, proj[:, at:at + self.gate_rows], self.gate_rows)
+                            turn_pairs=self.interleaved, gate=gate if self.head_gate else None)
+        if self.element_gate:
+            gated.head_gate_(o, gate, self.gate_rows)      # one gate per element (a "head" of one channel)
         return self._output(o, step)
 
     def _project(self, x, step, group, slot, write, inv_freq, freq_row) -> torch.Tensor:

@@ -249,7 +249,7 @@ def test_a_gate_per_head(nh, hd, dtype):
 
 @pytest.mark.parametrize("window", [None, 37, 90])
 @pytest.mark.parametrize("nq, nkv, hd", [(4, 2, 128), (6, 2, 48), (3, 3, 64), (5, 1, 16)])
-def test_sinks_in_every_kind_of_matrix_core_attention(nq, nkv, hd, window, monkeypatch):
+def test_sinks_and_gates_in_every_kind_of_matrix_core_attention(nq, nkv, hd, window, monkeypatch):
     """Prompt portions with one and two groups of waves and with three column tiles a wave; decoded tokens with the keys
     whole, split among blocks and merged in the launch, and merged by a second one.  Two sinks stand out: one that takes
     most of the weight and one that takes none."""
@@ -261,6 +261,7 @@ def test_sinks_in_every_kind_of_matrix_core_attention(nq, nkv, hd, window, monke
     k[11] *= 4.0                                  # a far key that some queries pick
     sinks = torch.randn(nq)
     sinks[0], sinks[-1] = 6.0, -30.0
+    gate = 2 * torch.randn(n, nq + 3)             # a gate per head, columns of a wider tensor
     q, k, v = (t.to(torch.bfloat16) for t in (q, k, v))
     want = plain.attend(q.double(), k.double(), v.double(), scale, window, sinks.double())
     none = plain.attend(q.double(), k.double(), v.double(), scale, window, None)
@@ -276,9 +277,12 @@ def test_sinks_in_every_kind_of_matrix_core_attention(nq, nkv, hd, window, monke
         monkeypatch.setattr(attention_mfma, "plan_splits", lambda *a: plan)
         step = SimpleNamespace(num_reqs=1, cu_q=_i32([0, m]), cu_q_host=[0, m], ctx_len=_i32([n]), ctx_len_host=[n], max_q_len=m,
                                max_ctx_len=n, derived={})
-        got = attention_mfma.try_attention(q[first:].reshape(m, -1).contiguous().cuda(), kc, vc, table, step, nq, window, scale,
-                                           sinks=sinks.cuda(), **kw)
-        assert torch.allclose(got.double().cpu().view(m, nq, hd), want[first:], atol=2e-2, rtol=2e-2), (first, plan, kw)
+        args = (q[first:].reshape(m, -1).contiguous().cuda(), kc, vc, table, step, nq, window, scale)
+        for s, g in ((sinks.cuda(), None), (sinks.cuda(), gate[first:, 1:1 + nq].cuda()), (None, gate[first:, 1:1 + nq].cuda())):
+            w = want if s is not None else none
+            w = w if g is None else w * torch.sigmoid(gate[:, 1:1 + nq].double())[:, :, None]
+            got = attention_mfma.try_attention(*args, sinks=s, gate=g, **kw)
+            assert torch.allclose(got.double().cpu().view(m, nq, hd), w[first:], atol=2e-2, rtol=2e-2), (first, plan, kw)
 
     for first in (0, 130):
         for kw in (dict(force_groups=1, force_wide=False), dict(force_groups=2, force_wide=False), dict(force_groups=1, force_wide=True)):
