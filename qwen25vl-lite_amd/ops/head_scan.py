@@ -17,7 +17,8 @@ _c_int, _c_float, _c_ptr, _c_ll = ctypes.c_int, ctypes.c_float, ctypes.c_void_p,
 MAX_KEY_SIZE = 512
 MAX_CHUNKED_KEY_SIZE = 256
 CHUNK = 64
-CHUNKED_FROM = 24     # a step whose longest run has this many tokens or more is scanned in chunks side by side
+CHUNKED_FROM = 40     # a step whose longest run has this many tokens or more is scanned in chunks side by side (one run of
+                      # 7B-sized heads: 39 us token after token at 32 tokens, 41 in chunks up to 64; eight runs: 42 and 70)
 
 
 def takes_chunks(dim: int, max_run: int) -> bool:
