@@ -528,9 +528,11 @@ def main(argv=None) -> int:
                 model = build_model(load_config(design_config(name)), dtype, "cuda:0")
                 fill_random(model, seed=0)
                 torch.cuda.synchronize()
+            print(f"[bench] {name}: prefill", file=sys.stderr, flush=True)
             sec = prefill_rate(2048)
             out[name] = {"prefill_tok_s": round(2048 / sec, 1), "prefill_ms": round(sec * 1e3, 3)}
             if not args.prefill_only:
+                print(f"[bench] {name}: decode", file=sys.stderr, flush=True)
                 rate, ms, _ = decode_rate(args.batch, steps, warmup)
                 out[name].update({"decode_tok_s": round(rate, 1), "decode_ms_per_step": round(ms, 4)})
         print(json.dumps(out))

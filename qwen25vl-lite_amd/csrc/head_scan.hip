@@ -454,65 +454,54 @@ __global__ __launch_bounds__(256) void hs_solve_kernel(HeadScan a) {
 // ---------------------------------------------------------------------------------------
 // The states from chunk to chunk: a block per (16 value channels, head, request)
 // ---------------------------------------------------------------------------------------
-#ifndef HS_WIDE_CARRY
-#define HS_WIDE_CARRY 0                         // plain rule: 1 stages a chunk's keys once for two tiles of value channels
-#endif
 #define HS_MT ((HS_KB + 3) / 4)                 // row blocks of S a wave keeps: wave w has blocks w, w + 4, ...
 
 // What a block reads of a chunk, asked for two chunks ahead: nothing here is waited for before it is used.
-template <typename TX, bool DELTA, int NV> struct CarryLoads {
+template <typename TX, bool DELTA> struct CarryLoads {
   Four<TX, true> k[HS_MT][4];
   f32x4 wk[DELTA ? HS_KB : 1];
-  f32x4 u[DELTA ? NV : 1];
-  TX v[DELTA ? 1 : NV][4];
+  f32x4 u;
+  TX v[4];
   f32x4 gate, tail, unit;
   float end;
   int n;
 };
 
-// NV neighbouring tiles of 16 value channels a block
-template <typename TX, bool DELTA, int NV>
+template <typename TX, bool DELTA>
 __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
-  __shared__ f32x4 us_place[2][NV][4 * 64];     // U, weighted by what is left of it at the chunk's end; two places, taken in turn
-  __shared__ f32x4 s[NV][HS_KB * 64];           // S as right operand
+  __shared__ f32x4 us_place[2][4 * 64];         // U, weighted by what is left of it at the chunk's end; two places, taken in turn
+  __shared__ f32x4 s[DELTA ? HS_KB * 64 : 1];   // S as right operand
   __shared__ float left[2];                     // what a chunk leaves of the state before it
   // Workgroups go to the 8 XCDs in turn: numbered so that an XCD gets neighbouring tiles and heads, whose blocks read the
-  // same keys and Wk, so that these come into its L2 once.
-  const int vtiles = (a.vdim + 15) / 16, across = (vtiles + NV - 1) / NV;
+  // same keys and Wk.
+  const int vtiles = (a.vdim + 15) / 16;
   const int item = (blockIdx.x & 7) * (gridDim.x >> 3) + (blockIdx.x >> 3);
-  if (item >= across * a.H) return;
-  const int head = item / across, vt0 = item % across * NV, req = blockIdx.y, grp = head / (a.H / a.G);
+  if (item >= vtiles * a.H) return;
+  const int head = item / vtiles, vtile = item % vtiles, req = blockIdx.y, grp = head / (a.H / a.G);
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, lg = lane >> 4;
   const int first = __builtin_amdgcn_readfirstlane(a.req_first[req]), last = __builtin_amdgcn_readfirstlane(a.req_first[req + 1]);
   if (first >= last) return;
   // a run's chunks follow one another and all but the last are full
   const int run_begin = __builtin_amdgcn_readfirstlane(a.bounds[first]), run_end = __builtin_amdgcn_readfirstlane(a.bounds[last]);
-  static_assert(HS_CHUNK == 64, "four blocks of 16 tokens");
-  float* slot = a.state + ((size_t)a.row_of[req] * a.H + head) * HS_DIM * a.vdim;
-  f32x4 S[NV][HS_MT];
+  const int vcol = vtile * 16 + col;
+  const bool in = vcol < a.vdim;
+  float* slot = a.state + ((size_t)a.row_of[req] * a.H + head) * HS_DIM * a.vdim + (in ? vcol : 0);
+  f32x4 S[HS_MT];
 #pragma unroll
-  for (int v = 0; v < NV; ++v) {
-    const int vcol = (vt0 + v) * 16 + col;
+  for (int m = 0; m < HS_MT; ++m) {
 #pragma unroll
-    for (int m = 0; m < HS_MT; ++m) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = (wave + 4 * m) * 16 + 4 * lg + r;
-        S[v][m][r] = vcol < a.vdim && d < HS_DIM ? slot[(size_t)d * a.vdim + vcol] : 0.f;
-      }
+    for (int r = 0; r < 4; ++r) {
+      const int d = (wave + 4 * m) * 16 + 4 * lg + r;
+      S[m][r] = in && d < HS_DIM ? slot[(size_t)d * a.vdim] : 0.f;
     }
   }
   const TX* x = reinterpret_cast<const TX*>(a.x);
   const int t_own = wave * 16 + 4 * lg;         // the first of this lane's four rows of U
-  typedef CarryLoads<TX, DELTA, NV> Loads;
+  typedef CarryLoads<TX, DELTA> Loads;
   // places of values within a chunk, in bytes from its first token's: the same for every chunk
-  unsigned v_at[NV][4];
+  unsigned v_at[4];
 #pragma unroll
-  for (int v = 0; v < NV; ++v) {
-    const int vcol = (vt0 + v) * 16 + col;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) v_at[v][r] = (unsigned)(((t_own + r) * (int)a.x_stride + (vcol < a.vdim ? vcol : 0)) * (int)sizeof(TX));
-  }
+  for (int r = 0; r < 4; ++r) v_at[r] = (unsigned)(((t_own + r) * (int)a.x_stride + (in ? vcol : 0)) * (int)sizeof(TX));
   auto ask_keys = [&](Loads& l, int c) {
     const TX* kt = reinterpret_cast<const TX*>(a.kt) + (((size_t)c * a.G + grp) * HS_KB * 4 * 64 + lane) * 4;
 #pragma unroll
@@ -531,75 +520,54 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
       const float* wk = a.wk + (ch * HS_CHUNK + wave * 16 + col) * HS_DIMP + 4 * lg;
 #pragma unroll
       for (int b = 0; b < HS_KB; ++b) l.wk[DELTA ? b : 0] = *reinterpret_cast<const f32x4*>(wk + b * 16);
-#pragma unroll
-      for (int v = 0; v < NV; ++v)
-        if (NV == 1 || vt0 + v < vtiles) l.u[DELTA ? v : 0] = *reinterpret_cast<const f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4);
+      l.u = *reinterpret_cast<const f32x4*>(a.u + ((ch * vtiles + vtile) * 4 + wave) * 256 + lane * 4);
     } else {
       l.gate = *reinterpret_cast<const f32x4*>(a.gate + ch * HS_CHUNK + t_own);
-      const int begin = run_begin + (c - first) * HS_CHUNK, n = run_end - begin < HS_CHUNK ? run_end - begin : HS_CHUNK;
-      l.n = n;
+      const int begin = run_begin + (c - first) * HS_CHUNK;
+      l.n = run_end - begin < HS_CHUNK ? run_end - begin : HS_CHUNK;
       const char* base = reinterpret_cast<const char*>(x + (size_t)begin * a.x_stride + a.v_off + (size_t)head * a.vdim);
 #pragma unroll
-      for (int v = 0; v < NV; ++v)
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          l.v[DELTA ? 0 : v][r] = *reinterpret_cast<const TX*>(base + (t_own + r < n ? v_at[v][r] : 0u));
+      for (int r = 0; r < 4; ++r) l.v[r] = *reinterpret_cast<const TX*>(base + (t_own + r < l.n ? v_at[r] : 0u));
     }
   };
   // The order of a step's memory operations is that in which they are waited for: what the next step needs first is asked
-  // for first, and the stores, which nobody waits for, come last.
+  // for first, and the stores, which nobody waits for, come behind what the next but one waits for.
   auto step = [&](Loads& l, int c) {
     const size_t ch = (size_t)c * a.H + head;
-    const int n = DELTA ? 0 : l.n, next = c + 2 < last ? c + 2 : last - 1;      // the last two ask for the last chunk again
-    f32x4 (*us)[4 * 64] = us_place[c & 1];
+    const int next = c + 2 < last ? c + 2 : last - 1;      // the last two ask for the last chunk again
+    f32x4* us = us_place[c & 1];
+    f32x4 u;
     if (DELTA) {
 #pragma unroll
-      for (int v = 0; v < NV; ++v)
-#pragma unroll
-        for (int m = 0; m < HS_MT; ++m)
-          if (HS_KB % 4 == 0 || wave + 4 * m < HS_KB) s[v][(wave + 4 * m) * 64 + lane] = S[v][m];
+      for (int m = 0; m < HS_MT; ++m)
+        if (HS_KB % 4 == 0 || wave + 4 * m < HS_KB) s[DELTA ? (wave + 4 * m) * 64 + lane : 0] = S[m];
       __syncthreads();
-    }
-    f32x4 u[NV];
+      f32x4 p0 = {0.f, 0.f, 0.f, 0.f}, p1 = p0;
 #pragma unroll
-    for (int v = 0; v < NV; ++v) {
-      if (DELTA) {
-        f32x4 p0 = {0.f, 0.f, 0.f, 0.f}, p1 = p0;
-#pragma unroll
-        for (int b = 0; b < HS_KB; b += 2) {
-          p0 = mma16(l.wk[DELTA ? b : 0], s[v][b * 64 + lane], p0);
-          if (b + 1 < HS_KB) p1 = mma16(l.wk[DELTA ? b + 1 : 0], s[v][(b + 1) * 64 + lane], p1);
-        }
-        u[v] = l.u[DELTA ? v : 0] - (p0 + p1);
-      } else {
-        const bool in = (vt0 + v) * 16 + col < a.vdim;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) u[v][r] = in && t_own + r < n ? l.gate[r] * ldf<TX>(&l.v[DELTA ? 0 : v][r]) : 0.f;
+      for (int b = 0; b < HS_KB; b += 2) {
+        p0 = mma16(l.wk[DELTA ? b : 0], s[DELTA ? b * 64 + lane : 0], p0);
+        if (b + 1 < HS_KB) p1 = mma16(l.wk[DELTA ? b + 1 : 0], s[DELTA ? (b + 1) * 64 + lane : 0], p1);
       }
-      us[v][wave * 64 + lane] = u[v] * l.tail * l.unit;
+      u = l.u - (p0 + p1);
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) u[r] = in && t_own + r < l.n ? l.gate[r] * ldf<TX>(l.v + r) : 0.f;
     }
+    us[wave * 64 + lane] = u * l.tail * l.unit;
     if (tid == 0) left[c & 1] = l.end;
     ask_rest(l, next);
-#pragma unroll
-    for (int v = 0; v < NV; ++v) {
-      if (NV > 1 && vt0 + v >= vtiles) continue;
-      float* s0 = a.s0 + ((ch * vtiles + vt0 + v) * HS_KB * 64 + lane) * 4;
-#pragma unroll
-      for (int m = 0; m < HS_MT; ++m)
-        if (HS_KB % 4 == 0 || wave + 4 * m < HS_KB) *reinterpret_cast<f32x4*>(s0 + (size_t)(wave + 4 * m) * 256) = S[v][m];
-      if (DELTA) *reinterpret_cast<f32x4*>(a.u + ((ch * vtiles + vt0 + v) * 4 + wave) * 256 + lane * 4) = u[v];
-    }
-    __syncthreads();
-    f32x4 ur[NV][4];
-#pragma unroll
-    for (int v = 0; v < NV; ++v)
-#pragma unroll
-      for (int tb = 0; tb < 4; ++tb) ur[v][tb] = us[v][tb * 64 + lane];
-    const float g = left[c & 1];
+    float* s0 = a.s0 + ((ch * vtiles + vtile) * HS_KB * 64 + lane) * 4;
 #pragma unroll
     for (int m = 0; m < HS_MT; ++m)
+      if (HS_KB % 4 == 0 || wave + 4 * m < HS_KB) *reinterpret_cast<f32x4*>(s0 + (size_t)(wave + 4 * m) * 256) = S[m];
+    if (DELTA) *reinterpret_cast<f32x4*>(a.u + ((ch * vtiles + vtile) * 4 + wave) * 256 + lane * 4) = u;
+    __syncthreads();
+    f32x4 ur[4];
 #pragma unroll
-      for (int v = 0; v < NV; ++v) S[v][m] *= g;
+    for (int tb = 0; tb < 4; ++tb) ur[tb] = us[tb * 64 + lane];
+    const float g = left[c & 1];
+#pragma unroll
+    for (int m = 0; m < HS_MT; ++m) S[m] *= g;
 #pragma unroll
     for (int tb = 0; tb < 4; ++tb) {
       f32x4 kt[HS_MT];
@@ -608,9 +576,7 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
-        for (int m = 0; m < HS_MT; ++m)
-#pragma unroll
-          for (int v = 0; v < NV; ++v) S[v][m] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[m][j], ur[v][tb][j], S[v][m], 0, 0, 0);
+        for (int m = 0; m < HS_MT; ++m) S[m] = __builtin_amdgcn_mfma_f32_16x16x4f32(kt[m][j], ur[tb][j], S[m], 0, 0, 0);
     }
     ask_keys(l, next);
   };
@@ -624,17 +590,13 @@ __global__ __launch_bounds__(256) void hs_carry_kernel(HeadScan a) {
     if (c + 1 >= last) break;
     step(odd, c + 1);
   }
+  if (in) {
 #pragma unroll
-  for (int v = 0; v < NV; ++v) {
-    const int vcol = (vt0 + v) * 16 + col;
-    if (vcol < a.vdim) {
+    for (int m = 0; m < HS_MT; ++m) {
 #pragma unroll
-      for (int m = 0; m < HS_MT; ++m) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int d = (wave + 4 * m) * 16 + 4 * lg + r;
-          if (d < HS_DIM) slot[(size_t)d * a.vdim + vcol] = S[v][m][r];
-        }
+      for (int r = 0; r < 4; ++r) {
+        const int d = (wave + 4 * m) * 16 + 4 * lg + r;
+        if (d < HS_DIM) slot[(size_t)d * a.vdim] = S[m][r];
       }
     }
   }
@@ -830,15 +792,12 @@ extern "C" int qvl_head_scan_chunks(const void* x, long long x_stride, int q_off
   if (delta) { a.u = at; at += c * H * vtiles * 4 * 256; }
   a.s0 = at;
   const bool vec = HS_DIM % 4 == 0 && x_stride % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0 && ((uintptr_t)x & 15) == 0;
-  const int wide = HS_WIDE_CARRY && !delta && vtiles > 1 ? 2 : 1;
-#define CARRY(TX, D, NV)                                                                                          \
-  hipLaunchKernelGGL((hs_carry_kernel<TX, D, NV>), dim3((((vtiles + NV - 1) / NV) * H + 7) / 8 * 8, R), dim3(256), 0, stream, a)
 #define LAUNCH(TX, D, V)                                                                                             \
   {                                                                                                                  \
     hipLaunchKernelGGL((hs_prep_kernel<D>), dim3(chunks, (H + 3) / 4), dim3(256), 0, stream, a);                     \
     hipLaunchKernelGGL((hs_score_kernel<TX, D, V>), dim3(chunks, G), dim3(256), 0, stream, a);                       \
     if (D) hipLaunchKernelGGL((hs_solve_kernel<TX>), dim3(chunks, H), dim3(256), 0, stream, a);                      \
-    if (D || wide == 1) CARRY(TX, D, 1); else CARRY(TX, false, 2);                                             \
+    hipLaunchKernelGGL((hs_carry_kernel<TX, D>), dim3((vtiles * H + 7) / 8 * 8, R), dim3(256), 0, stream, a);          \
     hipLaunchKernelGGL((hs_out_kernel<TX, D, V>), dim3(chunks, H), dim3(256), 0, stream, a);                            \
   }
 #define BY_VEC(TX, D) { if (vec) LAUNCH(TX, D, true) else LAUNCH(TX, D, false) }
@@ -847,7 +806,6 @@ extern "C" int qvl_head_scan_chunks(const void* x, long long x_stride, int q_off
   else return QVL_ERR_DTYPE;
 #undef BY_VEC
 #undef LAUNCH
-#undef CARRY
   return qvl_launch_status();
 #else
   return QVL_ERR_LIMIT;

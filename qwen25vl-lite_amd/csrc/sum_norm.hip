@@ -6,6 +6,8 @@
 // A block owns a row and keeps it in registers between the passes: PER groups of VEC neighbouring values a thread.
 #include "common.h"
 
+#define SUM_NORM_MANY 512       // rows from which blocks are narrow
+
 template <typename T, int VEC> struct Row;
 template <typename T> struct Row<T, 1> {
   static __device__ __forceinline__ void load(float* v, const T* p) { v[0] = ldf<T>(p); }
@@ -154,10 +156,13 @@ extern "C" int qvl_sum_norm(void* h, float alpha, const void* t1, int dtype1, in
   if (dtype1 < 0 || dtype1 > 1 || dtype2 < 0 || dtype2 > 1 || copy_dtype < 0 || copy_dtype > 1) return QVL_ERR_DTYPE;
   const Term a{t1, nslabs1, (long long)N * H, (const float*)gain1, eps1, factor1};
   const Term b{t2, t2 ? nslabs2 : 1, (long long)N * H, (const float*)gain2, eps2, factor2};
-  const bool vec = H % 4 == 0 && on16(h) && on16(t1) && on16(t2) && on16(gain1) && on16(gain2) && on16(w) && on16(bias) && on16(copy);
+  const bool vec = H % 4 == 0 && H <= 4 * 8 * 1024 && on16(h) && on16(t1) && on16(t2) && on16(gain1) && on16(gain2) && on16(w) && on16(bias) && on16(copy);
   const int units = vec ? H / 4 : H;
   if (units > 1024 * 32) return QVL_ERR_LIMIT;
-  const int per = (units + 1023) / 1024;
+  // few rows: a thread has little of a row (short chains of waits); many: narrow blocks, whose barriers hold up fewer waves
+  // (2,048 rows of 3,584, two terms: 23 us with blocks of 512 threads, 34 with 1,024)
+  const int most = N < SUM_NORM_MANY || units > 512 * 8 ? 1024 : (units <= 512 ? 256 : 512);
+  const int per = (units + most - 1) / most;
   const int slots = per <= 1 ? 1 : (per <= 2 ? 2 : (per <= 4 ? 4 : (per <= 8 ? 8 : 32)));
   const int threads = ((units + slots - 1) / slots + 63) / 64 * 64;
 #define LAUNCH(TA, TB, TC, TERMS, VEC, PER)                                                                             \
@@ -169,8 +174,7 @@ extern "C" int qvl_sum_norm(void* h, float alpha, const void* t1, int dtype1, in
     else if (slots == 2) LAUNCH(TA, TB, TC, TERMS, VEC, 2);    \
     else if (slots == 4) LAUNCH(TA, TB, TC, TERMS, VEC, 4);    \
     else if (slots == 8) LAUNCH(TA, TB, TC, TERMS, VEC, 8);    \
-    else if (VEC == 1) LAUNCH(TA, TB, TC, TERMS, 1, 32);       \
-    else return QVL_ERR_LIMIT;                                 \
+    else LAUNCH(TA, TB, TC, TERMS, 1, 32);                     \
   }
 #define BY_VEC(TA, TB, TC, TERMS) { if (vec) BY_PER(TA, TB, TC, TERMS, 4) else BY_PER(TA, TB, TC, TERMS, 1) }
 #define BY_TERMS(TC)                                                              \

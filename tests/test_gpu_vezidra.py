@@ -181,6 +181,24 @@ def test_sum_and_norm_in_one_pass(width, kinds, gains, norm):
         assert got is None if copy is None else torch.equal(got, hd.to(copy))
 
 
+@pytest.mark.parametrize("width", [6, 300, 3584, 9001, 20000])
+def test_sum_and_norm_of_many_rows(width):
+    """Narrow blocks from some hundred rows on: the same rows as among few."""
+    from qwen25vl_lite_amd.ops.sum_norm import sum_norm_
+    from qwen25vl_lite_amd.parts import SumTerm
+    torch.manual_seed(width)
+    n = 600
+    h, y, z = torch.randn(n, width), torch.randn(n, width).to(torch.bfloat16), torch.randn(n, width)
+    w, b, gain = 1 + 0.3 * torch.randn(width), torch.randn(width), 1 + 0.3 * torch.randn(width)
+    want = plain.layer_norm(0.9 * h.double() + 0.5 * plain.unit_rms(y.double(), 1e-5) * gain.double() - 2.0 * z.double(),
+                            w.double(), b.double(), 1e-5)
+    for rows in (slice(0, n), slice(0, 4)):
+        hd = h[rows].contiguous().cuda()
+        terms = [SumTerm(y[rows].contiguous().cuda(), 0.5, gain.cuda(), 1e-5), SumTerm(z[rows].contiguous().cuda(), -2.0)]
+        copy = sum_norm_(hd, 0.9, terms, w.cuda(), b.cuda(), 1e-5, torch.bfloat16)
+        assert torch.allclose(hd.double().cpu(), want[rows], atol=3e-5) and torch.equal(copy, hd.to(torch.bfloat16))
+
+
 @pytest.mark.parametrize("width", [7, 72, 1100, 4400])
 def test_layer_norm_with_a_bias_on_chosen_rows(width):
     from qwen25vl_lite_amd.ops.rownorm import layer_norm
